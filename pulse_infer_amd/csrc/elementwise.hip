@@ -344,7 +344,8 @@ extern "C" int pulse_swiglu(const void* gu, void* out, int dtype, int tokens, in
 // comes from the host in float64.
 // (reference angle: src/ops/kernels/cuda/rope_kernel.cu:119-123, float32 throughout)
 __global__ void rope_table_kernel(const int* __restrict__ positions, const double* __restrict__ inv_freq,
-                                  float* __restrict__ cos_out, float* __restrict__ sin_out, int half, int64_t total) {
+                                  float* __restrict__ cos_out, float* __restrict__ sin_out, int half, int64_t total,
+                                  double magnitude) {
     const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const int64_t t = idx / half;
@@ -352,18 +353,18 @@ __global__ void rope_table_kernel(const int* __restrict__ positions, const doubl
     const double angle = static_cast<double>(positions[t]) * inv_freq[i];
     double s, c;
     sincos(angle, &s, &c);
-    cos_out[idx] = static_cast<float>(c);
-    sin_out[idx] = static_cast<float>(s);
+    cos_out[idx] = static_cast<float>(c * magnitude);
+    sin_out[idx] = static_cast<float>(s * magnitude);
 }
 
 extern "C" int pulse_rope_table(const int* positions, const double* inv_freq, float* cos_out, float* sin_out,
-                                int tokens, int half, hipStream_t stream) {
+                                int tokens, int half, double magnitude, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && half > 0 && positions && inv_freq && cos_out && sin_out, "rope_table: bad arguments");
     const int64_t total = static_cast<int64_t>(tokens) * half;
     if (total == 0) return 0;
     const int64_t blocks = (total + 255) / 256;
     hipLaunchKernelGGL(rope_table_kernel, dim3(static_cast<unsigned>(blocks)), dim3(256), 0, stream, positions,
-                       inv_freq, cos_out, sin_out, half, total);
+                       inv_freq, cos_out, sin_out, half, total, magnitude);
     PULSE_LAUNCH_CHECK("rope_table");
     return 0;
 }

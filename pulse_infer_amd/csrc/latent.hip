@@ -7,6 +7,8 @@
 // [c | turned part], its "value" is c, and head h's result W_uv,h (sum_j a_h(j) c_j) is expanded afterwards.
 //
 // pulse_latent_rows:   c and the turned key part into the pages; the queries' turned parts into their places.
+// pulse_rms_rows:      some columns of every row divided by their root mean square, times a weight (a latent that queries
+//                      come from)
 // pulse_latent_absorb: q_abs[t, h, :] = W_uk,h^T q_plain[t, h]        (float32 sums, one rounding)
 // pulse_latent_expand: y[t, h, :] = (W_uv,h o[t, h, :rank]) * sigmoid(gate[t, h, :])
 // pulse_heads_product: both of these products for bfloat16 weights on the matrix cores: y[t, h, m] = sum_k
@@ -19,8 +21,8 @@ namespace {
 
 struct LatentArgs {
     int heads, d, rot, rank, stored;   // stored: channels of a stored key / value row (>= rank + rot)
-    int64_t x_stride, q_stride;
-    int q0, c0;                        // first columns of the queries and of the down projection in a row of x
+    int64_t x_stride, down_stride, q_stride;
+    int q0, c0;                        // first columns of the queries in a row of x and of the down projection in its
     int page_size, num_pages, bt_width;
     int pairing, write;
     float eps;
@@ -28,7 +30,8 @@ struct LatentArgs {
 
 // One workgroup a token.
 template <typename TX, typename TW, typename TC>
-__global__ void latent_rows_kernel(const TX* __restrict__ x, TX* __restrict__ q, const TW* __restrict__ w,
+__global__ void latent_rows_kernel(const TX* __restrict__ x, const TX* __restrict__ down_x, TX* __restrict__ q,
+                                   const TW* __restrict__ w,
                                    const float* __restrict__ cos_t, const float* __restrict__ sin_t,
                                    TC* __restrict__ kcache, TC* __restrict__ vcache, const int* __restrict__ positions,
                                    const int* __restrict__ token_entry, const int* __restrict__ block_table, LatentArgs a) {
@@ -59,7 +62,7 @@ __global__ void latent_rows_kernel(const TX* __restrict__ x, TX* __restrict__ q,
         qrow[static_cast<int64_t>(h) * a.stored + width + e] = from_f32<TX>(0.f);
     }
     if (!a.write) return;
-    const TX* down = row + a.c0;
+    const TX* down = down_x + static_cast<int64_t>(t) * a.down_stride + a.c0;
     float ss = 0.f;
     for (int i = threadIdx.x; i < a.rank; i += blockDim.x) { const float v = to_f32<TX>(down[i]); ss = fmaf(v, v, ss); }
     ss = block_sum(ss, scratch);
@@ -78,6 +81,19 @@ __global__ void latent_rows_kernel(const TX* __restrict__ x, TX* __restrict__ q,
         krow[i] = from_f32<TC>(k);
         vrow[static_cast<int64_t>(i) * a.page_size] = from_f32<TC>(v);
     }
+}
+
+// out[t, i] = x[t, c0 + i] / sqrt(mean over the n columns of x^2 + eps) * w[i]; one workgroup a row.
+template <typename TX, typename TW>
+__global__ void rms_rows_kernel(const TX* __restrict__ x, int64_t x_stride, int c0, const TW* __restrict__ w,
+                                TX* __restrict__ out, int64_t o_stride, int n, float eps) {
+    __shared__ float scratch[16];
+    const TX* row = x + static_cast<int64_t>(blockIdx.x) * x_stride + c0;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < n; i += blockDim.x) { const float v = to_f32<TX>(row[i]); ss = fmaf(v, v, ss); }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(n) + eps);
+    TX* dst = out + static_cast<int64_t>(blockIdx.x) * o_stride;
+    for (int i = threadIdx.x; i < n; i += blockDim.x) dst[i] = from_f32<TX>(to_f32<TX>(row[i]) * inv * to_f32<TW>(w[i]));
 }
 
 // q_abs[t, h, r] = sum_e q[t, h, e] * W_uk[h * d + e, r]; one workgroup a (token, head), a thread a latent channel.
@@ -102,7 +118,7 @@ __global__ void latent_absorb_kernel(const TX* __restrict__ x, int64_t x_stride,
 template <typename TO, typename TX, typename TW>
 __global__ void latent_expand_kernel(const TO* __restrict__ o, int64_t o_stride, int stored, const TW* __restrict__ w,
                                      const TX* __restrict__ gate, int64_t gate_stride, TX* __restrict__ y,
-                                     int64_t y_stride, int dv, int rank, float scale) {
+                                     int64_t y_stride, int dv, int rank, float scale, int gate_heads) {
     extern __shared__ float o_s[];
     const int t = blockIdx.x, h = blockIdx.y;
     const TO* src = o + static_cast<int64_t>(t) * o_stride + static_cast<int64_t>(h) * stored;
@@ -116,7 +132,7 @@ __global__ void latent_expand_kernel(const TO* __restrict__ o, int64_t o_stride,
         sum = wave_sum(sum);
         if (lane == 0) {
             float v = sum * scale;
-            if (gate) v *= 1.0f / (1.0f + expf(-to_f32<TX>(gate[static_cast<int64_t>(t) * gate_stride + static_cast<int64_t>(h) * dv + e])));
+            if (gate) v *= 1.0f / (1.0f + expf(-to_f32<TX>(gate[static_cast<int64_t>(t) * gate_stride + (gate_heads ? h : static_cast<int64_t>(h) * dv + e)])));
             y[static_cast<int64_t>(t) * y_stride + static_cast<int64_t>(h) * dv + e] = from_f32<TX>(v);
         }
     }
@@ -144,7 +160,7 @@ template <typename TX>
 __global__ __launch_bounds__(256) void heads_product_kernel(const TX* __restrict__ x, int64_t x_stride, int x_head,
                                                             const bf16_t* __restrict__ w, const bf16_t* __restrict__ gate,
                                                             int64_t gate_stride, bf16_t* __restrict__ y, int64_t y_stride,
-                                                            int y_head, int tokens, int m_out, int k_in, float scale) {
+                                                            int y_head, int tokens, int m_out, int k_in, float scale, int gate_heads) {
     const int t0 = blockIdx.x * 16, h = blockIdx.y;
     const int lane = threadIdx.x % PULSE_WAVE, wave = threadIdx.x / PULSE_WAVE;
     const int r = lane % 16, g = lane / 16;
@@ -166,12 +182,12 @@ __global__ __launch_bounds__(256) void heads_product_kernel(const TX* __restrict
         if (t0 + r < tokens) {
             const int c0 = m0 + 4 * g;
             bf16_t* dst = y + static_cast<int64_t>(t0 + r) * y_stride + static_cast<int64_t>(h) * y_head + c0;
-            const bf16_t* gr = gate ? gate + static_cast<int64_t>(t0 + r) * gate_stride + static_cast<int64_t>(h) * m_out + c0 : nullptr;
+            const bf16_t* gr = gate ? gate + static_cast<int64_t>(t0 + r) * gate_stride + (gate_heads ? h : static_cast<int64_t>(h) * m_out + c0) : nullptr;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 if (c0 + i < m_out) {
                     float v = acc[i] * scale;
-                    if (gr) v *= 1.0f / (1.0f + expf(-bf16_to_f32(gr[i])));
+                    if (gr) v *= 1.0f / (1.0f + expf(-bf16_to_f32(gr[gate_heads ? 0 : i])));
                     dst[i] = f32_to_bf16(v);
                 }
             }
@@ -181,33 +197,49 @@ __global__ __launch_bounds__(256) void heads_product_kernel(const TX* __restrict
 
 }  // namespace
 
-// x [tokens, x_stride]: the projection output; queries from column q0 (heads x (d + rot), the turned part last), the
-// down projection from column c0 (rank + rot).  q [tokens, q_stride] receives, for head h at h * stored, the turned
+// x [tokens, x_stride]: queries from column q0 (heads x (d + rot), the turned part last); down_x [tokens, down_stride]:
+// the down projection from column c0 (rank + rot; the two may be one matrix; without `write` down_x is not read).  q [tokens, q_stride] receives, for head h at h * stored, the turned
 // part at rank .. rank + rot and zeros behind it (the first rank channels are pulse_latent_absorb's).  With `write`
 // the token's c and turned key part go to kcache [pages, 1, page, stored] and c to vcache [pages, 1, stored, page].
-extern "C" int pulse_latent_rows(const void* x, int64_t x_stride, int x_dtype, int q0, int c0, void* q, int64_t q_stride,
+extern "C" int pulse_latent_rows(const void* x, int64_t x_stride, int x_dtype, int q0, const void* down_x,
+                                 int64_t down_stride, int c0, void* q, int64_t q_stride,
                                  const void* norm_w, int w_dtype, const float* cos_t, const float* sin_t, int pairing,
                                  void* kcache, void* vcache, int c_dtype, const int* positions, const int* token_entry,
                                  const int* block_table, int bt_width, int tokens, int heads, int d, int rot, int rank,
                                  int stored, int page_size, int num_pages, float eps, int write, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && heads > 0 && d >= 0 && rank > 0 && rot > 0 && rot % 2 == 0, "latent_rows: bad sizes");
     PULSE_REQUIRE(stored >= rank + rot && q_stride >= static_cast<int64_t>(heads) * stored, "latent_rows: stored rows too narrow");
-    PULSE_REQUIRE(x && q && norm_w && cos_t && sin_t && kcache && vcache && positions && token_entry && block_table,
-                  "latent_rows: null pointer");
+    PULSE_REQUIRE(x && q && cos_t && sin_t && positions && token_entry && (!write || (down_x && norm_w && kcache && vcache &&
+                  block_table)), "latent_rows: null pointer");
     PULSE_REQUIRE(pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype) && pulse_dtype_ok(c_dtype), "latent_rows: bad dtype tag");
     PULSE_REQUIRE(q0 >= 0 && c0 >= 0 && x_stride >= static_cast<int64_t>(q0) + static_cast<int64_t>(heads) * (d + rot) &&
-                  x_stride >= static_cast<int64_t>(c0) + rank + rot, "latent_rows: the rows are too short");
-    PULSE_REQUIRE(page_size > 0 && num_pages > 0 && bt_width > 0 && (pairing == 0 || pairing == 1), "latent_rows: bad cache geometry");
+                  (!write || down_stride >= static_cast<int64_t>(c0) + rank + rot), "latent_rows: the rows are too short");
+    PULSE_REQUIRE((!write || (page_size > 0 && num_pages > 0 && bt_width > 0)) && (pairing == 0 || pairing == 1),
+                  "latent_rows: bad cache geometry");
     if (tokens == 0) return 0;
     LatentArgs a;
-    a.heads = heads; a.d = d; a.rot = rot; a.rank = rank; a.stored = stored; a.x_stride = x_stride; a.q_stride = q_stride;
+    a.heads = heads; a.d = d; a.rot = rot; a.rank = rank; a.stored = stored; a.x_stride = x_stride;
+    a.down_stride = down_stride; a.q_stride = q_stride;
     a.q0 = q0; a.c0 = c0; a.page_size = page_size; a.num_pages = num_pages; a.bt_width = bt_width; a.pairing = pairing;
     a.write = write; a.eps = eps;
     PULSE_DISPATCH_DTYPE(x_dtype, TX, PULSE_DISPATCH_DTYPE(w_dtype, TW, PULSE_DISPATCH_DTYPE(c_dtype, TC,
         hipLaunchKernelGGL((latent_rows_kernel<TX, TW, TC>), dim3(tokens), dim3(256), 0, stream, static_cast<const TX*>(x),
-                           static_cast<TX*>(q), static_cast<const TW*>(norm_w), cos_t, sin_t, static_cast<TC*>(kcache),
+                           static_cast<const TX*>(down_x), static_cast<TX*>(q), static_cast<const TW*>(norm_w), cos_t, sin_t, static_cast<TC*>(kcache),
                            static_cast<TC*>(vcache), positions, token_entry, block_table, a))));
     PULSE_LAUNCH_CHECK("latent_rows");
+    return 0;
+}
+
+extern "C" int pulse_rms_rows(const void* x, int64_t x_stride, int x_dtype, int c0, const void* w, int w_dtype, void* out,
+                              int64_t o_stride, int tokens, int n, float eps, hipStream_t stream) {
+    PULSE_REQUIRE(tokens >= 0 && n > 0 && c0 >= 0 && x && w && out && pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype),
+                  "rms_rows: bad arguments");
+    PULSE_REQUIRE(x_stride >= static_cast<int64_t>(c0) + n && o_stride >= n, "rms_rows: the rows are too short");
+    if (tokens == 0) return 0;
+    PULSE_DISPATCH_DTYPE(x_dtype, TX, PULSE_DISPATCH_DTYPE(w_dtype, TW,
+        hipLaunchKernelGGL((rms_rows_kernel<TX, TW>), dim3(tokens), dim3(256), 0, stream, static_cast<const TX*>(x), x_stride,
+                           c0, static_cast<const TW*>(w), static_cast<TX*>(out), o_stride, n, eps)));
+    PULSE_LAUNCH_CHECK("rms_rows");
     return 0;
 }
 
@@ -230,37 +262,38 @@ extern "C" int pulse_latent_absorb(const void* x, int64_t x_stride, int x_dtype,
 }
 
 // o [tokens, o_stride] (float32 or the activations' type): head h's weighted latent row at h * stored; w_uv
-// [heads * dv, rank]; gate [tokens, gate_stride] holds heads * dv logits a token (null: no gate).
+// [heads * dv, rank]; gate [tokens, gate_stride] holds heads * dv logits a token, with gate_heads one a head (null: no
+// gate).
 extern "C" int pulse_latent_expand(const void* o, int64_t o_stride, int o_dtype, int stored, const void* w_uv, int w_dtype,
                                    const void* gate, int64_t gate_stride, void* y, int64_t y_stride, int x_dtype,
-                                   int tokens, int heads, int dv, int rank, float scale, hipStream_t stream) {
+                                   int tokens, int heads, int dv, int rank, float scale, int gate_heads, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && heads > 0 && dv > 0 && rank > 0 && stored >= rank, "latent_expand: bad sizes");
     PULSE_REQUIRE(heads < 65536 && o && w_uv && y && pulse_dtype_ok(o_dtype) && pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype),
                   "latent_expand: bad arguments");
     PULSE_REQUIRE(o_stride >= static_cast<int64_t>(heads) * stored && y_stride >= static_cast<int64_t>(heads) * dv &&
-                  (!gate || gate_stride >= static_cast<int64_t>(heads) * dv), "latent_expand: the rows are too short");
+                  (!gate || gate_stride >= static_cast<int64_t>(heads) * (gate_heads ? 1 : dv)), "latent_expand: the rows are too short");
     PULSE_REQUIRE(rank * sizeof(float) <= 60 * 1024, "latent_expand: a latent row of %d values does not fit", rank);
     if (tokens == 0) return 0;
     PULSE_DISPATCH_DTYPE(o_dtype, TO, PULSE_DISPATCH_DTYPE(x_dtype, TX, PULSE_DISPATCH_DTYPE(w_dtype, TW,
         hipLaunchKernelGGL((latent_expand_kernel<TO, TX, TW>), dim3(tokens, heads), dim3(256), sizeof(float) * rank, stream,
                            static_cast<const TO*>(o), o_stride, stored, static_cast<const TW*>(w_uv),
-                           static_cast<const TX*>(gate), gate_stride, static_cast<TX*>(y), y_stride, dv, rank, scale))));
+                           static_cast<const TX*>(gate), gate_stride, static_cast<TX*>(y), y_stride, dv, rank, scale, gate_heads))));
     PULSE_LAUNCH_CHECK("latent_expand");
     return 0;
 }
 
 // y[t, h * y_head + m] = scale * (sum_k w[h, m, k] * x[t, h * x_head + k]) * sigmoid(gate[t, h * m_out + m]) for bfloat16
 // w [heads, m_out, k_in] and y, x bfloat16 or float32 (rounded to bfloat16 as it is read); k_in a multiple of 8, rows
-// of x and w 16-byte aligned.  gate may be null.
+// of x and w 16-byte aligned.  gate may be null; with gate_heads it holds one logit a head, gate[t, h].
 extern "C" int pulse_heads_product(const void* x, int64_t x_stride, int x_head, int x_dtype, const void* w, const void* gate,
                                    int64_t gate_stride, void* y, int64_t y_stride, int y_head, int tokens, int heads,
-                                   int m_out, int k_in, float scale, hipStream_t stream) {
+                                   int m_out, int k_in, float scale, int gate_heads, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && heads > 0 && heads < 65536 && m_out > 0 && k_in > 0 && k_in % 8 == 0, "heads_product: bad sizes");
     PULSE_REQUIRE(x && w && y && pulse_dtype_ok(x_dtype), "heads_product: bad arguments");
     const int xb = x_dtype == PULSE_F32 ? 4 : 2;
     PULSE_REQUIRE(x_head >= k_in && x_stride >= static_cast<int64_t>(heads - 1) * x_head + k_in &&
                   y_head >= m_out && y_stride >= static_cast<int64_t>(heads - 1) * y_head + m_out &&
-                  (!gate || gate_stride >= static_cast<int64_t>(heads) * m_out), "heads_product: the rows are too short");
+                  (!gate || gate_stride >= static_cast<int64_t>(heads) * (gate_heads ? 1 : m_out)), "heads_product: the rows are too short");
     PULSE_REQUIRE(reinterpret_cast<uintptr_t>(x) % 16 == 0 && (x_stride * xb) % 16 == 0 && (static_cast<int64_t>(x_head) * xb) % 16 == 0 &&
                   reinterpret_cast<uintptr_t>(w) % 16 == 0, "heads_product: operands must be 16-byte aligned");
     if (tokens == 0) return 0;
@@ -268,7 +301,7 @@ extern "C" int pulse_heads_product(const void* x, int64_t x_stride, int x_head, 
     PULSE_DISPATCH_DTYPE(x_dtype, TX,
         hipLaunchKernelGGL(heads_product_kernel<TX>, grid, dim3(256), 0, stream, static_cast<const TX*>(x), x_stride, x_head,
                            static_cast<const bf16_t*>(w), static_cast<const bf16_t*>(gate), gate_stride,
-                           static_cast<bf16_t*>(y), y_stride, y_head, tokens, m_out, k_in, scale));
+                           static_cast<bf16_t*>(y), y_stride, y_head, tokens, m_out, k_in, scale, gate_heads));
     PULSE_LAUNCH_CHECK("heads_product");
     return 0;
 }

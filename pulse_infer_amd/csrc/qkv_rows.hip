@@ -6,8 +6,8 @@
 //   q += bq, k += bk, v += bv                                  (biases optional)
 //   q <- q / sqrt(mean over all nq*d values of q^2 + eps) * wq  (one norm over the row; wq [nq*d]; optional)
 //   k likewise with wk [nkv*d]
-//   or (norm 2) every head of q and of k divided by the root mean square of its own d values, without weights;
-//   a rotation keeps a head's sum of squares, so this is the same before or after it
+//   or (norm 2) every head of q and of k divided by the root mean square of its own d values (a rotation keeps a
+//   head's sum of squares, so this is the same before or after it), optionally times weights [d] shared by the heads
 //   q, k <- rotated at the token's position on the first rotary_dim channels of every head
 //           (pairing 0: channels 2i, 2i+1; pairing 1: channels i, i + rotary_dim/2)
 //   v <- v * value_scale
@@ -26,7 +26,7 @@ namespace {
 struct PrepArgs {
     int nq, nkv, d, dv, D;
     int64_t x_stride, q_stride;
-    int norm;           // 0: none, 1: over the whole projection, 2: every head by itself, no weights
+    int norm;           // 0: none, 1: over the whole projection, 2: every head by itself (weights, if any, of d values)
     float eps;
     int rotary_dim, pairing;
     int page_size, num_pages, bt_width;
@@ -93,7 +93,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(const TX* __restrict__ x,
         const int at = base + hd * a.d + c;
         if (a.norm == 2) inv = inv_s[base / a.d + hd];
         float u = row_s[at] * inv;
-        if (w) u *= to_f32<TW>(w[at - base]);
+        if (w) u *= to_f32<TW>(w[a.norm == 2 ? c : at - base]);
         if (cs && c < a.rotary_dim) {
             int partner, i;
             bool first;
@@ -101,7 +101,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(const TX* __restrict__ x,
             else { i = c % half; first = c < half; partner = first ? c + half : c - half; }
             const int pat = base + hd * a.d + partner;
             float p = row_s[pat] * inv;
-            if (w) p *= to_f32<TW>(w[pat - base]);
+            if (w) p *= to_f32<TW>(w[a.norm == 2 ? partner : pat - base]);
             // (u, p) -> first: u cos - p sin; second: u cos + p sin   (u the element itself, p its partner)
             u = first ? u * cs[i] - p * sn[i] : u * cs[i] + p * sn[i];
         }
@@ -174,7 +174,6 @@ extern "C" int pulse_qkv_rows(const void* x, int x_dtype, int64_t x_stride, cons
     PULSE_REQUIRE(D >= d && D >= dv, "qkv_rows: the stored head width %d is below %d or %d", D, d, dv);
     PULSE_REQUIRE(pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype) && pulse_dtype_ok(c_dtype), "qkv_rows: bad dtype tag");
     PULSE_REQUIRE(norm == 0 || norm == 1 || norm == 2, "qkv_rows: unknown norm %d", norm);
-    PULSE_REQUIRE(norm != 2 || (!wq && !wk), "qkv_rows: the norm of every head by itself has no weights");
     PULSE_REQUIRE(x && q_out && positions && token_entry, "qkv_rows: null pointer");
     PULSE_REQUIRE(!write_kv || (kcache && vcache && block_table && page_size > 0 && num_pages > 0 && bt_width > 0),
                   "qkv_rows: the cache is missing");

@@ -43,7 +43,8 @@ __global__ void rotate_qk_rows_kernel(const TX* __restrict__ x, int64_t x_stride
 template <typename TX, typename TW>
 __global__ void group_norm_gate_kernel(const float* __restrict__ o, int64_t o_stride, const TW* __restrict__ w,
                                        const TX* __restrict__ gate, int64_t gate_stride, TX* __restrict__ y,
-                                       int64_t y_stride, int groups, int n, float eps, float scale, int gate_act) {
+                                       int64_t y_stride, int groups, int n, float eps, float scale, int gate_act,
+                                       int w_group) {
     // one wavefront a (token, group)
     const int t = blockIdx.x, g = blockIdx.y * (blockDim.x / PULSE_WAVE) + threadIdx.x / PULSE_WAVE;
     if (g >= groups) return;
@@ -57,7 +58,7 @@ __global__ void group_norm_gate_kernel(const float* __restrict__ o, int64_t o_st
     TX* dst = y + static_cast<int64_t>(t) * y_stride + static_cast<int64_t>(g) * n;
     for (int i = lane; i < n; i += PULSE_WAVE) {
         float v = row[i] * inv;
-        if (w) v *= to_f32<TW>(w[static_cast<int64_t>(g) * n + i]);
+        if (w) v *= to_f32<TW>(w[static_cast<int64_t>(g) * w_group + i]);
         if (gr) {
             const float z = to_f32<TX>(gr[i]);
             const float sg = 1.0f / (1.0f + expf(-z));
@@ -90,10 +91,10 @@ extern "C" int pulse_rotate_qk_rows(const void* x, int64_t x_stride, int x_dtype
 }
 
 // y[t, g n + i] = scale * o[t, g n + i] / sqrt(mean_i(o[t, g n + .]^2) + eps) * w[g n + i] * act(gate[t, g n + i]);
-// w and gate may be null; gate_act 0: sigmoid, 1: silu.
+// w and gate may be null; with shared_w all groups have the weights w[i]; gate_act 0: sigmoid, 1: silu.
 extern "C" int pulse_group_norm_gate(const float* o, int64_t o_stride, const void* w, int w_dtype, const void* gate,
                                      int64_t gate_stride, void* y, int64_t y_stride, int x_dtype, int tokens, int groups,
-                                     int n, float eps, float scale, int gate_act, hipStream_t stream) {
+                                     int n, float eps, float scale, int gate_act, int shared_w, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && groups > 0 && n > 0 && o && y, "group_norm_gate: bad arguments");
     PULSE_REQUIRE(pulse_dtype_ok(w_dtype) && pulse_dtype_ok(x_dtype) && (gate_act == 0 || gate_act == 1),
                   "group_norm_gate: bad dtype tag or gate");
@@ -106,7 +107,7 @@ extern "C" int pulse_group_norm_gate(const float* o, int64_t o_stride, const voi
     PULSE_DISPATCH_DTYPE(x_dtype, TX, PULSE_DISPATCH_DTYPE(w_dtype, TW,
         hipLaunchKernelGGL((group_norm_gate_kernel<TX, TW>), grid, dim3(waves * PULSE_WAVE), 0, stream, o,
                            o_stride, static_cast<const TW*>(w), static_cast<const TX*>(gate), gate_stride,
-                           static_cast<TX*>(y), y_stride, groups, n, eps, scale, gate_act)));
+                           static_cast<TX*>(y), y_stride, groups, n, eps, scale, gate_act, shared_w ? 0 : n)));
     PULSE_LAUNCH_CHECK("group_norm_gate");
     return 0;
 }

@@ -162,8 +162,9 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor, slab: int = 0, activation: 
          _i32(slab), _i32(GATE_ACTIVATIONS[activation]), _stream())
 
 
-def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, cos_out: torch.Tensor, sin_out: torch.Tensor) -> None:
-    """cos/sin of position * inv_freq, computed in float64 and stored as float32 [T, half]."""
+def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, cos_out: torch.Tensor, sin_out: torch.Tensor,
+               magnitude: float = 1.0) -> None:
+    """magnitude * cos/sin of position * inv_freq, computed in float64 and stored as float32 [T, half]."""
     _gpu("rope_table", positions, inv_freq, cos_out, sin_out)
     tokens, half = positions.numel(), inv_freq.numel()
     _int_vec("rope_table: positions", positions)
@@ -172,7 +173,7 @@ def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, cos_out: torch.T
         _need(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (tokens, half),
               f"rope_table: tables must be float32 [{tokens}, {half}]")
     call("pulse_rope_table", _ptr(positions), _ptr(inv_freq), _ptr(cos_out), _ptr(sin_out), _i32(tokens), _i32(half),
-         _stream())
+         ctypes.c_double(float(magnitude)), _stream())
 
 
 def gather_rows(src: torch.Tensor, rows: torch.Tensor, out: torch.Tensor) -> None:
@@ -665,7 +666,7 @@ GATE_FORMS = {"sigmoid": 0, "silu": 1}
 def group_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], gate: Optional[torch.Tensor], out: torch.Tensor,
                     groups: int, eps: float, scale: float = 1.0, gate_form: str = "sigmoid") -> None:
     """Every one of the ``groups`` equal parts of a row of ``o`` (float32) divided by its own root mean square, times
-    ``weight`` (optional, one a column), times sigmoid(gate) or silu(gate) (optional), times ``scale``; one rounding."""
+    ``weight`` (optional, one a column, or one a column of a part: the parts share it then), times sigmoid(gate) or silu(gate) (optional), times ``scale``; one rounding."""
     _gpu("group_norm_gate", o, weight, gate, out)
     tokens, width = o.shape
     _need(groups > 0 and width % groups == 0, f"group_norm_gate: {width} columns in {groups} groups")
@@ -675,23 +676,29 @@ def group_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], gate: Optio
           f"group_norm_gate: out must be [{tokens}, {width}] with contiguous rows")
     _need(gate is None or (gate.shape == out.shape and gate.stride(1) == 1 and gate.dtype == out.dtype),
           "group_norm_gate: the gate must have out's shape and storage type")
-    _need(weight is None or (weight.numel() == width and weight.is_contiguous()),
-          f"group_norm_gate: weight must hold {width} values")
+    _need(weight is None or (weight.numel() in (width, width // groups) and weight.is_contiguous()),
+          f"group_norm_gate: weight must hold {width} or {width // groups} values")
     row = lambda t: t.stride(0) if tokens > 1 else max(width, t.shape[1])
     call("pulse_group_norm_gate", _ptr(o), _i64(row(o)), _ptr(weight),
          _i32(_tag(weight, "group_norm_gate") if weight is not None else 0), _ptr(gate),
          _i64(row(gate) if gate is not None else 0), _ptr(out), _i64(row(out)), _i32(_tag(out, "group_norm_gate")),
-         _i32(tokens), _i32(groups), _i32(width // groups), _f32(eps), _f32(scale), _i32(GATE_FORMS[gate_form]), _stream())
+         _i32(tokens), _i32(groups), _i32(width // groups), _f32(eps), _f32(scale), _i32(GATE_FORMS[gate_form]),
+         _i32(1 if weight is not None and weight.numel() != width else 0), _stream())
 
 
-def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight: torch.Tensor, cos: torch.Tensor,
+def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight: Optional[torch.Tensor], cos: torch.Tensor,
                 sin: torch.Tensor, pairing: int, kcache: torch.Tensor, vcache: torch.Tensor, positions: torch.Tensor,
                 token_entry: torch.Tensor, block_table: torch.Tensor, heads: int, d: int, rot: int, rank: int,
-                stored: int, eps: float, write: bool = True) -> None:
+                stored: int, eps: float, write: bool = True, down: Optional[torch.Tensor] = None) -> None:
     """Latent attention's preparation: the normed latent row and the turned key part of every token into the pages
     (keys [pages, 1, page, stored] = [c | turned | 0], values [pages, 1, stored, page] = [c | 0]) and the queries'
-    turned parts into ``q`` [T, heads * stored] at rank .. rank + rot of every head (zeros behind)."""
-    _gpu("latent_rows", x, q, norm_weight, cos, sin, kcache, vcache, positions, token_entry, block_table)
+    turned parts into ``q`` [T, heads * stored] at rank .. rank + rot of every head (zeros behind).  The queries are
+    columns q0 .. of ``x``, the down projection columns c0 .. of ``down`` (None: of ``x`` too); without ``write`` only the
+    queries are prepared."""
+    down = x if down is None else down
+    _need(not write or (norm_weight is not None and down.dtype == x.dtype and down.dim() == 2 and down.stride(1) == 1
+                        and down.shape[0] == x.shape[0]), "latent_rows: the down projection must be a matrix of x's type and rows")
+    _gpu("latent_rows", x, down, q, norm_weight, cos, sin, kcache, vcache, positions, token_entry, block_table)
     tokens = x.shape[0]
     _need(x.dim() == 2 and x.stride(1) == 1 and q.dim() == 2 and q.stride(1) == 1 and q.dtype == x.dtype
           and q.shape[0] == tokens and q.shape[1] >= heads * stored, "latent_rows: x and q must be matrices of one type")
@@ -700,13 +707,14 @@ def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight:
     _int_vec("latent_rows: token_entry", token_entry, tokens)
     _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.is_contiguous(),
           "latent_rows: block_table must be contiguous int32 [entries, width]")
-    _need(norm_weight.numel() == rank and norm_weight.is_contiguous(), f"latent_rows: the norm's weight must hold {rank} values")
+    _need(norm_weight is None or (norm_weight.numel() == rank and norm_weight.is_contiguous()), f"latent_rows: the norm's weight must hold {rank} values")
     for t in (cos, sin):
         _need(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (tokens, rot // 2),
               f"latent_rows: the tables must be contiguous float32 [{tokens}, {rot // 2}]")
     call("pulse_latent_rows", _ptr(x), _i64(x.stride(0) if tokens > 1 else x.shape[1]), _i32(_tag(x, "latent_rows")),
-         _i32(q0), _i32(c0), _ptr(q), _i64(q.stride(0) if tokens > 1 else q.shape[1]), _ptr(norm_weight),
-         _i32(_tag(norm_weight, "latent_rows")), _ptr(cos), _ptr(sin), _i32(pairing), _ptr(kcache), _ptr(vcache),
+         _i32(q0), _ptr(down), _i64(down.stride(0) if tokens > 1 else down.shape[1]), _i32(c0), _ptr(q),
+         _i64(q.stride(0) if tokens > 1 else q.shape[1]), _ptr(norm_weight),
+         _i32(_tag(norm_weight, "latent_rows") if norm_weight is not None else 0), _ptr(cos), _ptr(sin), _i32(pairing), _ptr(kcache), _ptr(vcache),
          _i32(_tag(kcache, "latent_rows")), _ptr(positions), _ptr(token_entry), _ptr(block_table),
          _i32(block_table.shape[1]), _i32(tokens), _i32(heads), _i32(d), _i32(rot), _i32(rank), _i32(stored),
          _i32(page_size), _i32(pages), _f32(eps), _i32(1 if write else 0), _stream())
@@ -727,10 +735,23 @@ def latent_absorb(x: torch.Tensor, q0: int, q_head: int, w_uk: torch.Tensor, q: 
          _stream())
 
 
+def rms_rows(x: torch.Tensor, c0: int, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
+    """out[t] = x[t, c0:c0 + n] / sqrt(mean of their squares + eps) * weight, n values; rows of x and out may be strided."""
+    _gpu("rms_rows", x, weight, out)
+    tokens, n = out.shape
+    _need(x.dim() == 2 and x.stride(1) == 1 and out.stride(1) == 1 and x.dtype == out.dtype and x.shape[0] == tokens
+          and x.shape[1] >= c0 + n, "rms_rows: x and out must be matrices of one type with contiguous rows")
+    _need(weight.numel() == n and weight.is_contiguous(), f"rms_rows: the weight must hold {n} values")
+    row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
+    call("pulse_rms_rows", _ptr(x), _i64(row(x)), _i32(_tag(x, "rms_rows")), _i32(c0), _ptr(weight),
+         _i32(_tag(weight, "rms_rows")), _ptr(out), _i64(row(out)), _i32(tokens), _i32(n), _f32(eps), _stream())
+
+
 def latent_expand(o: torch.Tensor, stored: int, w_uv: torch.Tensor, gate: Optional[torch.Tensor], out: torch.Tensor,
-                  heads: int, dv: int, rank: int, scale: float = 1.0) -> None:
+                  heads: int, dv: int, rank: int, scale: float = 1.0, gate_heads: bool = False) -> None:
     """out[t, h * dv + e] = scale * (sum_r w_uv[h * dv + e, r] * o[t, h * stored + r]) * sigmoid(gate[t, h * dv + e]):
-    the heads' weighted latent rows expanded to their values, gated channel by channel; one rounding."""
+    the heads' weighted latent rows expanded to their values, gated channel by channel (``gate_heads``: by the one number
+    gate[t, h]); one rounding."""
     _gpu("latent_expand", o, w_uv, gate, out)
     tokens = o.shape[0]
     _need(o.dim() == 2 and o.stride(1) == 1 and o.shape[1] >= heads * stored, "latent_expand: o too narrow")
@@ -738,12 +759,12 @@ def latent_expand(o: torch.Tensor, stored: int, w_uv: torch.Tensor, gate: Option
     _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == tokens and out.shape[1] >= heads * dv,
           "latent_expand: out too narrow")
     _need(gate is None or (gate.dtype == out.dtype and gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] == tokens
-                           and gate.shape[1] >= heads * dv), "latent_expand: the gate must be of out's type and width")
+                           and gate.shape[1] >= heads * (1 if gate_heads else dv)), "latent_expand: the gate must be of out's type and width")
     row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
     call("pulse_latent_expand", _ptr(o), _i64(row(o)), _i32(_tag(o, "latent_expand")), _i32(stored), _ptr(w_uv),
          _i32(_tag(w_uv, "latent_expand")), _ptr(gate), _i64(row(gate) if gate is not None else 0), _ptr(out),
          _i64(row(out)), _i32(_tag(out, "latent_expand")), _i32(tokens), _i32(heads), _i32(dv), _i32(rank), _f32(scale),
-         _stream())
+         _i32(1 if gate_heads else 0), _stream())
 
 
 def heads_product_takes(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, x_head: int) -> bool:
@@ -755,9 +776,10 @@ def heads_product_takes(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, x_h
 
 
 def heads_product(x: torch.Tensor, x_head: int, w: torch.Tensor, gate: Optional[torch.Tensor], out: torch.Tensor,
-                  out_head: int, scale: float = 1.0) -> None:
+                  out_head: int, scale: float = 1.0, gate_heads: bool = False) -> None:
     """out[t, h * out_head + m] = scale * (sum_k w[h, m, k] * x[t, h * x_head + k]) * sigmoid(gate[t, h * M + m]) on
-    the matrix cores: a product a head (w bfloat16 [heads, M, K]; x bfloat16 or float32; gate optional, of out's type)."""
+    the matrix cores: a product a head (w bfloat16 [heads, M, K]; x bfloat16 or float32; gate optional, of
+    out's type, with ``gate_heads`` one number a head)."""
     _gpu("heads_product", x, w, gate, out)
     tokens = x.shape[0]
     heads, m_out, k_in = w.shape
@@ -766,11 +788,11 @@ def heads_product(x: torch.Tensor, x_head: int, w: torch.Tensor, gate: Optional[
     _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == tokens and out.shape[1] >= (heads - 1) * out_head + m_out,
           "heads_product: out too narrow")
     _need(gate is None or (gate.dtype == out.dtype and gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] == tokens
-                           and gate.shape[1] >= heads * m_out), "heads_product: the gate must be of out's type and width")
+                           and gate.shape[1] >= heads * (1 if gate_heads else m_out)), "heads_product: the gate must be of out's type and width")
     row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
     call("pulse_heads_product", _ptr(x), _i64(row(x)), _i32(x_head), _i32(_tag(x, "heads_product")), _ptr(w), _ptr(gate),
          _i64(row(gate) if gate is not None else 0), _ptr(out), _i64(row(out)), _i32(out_head), _i32(tokens), _i32(heads),
-         _i32(m_out), _i32(k_in), _f32(scale), _stream(), label=f"M={m_out} K={k_in}")
+         _i32(m_out), _i32(k_in), _f32(scale), _i32(1 if gate_heads else 0), _stream(), label=f"M={m_out} K={k_in}")
 
 
 def xielu(x: torch.Tensor, out: torch.Tensor, pq: torch.Tensor) -> None:
@@ -962,6 +984,67 @@ def round_rows(x: torch.Tensor, out: torch.Tensor) -> None:
 
 
 # ---------------------------------------------------------------------------
+# A layer with a norm before and after every sublayer
+NORM_KINDS = {"layernorm": 0, "rmsnorm": 1}
+
+
+def sandwich_step(h: torch.Tensor, terms: list, post: Optional[tuple] = None, term_scale: float = 1.0,
+                  term_eps: float = 0.0, norm: Optional[tuple] = None, out: Optional[torch.Tensor] = None,
+                  rows: Optional[torch.Tensor] = None) -> None:
+    """h <- h + post(y), and, with ``norm`` and ``out``, out = norm(h) of all rows or of the gathered ``rows`` (the
+    updated rows are then used but not stored).  ``terms``: [(y, None)] for a result as it is, or one or two (y, weight):
+    y = term_scale * sum of y_i / sqrt(mean(y_i^2) + term_eps) * weight_i.  ``post`` and ``norm`` are (kind, weight, bias or
+    None, eps) with kind "layernorm" or "rmsnorm"; ``post`` None adds y itself."""
+    _need(1 <= len(terms) <= 2 and (len(terms) == 1 or all(w is not None for _, w in terms)),
+          "sandwich_step: one result, or one or two with weights")
+    ys, tws = [y for y, _ in terms], [w for _, w in terms]
+    kinds = [post, norm]
+    weights = [t for t in tws if t is not None] + [t for n in kinds if n is not None for t in n[1:3] if t is not None]
+    _gpu("sandwich_step", h, *ys, *weights, out, rows)
+    _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous(), "sandwich_step: h must be contiguous float32 [T, H]")
+    tokens, hidden = h.shape
+    _need(all(y.shape == h.shape and y.is_contiguous() and y.dtype == ys[0].dtype for y in ys),
+          f"sandwich_step: results must be contiguous [{tokens}, {hidden}] of one storage type")
+    _need(all(w.numel() == hidden and w.is_contiguous() and w.dtype == weights[0].dtype for w in weights),
+          f"sandwich_step: weights must hold {hidden} values of one storage type")
+    _need(all(n is None or n[0] in NORM_KINDS for n in kinds), f"sandwich_step: a norm is one of {sorted(NORM_KINDS)}")
+    _need((norm is None) == (out is None), "sandwich_step: the next norm comes with its output")
+    n_rows = tokens
+    if rows is not None:
+        _int_vec("sandwich_step: rows", rows)
+        n_rows = rows.numel()
+    if out is not None:
+        _need(out.is_contiguous() and tuple(out.shape) == (n_rows, hidden), f"sandwich_step: out must be [{n_rows}, {hidden}]")
+    part = lambda n, i: n[i] if n is not None else None
+    call("pulse_sandwich_step", _ptr(h), _i32(tokens), _i32(hidden), _ptr(ys[0]), _ptr(ys[1] if len(ys) > 1 else None),
+         _i32(_tag(ys[0], "sandwich_step")), _i32(len(terms) if tws[0] is not None else 0), _ptr(tws[0]),
+         _ptr(tws[1] if len(tws) > 1 else None), _f32(term_scale), _f32(term_eps),
+         _i32(NORM_KINDS[post[0]] if post is not None else 2), _ptr(part(post, 1)), _ptr(part(post, 2)),
+         _f32(post[3] if post is not None else 0.0), _ptr(rows), _i32(n_rows),
+         _i32(NORM_KINDS[norm[0]] if norm is not None else 0), _ptr(part(norm, 1)), _ptr(part(norm, 2)),
+         _f32(norm[3] if norm is not None else 0.0), _i32(_tag(weights[0], "sandwich_step") if weights else 0), _ptr(out),
+         _i32(_tag(out, "sandwich_step") if out is not None else 0), _stream())
+
+
+def embed_norm(ids: torch.Tensor, table: torch.Tensor, weight: torch.Tensor, kind: str, eps: float, out: torch.Tensor,
+               bad_id: torch.Tensor, scale: float = 1.0) -> None:
+    """out[t] = norm(float32(table[ids[t]]) * scale) * weight, kind "layernorm" or "rmsnorm"; ``bad_id`` as for
+    ``embed_gather``."""
+    _gpu("embed_norm", ids, table, weight, out, bad_id)
+    tokens = ids.numel()
+    vocab, hidden = table.shape
+    _int_vec("embed_norm: ids", ids)
+    _need(kind in NORM_KINDS, f"embed_norm: a norm is one of {sorted(NORM_KINDS)}, not '{kind}'")
+    _need(table.is_contiguous() and out.is_contiguous() and out.dtype == torch.float32
+          and tuple(out.shape) == (tokens, hidden), f"embed_norm: out must be contiguous float32 [{tokens}, {hidden}]")
+    _need(weight.numel() == hidden and weight.is_contiguous(), f"embed_norm: weight must hold {hidden} values")
+    _need(bad_id.dtype == torch.int32 and bad_id.numel() >= 1, "embed_norm: bad_id must be int32[1]")
+    call("pulse_embed_norm", _ptr(ids), _ptr(table), _i32(_tag(table, "embed_norm")), _ptr(weight),
+         _i32(_tag(weight, "embed_norm")), _i32(NORM_KINDS[kind]), _f32(eps), _ptr(out), _i32(tokens), _i32(hidden),
+         _i32(vocab), _ptr(bad_id), _f32(scale), _stream())
+
+
+# ---------------------------------------------------------------------------
 # Attention inputs with a norm over the whole projection, biases, and keys and values of different widths
 def qkv_rows(qkv: torch.Tensor, q_out: torch.Tensor, nq: int, nkv: int, d: int, dv: int, stored: int,
              biases: Optional[tuple], norm_weights: Optional[tuple], eps: float, cos: Optional[torch.Tensor],
@@ -970,7 +1053,7 @@ def qkv_rows(qkv: torch.Tensor, q_out: torch.Tensor, nq: int, nkv: int, d: int, 
              block_table: Optional[torch.Tensor], write_kv: bool = True, value_scale: float = 1.0,
              norm: Any = True) -> None:
     """q, k, v of ``qkv`` [T, nq*d + nkv*d + nkv*dv] -> biased, q and k normed over the whole row (``norm`` True, with
-    ``norm_weights`` = (wq [nq*d], wk [nkv*d]) or None) or head by head without weights (``norm`` "head"), rotated; q to ``q_out`` [T, nq*stored], k and v (times
+    ``norm_weights`` = (wq [nq*d], wk [nkv*d]) or None) or head by head (``norm`` "head", with weights of d values that the heads share, or None), rotated; q to ``q_out`` [T, nq*stored], k and v (times
     ``value_scale``) to their pages, every head filled with zeros up to ``stored`` channels."""
     _gpu("qkv_rows", qkv, q_out, cos, sin, kcache, vcache, positions, token_entry, block_table)
     tokens = qkv.shape[0]
@@ -982,7 +1065,7 @@ def qkv_rows(qkv: torch.Tensor, q_out: torch.Tensor, nq: int, nkv: int, d: int, 
     _int_vec("qkv_rows: token_entry", token_entry, tokens)
     w_tag = None
     ptrs = [None] * 5
-    sizes = (nq * d, nkv * d, nkv * dv, nq * d, nkv * d)
+    sizes = (nq * d, nkv * d, nkv * dv, *((d, d) if norm == "head" else (nq * d, nkv * d)))
     given = list(biases or (None, None, None)) + list(norm_weights or (None, None))
     for i, (t, n) in enumerate(zip(given, sizes)):
         if t is None:
@@ -1126,6 +1209,124 @@ def gated_rmsnorm(o: torch.Tensor, weight: torch.Tensor, gate: Optional[torch.Te
     call("pulse_gated_rmsnorm", _ptr(o), _i64(row(o)), _ptr(weight), _i32(_tag(weight, "gated_rmsnorm")), _ptr(gate),
          _i64(row(gate) if gate is not None else 0), _ptr(out), _i64(row(out)), _i32(_tag(out, "gated_rmsnorm")),
          _i32(tokens), _i32(n), _f32(eps), _f32(scale), _stream())
+
+
+# ---------------------------------------------------------------------------
+# The gated delta rule
+DELTA_MAX_DIM = 256
+DELTA_MAX_TAPS = 16
+
+
+def delta_slot_floats(heads: int, groups: int, d: int, dv: int, taps: int) -> int:
+    """Float32 values of a request's slot: the state, then the ring of the convolutions' inputs, filled up to a multiple
+    of 4."""
+    n = heads * d * dv + taps * (2 * groups * d + heads * dv)
+    return (n + 3) // 4 * 4
+
+
+def _delta_common(what: str, state: torch.Tensor, heads: int, groups: int, d: int, dv: int, taps: torch.Tensor) -> int:
+    channels = 2 * groups * d + heads * dv
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2
+          and state.shape[1] >= delta_slot_floats(heads, groups, d, dv, taps.shape[0]),
+          f"{what}: state must be float32 [slots, {delta_slot_floats(heads, groups, d, dv, taps.shape[0])}]")
+    _need(taps.dtype == torch.float32 and taps.is_contiguous() and taps.dim() == 2 and taps.shape[1] == channels,
+          f"{what}: the taps must be float32 [taps, {channels}]")
+    return channels
+
+
+def _delta_gates(what: str, heads: int, a_log: torch.Tensor, dt_bias: torch.Tensor) -> None:
+    for t in (a_log, dt_bias):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == heads, f"{what}: A_log and dt_bias must be float32 [{heads}]")
+
+
+def delta_prepare(x: torch.Tensor, b0: int, a0: int, taps: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
+                  state: torch.Tensor, rows: torch.Tensor, gates: torch.Tensor, positions: torch.Tensor,
+                  token_entry: torch.Tensor, entry_start: torch.Tensor, entry_first_row: torch.Tensor,
+                  entry_slot: torch.Tensor, heads: int, groups: int, d: int, dv: int) -> None:
+    """rows [T, channels] float32 = silu of the convolved columns 0 .. channels of ``x``, q and k (groups x d each) as unit
+    vectors, q times d^(-1/2), then v (heads x dv); gates [T, 2 heads] float32 = logarithms of the decays, strengths.  The
+    convolutions' rings in ``state`` [slots, n] are read and moved on."""
+    _gpu("delta_prepare", x, taps, a_log, dt_bias, state, rows, gates, positions, token_entry, entry_start, entry_first_row, entry_slot)
+    tokens, entries = x.shape[0], entry_start.numel()
+    channels = _delta_common("delta_prepare", state, heads, groups, d, dv, taps)
+    _delta_gates("delta_prepare", heads, a_log, dt_bias)
+    _need(x.dim() == 2 and x.stride(1) == 1 and min(b0, a0) >= 0 and x.shape[1] >= max(channels, b0 + heads, a0 + heads),
+          "delta_prepare: x too narrow")
+    _need(rows.dtype == torch.float32 and rows.is_contiguous() and tuple(rows.shape) == (tokens, channels)
+          and gates.dtype == torch.float32 and gates.is_contiguous() and tuple(gates.shape) == (tokens, 2 * heads),
+          f"delta_prepare: rows and gates must be float32 [{tokens}, {channels}] and [{tokens}, {2 * heads}]")
+    for name, t, n in (("positions", positions, tokens), ("token_entry", token_entry, tokens), ("entry_start", entry_start, entries),
+                       ("entry_first_row", entry_first_row, entries + 1), ("entry_slot", entry_slot, entries)):
+        _int_vec(f"delta_prepare: {name}", t, n)
+    call("pulse_delta_prepare", _ptr(x), _i32(_tag(x, "delta_prepare")), _i64(x.stride(0) if tokens > 1 else x.shape[1]), _i32(b0),
+         _i32(a0), _ptr(taps), _ptr(a_log), _ptr(dt_bias), _ptr(state), _i32(state.shape[0]), _i64(state.shape[1]), _ptr(rows),
+         _ptr(gates), _ptr(positions), _ptr(token_entry), _ptr(entry_start), _ptr(entry_first_row), _ptr(entry_slot),
+         _i32(tokens), _i32(entries), _i32(heads), _i32(groups), _i32(d), _i32(dv), _i32(taps.shape[0]), _stream())
+
+
+def delta_row_groups(entries: int, heads: int, d: int, dv: int) -> int:
+    """Over how many lanes ``delta_walk`` shares a column's rows out: 16, unless 4 give the launch wavefronts enough."""
+    from .device import compute_units
+    if d <= 32 or entries * heads * ((dv + 63) // 64) >= 4 * compute_units():
+        return 4
+    return 16
+
+
+def delta_walk(rows: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, state: torch.Tensor, entry_first_row: torch.Tensor,
+               entry_start: torch.Tensor, entry_slot: torch.Tensor, heads: int, groups: int, d: int, dv: int,
+               n_taps: int, row_groups: int) -> None:
+    """For every entry, token by token over prepared rows: S <- e^g S, u = beta (v - S^T k), S <- S + k u^T, out = S^T q, per
+    head, in float32; S is the front of the entry's slot, zero when the entry starts at position 0."""
+    _gpu("delta_walk", rows, gates, out, state, entry_first_row, entry_start, entry_slot)
+    tokens, entries = rows.shape[0], entry_start.numel()
+    channels = 2 * groups * d + heads * dv
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2
+          and state.shape[1] >= delta_slot_floats(heads, groups, d, dv, n_taps), "delta_walk: the slots are too small")
+    _need(all(t.dtype == torch.float32 and t.is_contiguous() for t in (rows, gates, out)) and tuple(rows.shape) == (tokens, channels)
+          and tuple(gates.shape) == (tokens, 2 * heads) and tuple(out.shape) == (tokens, heads * dv),
+          f"delta_walk: float32 rows [T, {channels}], gates [T, {2 * heads}] and out [T, {heads * dv}] are needed")
+    for name, t, n in (("entry_start", entry_start, entries), ("entry_first_row", entry_first_row, entries + 1),
+                       ("entry_slot", entry_slot, entries)):
+        _int_vec(f"delta_walk: {name}", t, n)
+    call("pulse_delta_walk", _ptr(rows), _ptr(gates), _ptr(out), _ptr(state), _i32(state.shape[0]), _i64(state.shape[1]),
+         _ptr(entry_first_row), _ptr(entry_start), _ptr(entry_slot), _i32(entries), _i32(heads), _i32(groups), _i32(d), _i32(dv),
+         _i32(n_taps), _i32(row_groups), _stream())
+
+
+def delta_decode_takes(d: int, dv: int) -> bool:
+    """Whether ``delta_decode`` takes heads of these sizes (as pulse_delta_decode_takes)."""
+    if not (1 <= d <= DELTA_MAX_DIM and 4 <= dv <= 512 and dv % 4 == 0):
+        return False
+    columns = 1
+    while columns < dv // 4:
+        columns *= 2
+    return -(-d // (512 // columns)) <= 32
+
+
+def delta_decode(x: torch.Tensor, g0: int, b0: int, a0: int, taps: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
+                 norm_weight: torch.Tensor, state: torch.Tensor, out: torch.Tensor, positions: torch.Tensor,
+                 token_entry: torch.Tensor, entry_slot: torch.Tensor, heads: int, groups: int, d: int, dv: int, eps: float,
+                 out_scale: float = 1.0) -> None:
+    """A step of single tokens in one launch: ``delta_prepare``, ``delta_walk`` and the heads' norm with its weight
+    (float32 [dv], shared) and silu gate (columns g0 .. of ``x``); out [T, heads * dv] of x's storage type."""
+    _gpu("delta_decode", x, taps, a_log, dt_bias, norm_weight, state, out, positions, token_entry, entry_slot)
+    tokens = x.shape[0]
+    channels = _delta_common("delta_decode", state, heads, groups, d, dv, taps)
+    _delta_gates("delta_decode", heads, a_log, dt_bias)
+    _need(delta_decode_takes(d, dv), f"delta_decode: heads of {d} x {dv} are not a size it takes")
+    _need(norm_weight.dtype == torch.float32 and norm_weight.is_contiguous() and norm_weight.numel() == dv,
+          f"delta_decode: the norm's weight must be float32 [{dv}]")
+    _need(x.dim() == 2 and x.stride(1) == 1 and min(g0, b0, a0) >= 0
+          and x.shape[1] >= max(channels, b0 + heads, a0 + heads, g0 + heads * dv), "delta_decode: x too narrow")
+    _need(out.dim() == 2 and out.stride(1) == 1 and out.dtype == x.dtype and out.shape[0] == tokens and out.shape[1] >= heads * dv,
+          "delta_decode: out must be of x's storage type and wide enough")
+    for name, t, n in (("positions", positions, tokens), ("token_entry", token_entry, tokens), ("entry_slot", entry_slot, tokens)):
+        _int_vec(f"delta_decode: {name}", t, n)
+    row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
+    call("pulse_delta_decode", _ptr(x), _i32(_tag(x, "delta_decode")), _i64(row(x)), _i32(g0), _i32(b0), _i32(a0), _ptr(taps),
+         _ptr(a_log), _ptr(dt_bias), _ptr(norm_weight), _ptr(state), _i32(state.shape[0]), _i64(state.shape[1]), _ptr(out),
+         _i64(row(out)), _ptr(positions), _ptr(token_entry), _ptr(entry_slot), _i32(tokens), _i32(heads), _i32(groups), _i32(d),
+         _i32(dv), _i32(taps.shape[0]), _f32(eps), _f32(out_scale), _stream())
 
 
 # ---------------------------------------------------------------------------

@@ -5,8 +5,8 @@ those of ``attention``; so are the attention kernels, which this part inherits.
 
 Parameters beyond those of ``attention``: ``value_dim`` (default ``head_dim``); ``bias`` (q, k and v have biases,
 named by ``names`` as ``q_bias`` ...); ``qk_norm``: "projection", "head" (every head of q and k divided by its own root
-mean square, no weights; the same before or after the rotation, which keeps a head's sum of squares) or False;
-``qk_norm_eps``; ``out_scale`` (a factor on the result; it is multiplied into the values as they are stored, in
+mean square before the rotation; without weights, or with ``qk_norm_weights`` True one vector of ``head_dim`` values for q
+and one for k, shared by the heads) or False; ``qk_norm_eps``; ``out_scale`` (a factor on the result; it is multiplied into the values as they are stored, in
 float32 before their one rounding); ``output_gate``: "channel": the heads' outputs are multiplied element by element
 by sigmoid(Wg x), Wg [heads * value_dim, hidden] (tensor ``gate``), whose rows ride behind q, k and v in the stacked
 projection and whose sigmoid the attention kernels apply as they store; ``score_cap`` and ``sink`` as for
@@ -64,6 +64,9 @@ class RowPreparedAttention(PagedAttention):
         if params.get("qk_norm", False) == "projection":
             specs[n["q_norm"]] = TensorSpec((nq * d,), kind="norm")
             specs[n["k_norm"]] = TensorSpec((nkv * d,), kind="norm")
+        if params.get("qk_norm", False) == "head" and params.get("qk_norm_weights", False):
+            specs[n["q_norm"]] = TensorSpec((d,), kind="norm")
+            specs[n["k_norm"]] = TensorSpec((d,), kind="norm")
         if params.get("output_gate", False):
             specs[n["gate"]] = TensorSpec((nq * dv, hidden), fan_in=hidden)
         if params.get("sink", False):
@@ -138,7 +141,8 @@ class RowPreparedAttention(PagedAttention):
         self.sink = self._load_sink(load, n["sink"]) if params.get("sink", False) else None
         self.talk = load.get(n["talk"]) if self.talks else None
         self.biases = tuple(load.get(n[k]) for k in ("q_bias", "k_bias", "v_bias")) if params.get("bias", False) else None
-        self.norm_weights = (load.get(n["q_norm"]), load.get(n["k_norm"])) if self.row_norm else None
+        weighted = self.row_norm or (self.head_norm and params.get("qk_norm_weights", False))
+        self.norm_weights = (load.get(n["q_norm"]), load.get(n["k_norm"])) if weighted else None
         o = load.get(n["o"])
         if self.d != self.v_dim:   # zero columns where the stored heads hold zero value channels
             wide = o.new_zeros(self.hidden, self.nq, self.d)

@@ -219,19 +219,62 @@ class LazyNorm:
         return self.norm.apply(self.h, None, out)
 
 
+class DeferredUpdate:
+    """An update of the residual that is more than a sum and has not been done yet.  A norm that says ``taken_by`` does it
+    inside its own kernel as it reads the residual; anyone else calls ``apply_to``."""
+
+    taken_by = ""
+
+    def apply_to(self, h: torch.Tensor) -> None:
+        raise NotImplementedError
+
+
 @dataclass
-class StreamUpdate:
+class StreamUpdate(DeferredUpdate):
     """An update of a residual kept in several streams that has not been done yet: every stream becomes a mix of the
     old ones plus a factor of its own times the sublayer's result ``y`` [T, H]: x_t <- sum_s mix[s, t] x_s +
-    out[t] * y.  A norm that says ``takes_streams`` does it inside its own kernel; anyone else calls ``apply_to``."""
+    out[t] * y."""
 
     y: torch.Tensor
     mix: torch.Tensor     # float32 [streams, streams], indexed [from, to]
     out: torch.Tensor     # float32 [streams]
 
+    taken_by = "takes_streams"
+
     def apply_to(self, h: torch.Tensor) -> None:
         from ..ops import kernels
         kernels.streams_step(h, self.out.numel(), update=(self.y, self.mix, self.out))
+
+
+@dataclass
+class NormedTerms:
+    """A sublayer's result that has not been formed yet: ``factor`` * the sum over (y, weight) of y / sqrt(mean(y^2) + eps)
+    * weight, y [T, H] (one or two of them)."""
+
+    terms: List[Tuple[torch.Tensor, torch.Tensor]]
+    eps: float
+    factor: float = 1.0
+
+
+@dataclass
+class PostNormUpdate(DeferredUpdate):
+    """A sublayer's result that goes through a norm of its own before it is added: h <- h + norm(result).  ``result`` is
+    [T, H] or ``NormedTerms``; ``norm`` = (kind, weight, bias or None, eps)."""
+
+    result: Any
+    norm: tuple
+
+    taken_by = "takes_post_norm"
+
+    def arguments(self) -> Dict[str, Any]:
+        """What ``kernels.sandwich_step`` takes for it."""
+        if isinstance(self.result, NormedTerms):
+            return {"terms": self.result.terms, "term_scale": self.result.factor, "term_eps": self.result.eps, "post": self.norm}
+        return {"terms": [(self.result, None)], "post": self.norm}
+
+    def apply_to(self, h: torch.Tensor) -> None:
+        from ..ops import kernels
+        kernels.sandwich_step(h, **self.arguments())
 
 
 class ResidualStream:
@@ -262,8 +305,8 @@ class ResidualStream:
             from ..ops import kernels
             kernels.residual_add(self.h, pending, scale)
             return None
-        if isinstance(pending, StreamUpdate):
-            if getattr(norm, "takes_streams", False):
+        if isinstance(pending, DeferredUpdate):
+            if getattr(norm, pending.taken_by, False):
                 return pending
             pending.apply_to(self.h)
             return None
@@ -297,7 +340,7 @@ class ResidualStream:
         lies in)."""
         if self.pending is not None:
             from ..ops import kernels
-            if isinstance(self.pending, StreamUpdate):
+            if isinstance(self.pending, DeferredUpdate):
                 self.pending.apply_to(self.h)
             else:
                 kernels.residual_add(self.h, self.pending, self.pending_scale)
@@ -317,7 +360,7 @@ class ResidualStream:
             return
         if self.pending is not None:
             from ..ops import kernels
-            if isinstance(self.pending, StreamUpdate):
+            if isinstance(self.pending, DeferredUpdate):
                 self.pending.apply_to(self.h)
             else:
                 kernels.residual_add(self.h, self.pending, self.pending_scale)

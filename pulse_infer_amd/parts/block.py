@@ -15,6 +15,9 @@ h <- h + mixer(norm(h)).
 sublayers read the stream itself, the norm comes after the sum, ``alpha`` weighs the
 stream in it and ``ls`` are optional factors, one a column, on a sublayer's result.
 
+``sandwich``: h <- h + post_a(mixer(norm_a(h))); h <- h + post_b(ffn(norm_b(h))): a norm before and after every
+sublayer; the feed-forward may be absent.
+
 ``hyper``: the residual is S streams x_1 .. x_S.  Sublayer q reads u = sum_s in_q[s] x_s through its norm, and its
 result y goes back as x_t <- sum_s mix_q[s, t] x_s + out_q[t] * y, all streams at once from the old ones.
 """
@@ -27,8 +30,8 @@ import torch
 from ..models.spec import LayerSpec
 from ..weights.store import TensorSpec
 from ..ops import kernels
-from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BuildContext, Part, ResidualStream, StepContext, StreamUpdate,
-                   joined, says)
+from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BuildContext, Part, PostNormUpdate, ResidualStream, StepContext,
+                   StreamUpdate, joined, says)
 
 
 @BLOCKS.register("prenorm")
@@ -328,6 +331,78 @@ class PostNormBlock(Part):
         self._close(stream, ctx, "mixer_norm", self.mixer.forward(self._rows(stream, ctx), ctx, cache))
         if self.ffn is not None:
             self._close(stream, ctx, "ffn_norm", self.ffn.forward(self._rows(stream, ctx), ctx))
+
+
+@BLOCKS.register("sandwich")
+class SandwichBlock(Part):
+    """A norm before and a norm after every sublayer: h <- h + post(sublayer(pre(h))).  Block parameters: ``mixer_norm`` /
+    ``mixer_post`` / ``ffn_norm`` / ``ffn_post``, the norms' tensor prefixes below the layer's.  A layer without a
+    feed-forward ends after the mixer.  A sublayer may hand back ``NormedTerms`` instead of a tensor.
+
+    The second norm and the sum are no launch of their own: they are handed on as a ``PostNormUpdate`` and done by the
+    kernel of the norm that reads the residual next (this layer's next one, the next layer's first, the model's last)."""
+
+    NORM_PLACES = ("mixer_norm", "mixer_post", "ffn_norm", "ffn_post")
+    SUBLAYERS = (("mixer_norm", "mixer_post"), ("ffn_norm", "ffn_post"))
+
+    @classmethod
+    def _places(cls, layer: LayerSpec):
+        return cls.NORM_PLACES if layer.ffn is not None else cls.SUBLAYERS[0]
+
+    @classmethod
+    def layer_weight_specs(cls, layer: LayerSpec) -> Dict[str, TensorSpec]:
+        p = layer.block.params
+        out: Dict[str, TensorSpec] = {}
+        for which in cls._places(layer):
+            norm = layer.norm(which)
+            for name, spec in NORMS.get(norm.kind).weight_specs(norm.params).items():
+                out[joined(joined(layer.prefix, p[which]), name)] = spec
+        parts = [(layer.mixer, MIXERS)] + ([(layer.ffn, FEED_FORWARDS)] if layer.ffn is not None else [])
+        for part, registry in parts:
+            sub = joined(layer.prefix, part.params.get("prefix", ""))
+            for name, spec in registry.get(part.kind).weight_specs(part.params).items():
+                out[joined(sub, name)] = spec
+        return out
+
+    def __init__(self, layer: LayerSpec, build: BuildContext):
+        p = layer.block.params
+        self.norms: Dict[str, Any] = {}
+        for which in self._places(layer):
+            norm = layer.norm(which)
+            self.norms[which] = NORMS.get(norm.kind)(norm.params, joined(layer.prefix, p[which]), build)
+        for which in ("mixer_post", "ffn_post"):
+            if which in self.norms and not hasattr(self.norms[which], "as_step"):
+                raise ValueError(f"the sandwich block has no kernel for a '{self.norms[which].kind}' behind a sublayer")
+        self.mixer = MIXERS.get(layer.mixer.kind)(layer.mixer.params,
+                                                  joined(layer.prefix, layer.mixer.params.get("prefix", "")), build)
+        self.ffn = None
+        if layer.ffn is not None:
+            self.ffn = FEED_FORWARDS.get(layer.ffn.kind)(layer.ffn.params,
+                                                         joined(layer.prefix, layer.ffn.params.get("prefix", "")), build)
+        self.act_dtype = build.act_dtype
+
+    def cache_spec(self) -> Optional[Any]:
+        return self.mixer.cache_spec()
+
+    def records_cleanly(self) -> bool:
+        return all(says(part, "records_cleanly") for part in (self.mixer, self.ffn, *self.norms.values())
+                   if part is not None)
+
+    def entry_norm(self) -> Any:
+        return self.norms["mixer_norm"]
+
+    def _sublayer(self, stream: ResidualStream, ctx: StepContext, place: int, run) -> None:
+        before, after = self.SUBLAYERS[place]
+        x = ctx.workspace.buffer("block.normed", ctx.num_tokens, stream.h.shape[1], self.act_dtype)
+        result = run(stream.normed(self.norms[before], x))
+        if isinstance(result, tuple):
+            raise TypeError("the sandwich block takes one result a sublayer")
+        stream.push(PostNormUpdate(result, self.norms[after].as_step()))
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: Any) -> None:
+        self._sublayer(stream, ctx, 0, lambda x: self.mixer.forward(x, ctx, cache))
+        if self.ffn is not None:
+            self._sublayer(stream, ctx, 1, lambda x: self.ffn.forward(x, ctx))
 
 
 @BLOCKS.register("hyper")

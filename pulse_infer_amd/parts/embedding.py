@@ -23,8 +23,11 @@ class TokenEmbedding(Part):
 
     @classmethod
     def weight_specs(cls, params: Dict[str, Any]) -> Dict[str, TensorSpec]:
-        return {params["name"]: TensorSpec((params["vocab_size"], params["hidden_size"]), kind="embedding",
-                                           fan_in=params["hidden_size"])}
+        specs = {params["name"]: TensorSpec((params["vocab_size"], params["hidden_size"]), kind="embedding",
+                                            fan_in=params["hidden_size"])}
+        if params.get("norm") is not None:
+            specs[params["norm"]["tensor"]] = TensorSpec((params["hidden_size"],), kind="norm")
+        return specs
 
     @classmethod
     def step_cost(cls, params: Dict[str, Any], entries: List[Tuple[int, int]], weight_bytes: int,
@@ -39,13 +42,23 @@ class TokenEmbedding(Part):
         self.table = build.loader.get(params["name"])
         self.scale = float(params.get("scale", 1.0))   # every gathered row is multiplied by it, in float32
         self.streams = int(params.get("streams", 1))   # a residual of several streams gets the row in every one
+        # a norm of every gathered row: {"kind": "layernorm" or "rmsnorm", "tensor": its weight's name, "eps"}
+        self.norm = None
+        if params.get("norm") is not None:
+            n = params["norm"]
+            if n["kind"] not in kernels.NORM_KINDS or self.streams > 1:
+                raise ValueError(f"the embedding has a norm of {sorted(kernels.NORM_KINDS)} in a residual of one stream")
+            self.norm = (build.loader.get(n["tensor"]), n["kind"], float(n["eps"]))
         self.bad_id = torch.zeros(1, dtype=torch.int32, device=build.device)
 
     def forward(self, ids: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
         """The step function checks ids on the host before it runs.  A caller that comes another way and brings an
         id outside the table gets a row of NaN, which reaches that token's logits (no token is chosen from them),
         never a silent row of zeros; ``saw_bad_id`` tells, at the price of a synchronisation."""
-        if self.streams > 1:
+        if self.norm is not None:
+            weight, kind, eps = self.norm
+            kernels.embed_norm(ids, self.table, weight, kind, eps, out, self.bad_id, self.scale)
+        elif self.streams > 1:
             kernels.embed_streams(ids, self.table, out, self.bad_id, self.streams, self.scale)
         else:
             kernels.embed_gather(ids, self.table, out, self.bad_id, self.scale)

@@ -12,7 +12,7 @@ import torch
 
 from ..ops import kernels
 from ..weights.store import TensorSpec
-from .base import NORMS, BuildContext, LazyNorm, Part, RowStats, StreamUpdate, joined
+from .base import NORMS, BuildContext, LazyNorm, Part, PostNormUpdate, RowStats, StreamUpdate, joined
 
 
 @NORMS.register("rmsnorm")
@@ -32,9 +32,22 @@ class RMSNorm(Part):
     takes_parts = True   # delta may be [parts, T, H] float32: the kernel adds the parts in order
     takes_scale = True   # ``apply`` takes a factor on the update
 
+    @property
+    def takes_post_norm(self) -> bool:   # ``apply`` takes a ``PostNormUpdate`` as the update and does it on the way
+        return self.weight_offset == 0.0
+
+    def as_step(self) -> tuple:
+        """(kind, weight, bias, eps) as ``kernels.sandwich_step`` takes a norm."""
+        if self.weight_offset != 0.0:
+            raise ValueError("a norm inside a step of several norms has plain weights")
+        return "rmsnorm", self.weight, None, self.eps
+
     def apply(self, h: torch.Tensor, delta: Optional[torch.Tensor], out: torch.Tensor,
               rows: Optional[torch.Tensor] = None, delta_scale: float = 1.0) -> torch.Tensor:
         """out = norm(h + delta_scale * delta) * w; h keeps the sum unless rows are gathered."""
+        if isinstance(delta, PostNormUpdate):
+            kernels.sandwich_step(h, **delta.arguments(), norm=self.as_step(), out=out, rows=rows)
+            return out
         kernels.add_rmsnorm(h, delta, self.weight, self.eps, out, rows=rows, weight_offset=self.weight_offset,
                             delta_scale=delta_scale)
         return out
@@ -65,6 +78,14 @@ class LayerNorm(Part):
     records_cleanly = True
     takes_streams = True    # ``apply`` takes a ``StreamUpdate`` as the update and does it on the way
 
+    @property
+    def takes_post_norm(self) -> bool:   # and a ``PostNormUpdate``, of a residual of one stream
+        return self.streams == 1
+
+    def as_step(self) -> tuple:
+        """(kind, weight, bias, eps) as ``kernels.sandwich_step`` takes a norm."""
+        return "layernorm", self.weight, self.bias, self.eps
+
     @classmethod
     def weight_specs(cls, params: Dict[str, Any]) -> Dict[str, TensorSpec]:
         out = {params.get("tensor", "weight"): TensorSpec((params["size"],), kind="norm")}
@@ -87,7 +108,10 @@ class LayerNorm(Part):
               stream_weights: Optional[torch.Tensor] = None) -> torch.Tensor:
         """out = norm(sum_s weights[s] * h_s) after ``delta`` has gone into h: a ``StreamUpdate`` (done by the same
         kernel; with gathered rows the updated streams are used but not stored: who gathers rows reads the residual
-        for the last time), a tensor of h's shape (added first), or None."""
+        for the last time), a ``PostNormUpdate`` (likewise), a tensor of h's shape (added first), or None."""
+        if isinstance(delta, PostNormUpdate):
+            kernels.sandwich_step(h, **delta.arguments(), norm=self.as_step(), out=out, rows=rows)
+            return out
         update = None
         if isinstance(delta, StreamUpdate):
             update = (delta.y, delta.mix, delta.out)

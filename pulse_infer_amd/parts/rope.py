@@ -6,9 +6,14 @@ The reference rotates ADJACENT pairs (x[2i], x[2i+1])
 Once per step this part makes the cos/sin tables for the step's positions (angles in
 float64, tables float32); the mixer's fused kernel applies them to q and k.
 ``scaling_factor`` f (default 1) divides every frequency by f ("linear scaling": position p turns like p / f).
+``yarn`` = {"factor", "original", "fast", "slow"} divides the slow frequencies by ``factor`` and leaves the fast ones as
+they are: with t(n) = rotary_dim ln(original / (2 pi n)) / (2 ln theta), the index of the frequency that makes n turns over
+``original`` positions, a ramp over i goes from 0 at max(floor(t(fast)), 0) to 1 at min(ceil(t(slow)), rotary_dim - 1),
+and frequency i becomes f_i (ramp / factor + 1 - ramp); the tables are multiplied by 0.1 ln(factor) + 1.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 from typing import Any, Dict
 
@@ -49,15 +54,29 @@ class RotaryEmbedding(Part):
         self.scaling_factor = float(params.get("scaling_factor", 1.0))
         if not self.scaling_factor > 0:
             raise ValueError(f"a rope scaling factor must be positive, got {self.scaling_factor}")
-        self.inv_freq = (torch.pow(torch.tensor(self.theta, dtype=torch.float64), -exponent)
-                         / self.scaling_factor).to(build.device)
+        freq = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -exponent) / self.scaling_factor
+        self.magnitude = 1.0
+        if params.get("yarn") is not None:
+            freq, self.magnitude = self.yarn(freq, params["yarn"])
+        self.inv_freq = freq.to(build.device)
         self.name = params.get("name", "rope")
+
+    def yarn(self, freq: torch.Tensor, params: Dict[str, Any]):
+        """(frequencies, magnitude) under the ``yarn`` scaling."""
+        factor, original, fast, slow = (float(params[k]) for k in ("factor", "original", "fast", "slow"))
+        if min(factor, original, fast, slow) <= 0 or self.theta == 1.0:
+            raise ValueError(f"yarn scaling needs positive numbers and a theta other than 1, got {params}, theta {self.theta}")
+        n = self.rotary_dim
+        index = lambda turns: n * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(self.theta))
+        low, high = max(math.floor(index(fast)), 0), min(math.ceil(index(slow)), n - 1)
+        ramp = ((torch.arange(n // 2, dtype=torch.float64) - low) / max(high - low, 0.001)).clamp(0.0, 1.0)
+        return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
     def prepare(self, ctx: StepContext) -> RotationTables:
         half = self.rotary_dim // 2
         cos = ctx.workspace.buffer(f"{self.name}.cos", ctx.num_tokens, half, torch.float32)
         sin = ctx.workspace.buffer(f"{self.name}.sin", ctx.num_tokens, half, torch.float32)
-        kernels.rope_table(ctx.positions, self.inv_freq, cos, sin)
+        kernels.rope_table(ctx.positions, self.inv_freq, cos, sin, self.magnitude)
         return RotationTables(cos, sin, self.rotary_dim, self.pairing)
 
 

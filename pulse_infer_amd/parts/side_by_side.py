@@ -9,6 +9,11 @@ A branch says what it computes up to its output projection: ``inner_width``, ``o
 and ``forward_inner(x, ctx, cache, out)``, which writes its share of one wide row with its factor already in it (its
 parameter ``out_scale``).  The output projections of all branches are then ONE product: the wide rows against the
 branches' output weights side by side.
+
+With ``branch_norm`` = {"tensor", "eps", "factor"} every branch's result is divided by its own root mean square over the
+model's width and multiplied by a weight (the tensor of that name below the branch's prefix) before the sum, which is then
+multiplied by ``factor``.  The branches are projected by products of their own, and the part hands back ``NormedTerms``:
+norms and sum are done by the kernel that adds the update to the residual.  At most two branches, without ``scale``.
 """
 from __future__ import annotations
 
@@ -18,7 +23,7 @@ import torch
 
 from ..cache.specs import CombinedSpec
 from ..weights.store import TensorSpec
-from .base import MIXERS, BuildContext, Part, StepContext, StepCost, joined, says
+from .base import MIXERS, BuildContext, NormedTerms, Part, StepContext, StepCost, joined, says
 from .linear import Linear
 
 
@@ -37,6 +42,8 @@ class SideBySideMixer(Part):
             sub = _branch_params(branch)
             for name, spec in MIXERS.get(branch["kind"]).weight_specs(sub).items():
                 out[joined(sub.get("prefix", ""), name)] = spec
+            if params.get("branch_norm") is not None:
+                out[joined(sub.get("prefix", ""), params["branch_norm"]["tensor"])] = TensorSpec((params["hidden_size"],), kind="norm")
         return out
 
     @classmethod
@@ -59,6 +66,16 @@ class SideBySideMixer(Part):
             self.branches.append(part)
         if not self.branches:
             raise ValueError("side_by_side needs at least one branch")
+        self.act_dtype = build.act_dtype
+        self.specs = [part.cache_spec() for part in self.branches]
+        self.branch_norm = params.get("branch_norm")
+        if self.branch_norm is not None:
+            if len(self.branches) > 2 or any(float(b.get("scale", 1.0)) != 1.0 for b in params["branches"]):
+                raise ValueError("side_by_side norms the results of at most two branches, which then have no factors")
+            self.outs = [Linear(part.out_weight(), build.mode) for part in self.branches]
+            self.norm_weights = [build.loader.get(joined(joined(prefix, b["params"].get("prefix", "")), self.branch_norm["tensor"]))
+                                 for b in params["branches"]]
+            return
         # where each branch writes in the wide row (starts kept at multiples of 16 values for the kernels' wide accesses)
         self.starts: List[int] = []
         at = 0
@@ -76,8 +93,6 @@ class SideBySideMixer(Part):
             weights = [w.to(torch.float32) for w in weights]
         self.out = Linear(torch.cat(weights, dim=1).contiguous(), build.mode)
         self.padded = any((part.inner_width % 16) for part in self.branches)
-        self.specs = [part.cache_spec() for part in self.branches]
-        self.act_dtype = build.act_dtype
 
     def records_cleanly(self) -> bool:
         return all(says(part, "records_cleanly") for part in self.branches)
@@ -86,9 +101,11 @@ class SideBySideMixer(Part):
         kept = tuple(spec for spec in self.specs if spec is not None)
         return CombinedSpec(kept) if kept else None
 
-    def forward(self, x: torch.Tensor, ctx: StepContext, cache: Any) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache: Any) -> Any:
         ws = ctx.workspace
         tokens = x.shape[0]
+        if self.branch_norm is not None:
+            return self._forward_normed(x, ctx, cache)
         wide = ws.buffer("side_by_side.inner", tokens, self.width, self.act_dtype)
         if self.padded:
             wide.zero_()   # (columns between the branches meet zero weights, but must not hold NaN)
@@ -97,3 +114,15 @@ class SideBySideMixer(Part):
             view = next(views) if spec is not None else None
             part.forward_inner(x, ctx, view, wide[:, start:start + part.inner_width])
         return self.out.forward(wide, ws.buffer("side_by_side.out", tokens, self.hidden, self.act_dtype))
+
+    def _forward_normed(self, x: torch.Tensor, ctx: StepContext, cache: Any) -> NormedTerms:
+        ws, tokens = ctx.workspace, x.shape[0]
+        views = iter(cache if cache is not None else ())
+        terms = []
+        for i, (part, spec) in enumerate(zip(self.branches, self.specs)):
+            view = next(views) if spec is not None else None
+            inner = ws.buffer("side_by_side.inner", tokens, part.inner_width, self.act_dtype)
+            part.forward_inner(x, ctx, view, inner)
+            y = ws.buffer(f"side_by_side.out{i}", tokens, self.hidden, self.act_dtype)
+            terms.append((self.outs[i].forward(inner, y), self.norm_weights[i]))
+        return NormedTerms(terms, float(self.branch_norm["eps"]), float(self.branch_norm.get("factor", 1.0)))
