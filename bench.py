@@ -55,14 +55,14 @@ def parse_args() -> argparse.Namespace:
     p.add_argument("--context", type=int, default=4096, help="context length the timed decode steps end at")
     p.add_argument("--model", choices=sorted(SHAPES), default="8b", help="layer sizes: Qwen3-8B (the default), 14B or 32B")
     p.add_argument("--layers", type=int, default=None, help="fewer layers than the model has, if memory or time needs it")
-    p.add_argument("--workload", choices=["decode", "serving", "long-prompt", "dirozen", "kesovik", "tipidra", "fosupel"], default="decode",
+    p.add_argument("--workload", choices=["decode", "serving", "long-prompt", "dirozen", "kesovik", "tipidra", "fosupel", "makezen"], default="decode",
                    help="decode: fixed batch at a fixed context; serving: continuous batching of requests with "
                         "seeded prompt lengths, chunked prefill mixed with decoding; long-prompt: one prompt of "
                         "--prompt-tokens tokens in portions of --chunk tokens; dirozen / kesovik: decoding and prefill of "
                         "that design beside Qwen3 layers of equal sizes, with both models' time by entry point; "
-                        "tipidra: the same beside Kesovik and Qwen3 layers")
-    p.add_argument("--compare-layers", type=int, default=4, help="dirozen, kesovik, tipidra: layers of the models that are compared")
-    p.add_argument("--compare-sizes", default="2k,4k,5k", help="dirozen, kesovik, tipidra: which of the layer sizes 2k, 4k, 5k (widths) to run")
+                        "tipidra, fosupel: the same beside Kesovik and Qwen3 layers; makezen: beside Fosupel, Kesovik and Qwen3")
+    p.add_argument("--compare-layers", type=int, default=4, help="dirozen, kesovik, tipidra, fosupel, makezen: layers of the models that are compared")
+    p.add_argument("--compare-sizes", default="2k,4k,5k", help="dirozen, kesovik, tipidra, fosupel, makezen: which of the layer sizes 2k, 4k, 5k (widths) to run")
     p.add_argument("--prompt-tokens", type=int, default=16384, help="long-prompt: length of the prompt")
     p.add_argument("--requests", type=int, default=32, help="serving: number of requests")
     p.add_argument("--prompt-range", type=int, nargs=2, default=[128, 2048], help="serving: prompt lengths drawn from [lo, hi]")
@@ -293,15 +293,39 @@ def fosupel_layers(size, layers):
     return [turn[i % len(turn)] for i in range(layers)]
 
 
+def makezen_layers(size, layers):
+    """Makezen layers at the comparison's sizes, in turn: capped attention (heads as Qwen3's, a blended rotation on half
+    of a head) beside a gated delta rule with half as many heads; latent attention (heads as Qwen3's, a latent row of 512
+    values and a turned part of 64, queries from 3/8 of the width, a window of 1,024 tokens); the gated delta rule alone
+    (heads as Qwen3's, half as many heads of q and k); latent attention that reads the rows of the one before.  All with
+    a dense feed-forward."""
+    dim, heads = size["dim"], size["heads"]
+    scaling = {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}
+    left = {"dim": dim, "heads": heads, "kv_heads": size["kv_heads"], "rot": {"base": 1e6, "dims": dim // 2, "scaling": scaling},
+            "scale": dim ** -0.5, "softcap": 30.0, "vdim": dim}
+    delta = lambda h, groups: {"conv": 4, "dim": dim, "heads": h, "kv_heads": groups, "vdim": dim}
+    latent = {"dim": dim, "heads": heads, "kv_rank": 512, "mask": {"size": 1024}, "q_rank": size["width"] * 3 // 8,
+              "rot": {"base": 1e6, "dims": 64, "scaling": scaling}, "rot_dim": 64, "scale": (dim + 64) ** -0.5, "vdim": dim}
+    dense = {"ff": size["ff"], "kind": "dense"}
+    turn = [("parallel", {"left": left, "right": delta(heads // 2, heads // 2)}), ("latent_attention", latent),
+            ("delta", delta(heads, heads // 2)), ("latent_attention", latent)]
+    out = []
+    for i in range(layers):
+        kind, mixer = turn[i % 4]
+        out.append({"type": kind, "mixer": dict(mixer, kv_from=i - 2) if i % 4 == 3 else mixer, "mlp": dense})
+    return out
+
+
 def dirozen_compare(args, design: str = "dirozen") -> int:
-    """Dirozen (or, with ``design`` "kesovik", Kesovik) beside Qwen3 layers of equal sizes (random weights, ``--compare-layers`` layers, a vocabulary of
+    """Dirozen (or, with ``design`` "kesovik", Kesovik, and so on) beside Qwen3 layers of equal sizes (random weights, ``--compare-layers`` layers, a vocabulary of
     32,000): decoding at batch 1 / 8 / 32 with contexts ending at ``--context`` and a prompt of ``--prefill-tokens``
     tokens, each through the engine's own serving loop, with the fraction of the roofline from the models' own
     descriptions, and where an eager decoding step and a prompt step spend their time by entry point.  One JSON
     line."""
     import torch
 
-    from pulse_infer_amd.config import DirozenConfig, FosupelConfig, KesovikConfig, Qwen3Config, TipidraConfig
+    from pulse_infer_amd.config import (DirozenConfig, FosupelConfig, KesovikConfig, MakezenConfig, Qwen3Config,
+                                        TipidraConfig)
     from pulse_infer_amd.engine.engine import ContinuousBatchEngine
     from pulse_infer_amd.engine.runner import StepEntry
     from pulse_infer_amd.models.causal_lm import expected_tensors
@@ -331,7 +355,7 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
                  "mlp": {"ff": size["ff"], "kind": "dense"}}
         dirozen = DirozenConfig.from_dict({"architecture": "Dirozen", "vocab": vocab, "width": size["width"],
                                            "norm": {"eps": 1e-6}, "layers": [entry] * layers}, "<bench>")
-        if design in ("kesovik", "tipidra", "fosupel"):
+        if design in ("kesovik", "tipidra", "fosupel", "makezen"):
             kesovik = KesovikConfig.from_dict({
                 "architecture": "Kesovik", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                 "embedding": {"scale": 1.0}, "postln_alpha": 2.0, "logit_softcap": 30.0,
@@ -342,10 +366,15 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
                     "embedding": {"scale": 1.0}, "logit_softcap": 30.0, "streams": 4,
                     "layers": tipidra_layers(size, layers)}, "<bench>")
                 return {"tipidra": tipidra, "kesovik": kesovik, "qwen3": qwen}
-            if design == "fosupel":
+            if design in ("fosupel", "makezen"):
                 fosupel = FosupelConfig.from_dict({
                     "architecture": "Fosupel", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                     "residual_mult": 0.5, "logit_softcap": 30.0, "layers": fosupel_layers(size, layers)}, "<bench>")
+                if design == "makezen":
+                    makezen = MakezenConfig.from_dict({
+                        "architecture": "Makezen", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
+                        "layers": makezen_layers(size, layers)}, "<bench>")
+                    return {"makezen": makezen, "fosupel": fosupel, "kesovik": kesovik, "qwen3": qwen}
                 return {"fosupel": fosupel, "kesovik": kesovik, "qwen3": qwen}
             return {"kesovik": kesovik, "qwen3": qwen}
         return {"dirozen": dirozen, "qwen3": qwen}
@@ -431,7 +460,8 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
         torch.cuda.empty_cache()
         return out
 
-    record = {"metric": f"{design}_beside_{'kesovik_and_' if design in ('tipidra', 'fosupel') else ''}qwen3_layers", "unit": "tokens/s", "n_gpus": 1, "dtype": args.dtype,
+    others = {"makezen": "fosupel_kesovik_and_qwen3", "tipidra": "kesovik_and_qwen3", "fosupel": "kesovik_and_qwen3"}
+    record = {"metric": f"{design}_beside_{others.get(design, 'qwen3')}_layers", "unit": "tokens/s", "n_gpus": 1, "dtype": args.dtype,
               "data": "synthetic", "layers": layers, "vocab": vocab, "context": args.context, "sizes": {}}
     for name, size in DIROZEN_SIZES.items():
         if name not in args.compare_sizes.split(","):
@@ -450,7 +480,7 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
 
 def main() -> int:
     args = parse_args()
-    if args.workload in ("kesovik", "tipidra", "fosupel"):
+    if args.workload in ("kesovik", "tipidra", "fosupel", "makezen"):
         return dirozen_compare(args, args.workload)
     if args.workload == "dirozen":
         if args.gpus != 1:
