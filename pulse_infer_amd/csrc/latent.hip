@@ -12,7 +12,15 @@
 // pulse_latent_absorb: q_abs[t, h, :] = W_uk,h^T q_plain[t, h]        (float32 sums, one rounding)
 // pulse_latent_expand: y[t, h, :] = (W_uv,h o[t, h, :rank]) * sigmoid(gate[t, h, :])
 // pulse_heads_product: both of these products for bfloat16 weights on the matrix cores: y[t, h, m] = sum_k
-//                      w[h, m, k] x[t, h, k] (w_uk transposed once at load, w_uv as it is), 16 tokens a workgroup
+//                      w[h, m, k] x[t, h, k] (w_uk transposed once at load, w_uv as it is)
+//
+// Long prompt portions attend to keys and values expanded to every head instead (a third of the arithmetic where the
+// latent row is much wider than a head), in pages of their own that live for one layer of one step:
+// pulse_latent_queries: q[t, h, :] = [plain | turned | 0]
+// pulse_latent_gather:  the cached latent rows of a list of pages, as one dense matrix (the up projections' input)
+// pulse_latent_pages:   the up projections' output and the cached turned parts as keys [pages, heads, page, width] and
+//                       values [pages, heads, width, page]
+// pulse_latent_compact: the heads' results side by side without the channels that fill them up
 #include "common.h"
 
 #include <math.h>
@@ -52,12 +60,12 @@ __global__ void latent_rows_kernel(const TX* __restrict__ x, const TX* __restric
     // the queries' turned parts: q[t, h, rank + e]
     TX* qrow = q + static_cast<int64_t>(t) * a.q_stride;
     const int width = a.rank + a.rot;
-    for (int i = threadIdx.x; i < a.heads * a.rot; i += blockDim.x) {
+    for (int i = threadIdx.x; q && i < a.heads * a.rot; i += blockDim.x) {
         const int h = i / a.rot, e = i % a.rot;
         qrow[static_cast<int64_t>(h) * a.stored + a.rank + e] =
             from_f32<TX>(turned(row + a.q0 + static_cast<int64_t>(h) * (a.d + a.rot) + a.d, e));
     }
-    for (int i = threadIdx.x; i < a.heads * (a.stored - width); i += blockDim.x) {
+    for (int i = threadIdx.x; q && i < a.heads * (a.stored - width); i += blockDim.x) {
         const int h = i / (a.stored - width), e = i % (a.stored - width);
         qrow[static_cast<int64_t>(h) * a.stored + width + e] = from_f32<TX>(0.f);
     }
@@ -153,45 +161,155 @@ template <> __device__ __forceinline__ hp_bf16x8 load8<float>(const float* p) {
     return out;
 }
 
-// A workgroup takes 16 tokens of one head; a wavefront a tile of 16 output channels at a time.  W rows are the matrix
-// cores' row operand (m = output channel), the tokens' rows of x the column operand, so a lane ends up with four
-// neighbouring channels of its token: one 8-byte store.
-template <typename TX>
+// A workgroup takes 16 TT tokens of one head; a wavefront a tile of 16 output channels at a time, whose W operands serve
+// all TT token tiles.  W rows are the matrix cores' row operand (m = output channel), the tokens' rows of x the column
+// operand, so a lane ends up with four neighbouring channels of its token: one 8-byte store.
+template <typename TX, int TT>
 __global__ __launch_bounds__(256) void heads_product_kernel(const TX* __restrict__ x, int64_t x_stride, int x_head,
                                                             const bf16_t* __restrict__ w, const bf16_t* __restrict__ gate,
                                                             int64_t gate_stride, bf16_t* __restrict__ y, int64_t y_stride,
                                                             int y_head, int tokens, int m_out, int k_in, float scale, int gate_heads) {
-    const int t0 = blockIdx.x * 16, h = blockIdx.y;
+    const int t0 = blockIdx.x * (16 * TT), h = blockIdx.y;
     const int lane = threadIdx.x % PULSE_WAVE, wave = threadIdx.x / PULSE_WAVE;
     const int r = lane % 16, g = lane / 16;
-    const int tok = min(t0 + r, tokens - 1);
-    const TX* xrow = x + static_cast<int64_t>(tok) * x_stride + static_cast<int64_t>(h) * x_head;
+    const TX* xrow[TT];
+#pragma unroll
+    for (int u = 0; u < TT; ++u)
+        xrow[u] = x + static_cast<int64_t>(min(t0 + 16 * u + r, tokens - 1)) * x_stride + static_cast<int64_t>(h) * x_head;
     const hp_bf16x8 zero = __builtin_bit_cast(hp_bf16x8, make_uint4(0u, 0u, 0u, 0u));
     for (int m0 = wave * 16; m0 < m_out; m0 += 64) {
         const int m = m0 + r;
         const bf16_t* wrow = m < m_out ? w + (static_cast<int64_t>(h) * m_out + m) * k_in : nullptr;
-        hp_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        hp_f32x4 acc[TT];
+#pragma unroll
+        for (int u = 0; u < TT; ++u) acc[u] = hp_f32x4{0.f, 0.f, 0.f, 0.f};
         for (int k0 = 0; k0 < k_in; k0 += 32) {
             const int k = k0 + 8 * g;
             const bool in = k < k_in;
             const hp_bf16x8 wa = (in && wrow) ? *reinterpret_cast<const hp_bf16x8*>(wrow + k) : zero;
-            const hp_bf16x8 xb = in ? load8<TX>(xrow + k) : zero;
-            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa, xb, acc, 0, 0, 0);
-        }
-        // lane: token r, channels m0 + 4 g + i
-        if (t0 + r < tokens) {
-            const int c0 = m0 + 4 * g;
-            bf16_t* dst = y + static_cast<int64_t>(t0 + r) * y_stride + static_cast<int64_t>(h) * y_head + c0;
-            const bf16_t* gr = gate ? gate + static_cast<int64_t>(t0 + r) * gate_stride + (gate_heads ? h : static_cast<int64_t>(h) * m_out + c0) : nullptr;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                if (c0 + i < m_out) {
-                    float v = acc[i] * scale;
-                    if (gr) v *= 1.0f / (1.0f + expf(-bf16_to_f32(gr[gate_heads ? 0 : i])));
-                    dst[i] = f32_to_bf16(v);
+            for (int u = 0; u < TT; ++u) {
+                const hp_bf16x8 xb = in ? load8<TX>(xrow[u] + k) : zero;
+                acc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa, xb, acc[u], 0, 0, 0);
+            }
+        }
+        // lane: token r of every tile, channels m0 + 4 g + i
+#pragma unroll
+        for (int u = 0; u < TT; ++u) {
+            const int tok = t0 + 16 * u + r, c0 = m0 + 4 * g;
+            if (tok < tokens) {
+                bf16_t* dst = y + static_cast<int64_t>(tok) * y_stride + static_cast<int64_t>(h) * y_head + c0;
+                const bf16_t* gr = gate ? gate + static_cast<int64_t>(tok) * gate_stride + (gate_heads ? h : static_cast<int64_t>(h) * m_out + c0) : nullptr;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    if (c0 + i < m_out) {
+                        float v = acc[u][i] * scale;
+                        if (gr) v *= 1.0f / (1.0f + expf(-bf16_to_f32(gr[gate_heads ? 0 : i])));
+                        dst[i] = f32_to_bf16(v);
+                    }
                 }
             }
         }
+    }
+}
+
+// ------------------------------------------------------------------ keys and values expanded to every head
+// One workgroup a token.
+template <typename TX>
+__global__ void latent_queries_kernel(const TX* __restrict__ x, int64_t x_stride, int q0, TX* __restrict__ q, int64_t q_stride,
+                                      const float* __restrict__ cos_t, const float* __restrict__ sin_t, int heads, int d,
+                                      int rot, int width, int pairing) {
+    const int t = blockIdx.x, half = rot / 2, in = d + rot;
+    const TX* row = x + static_cast<int64_t>(t) * x_stride + q0;
+    const float* ct = cos_t + static_cast<int64_t>(t) * half;
+    const float* st = sin_t + static_cast<int64_t>(t) * half;
+    TX* dst = q + static_cast<int64_t>(t) * q_stride;
+    for (int i = threadIdx.x; i < heads * width; i += blockDim.x) {
+        const int h = i / width, c = i % width;
+        const TX* src = row + static_cast<int64_t>(h) * in;
+        if (c < d) { dst[i] = src[c]; continue; }
+        float v = 0.f;
+        if (c < in) {
+            const int e = c - d;
+            int pair, freq;
+            bool first;
+            if (pairing == 1) { first = e < half; pair = first ? e + half : e - half; freq = first ? e : e - half; }
+            else { first = (e & 1) == 0; pair = e ^ 1; freq = e >> 1; }
+            const float u = to_f32<TX>(src[c]), o = to_f32<TX>(src[d + pair]);
+            v = first ? u * ct[freq] - o * st[freq] : u * ct[freq] + o * st[freq];
+        }
+        dst[i] = from_f32<TX>(v);
+    }
+}
+
+struct ExpandArgs {
+    int heads, d, rot, dv, rank, stored, width;   // width: channels of an expanded head
+    int page, src_page, src_pages, bt_width;      // slots of an expanded page and of a cached one
+};
+
+// The cached row of (entry, position), null where there is none (behind the entry's last token, below its window).
+__device__ __forceinline__ const bf16_t* cached_row(const bf16_t* __restrict__ kcache, const int* __restrict__ block_table,
+                                                    int entry, int pos, int end, const ExpandArgs& a) {
+    if (pos >= end) return nullptr;
+    const int pi = pos / a.src_page;
+    const int pg = pi < a.bt_width ? block_table[static_cast<int64_t>(entry) * a.bt_width + pi] : -1;
+    if (pg < 0 || pg >= a.src_pages) return nullptr;
+    return kcache + (static_cast<int64_t>(pg) * a.src_page + pos % a.src_page) * a.stored;
+}
+
+// pages: [n][4] = entry, first position, end of the entry's tokens, 0.  A wavefront a row, 16 bytes a lane.
+__global__ __launch_bounds__(256) void latent_gather_kernel(const bf16_t* __restrict__ kcache, const int* __restrict__ block_table,
+                                                            const int* __restrict__ pages, bf16_t* __restrict__ rows,
+                                                            ExpandArgs a) {
+    const int p = blockIdx.x, slot = blockIdx.y * 4 + threadIdx.x / PULSE_WAVE, lane = threadIdx.x % PULSE_WAVE;
+    if (slot >= a.page) return;
+    const int* pg = pages + 4 * p;
+    const bf16_t* src = cached_row(kcache, block_table, pg[0], pg[1] + slot, pg[2], a);
+    uint4* dst = reinterpret_cast<uint4*>(rows + (static_cast<int64_t>(p) * a.page + slot) * a.rank);
+    for (int i = lane; i < a.rank / 8; i += PULSE_WAVE)
+        dst[i] = src ? reinterpret_cast<const uint4*>(src)[i] : make_uint4(0u, 0u, 0u, 0u);
+}
+
+// A workgroup a (page, head): keys as they come, values turned around through LDS.
+__global__ __launch_bounds__(256) void latent_pages_kernel(const bf16_t* __restrict__ kcache, const int* __restrict__ block_table,
+                                                           const int* __restrict__ pages, const bf16_t* __restrict__ up,
+                                                           bf16_t* __restrict__ keys, bf16_t* __restrict__ values,
+                                                           ExpandArgs a) {
+    extern __shared__ bf16_t v_s[];    // [page][dv + 2]
+    const int p = blockIdx.x, h = blockIdx.y;
+    const int* pg = pages + 4 * p;
+    const int64_t up_cols = static_cast<int64_t>(a.heads) * (a.d + a.dv);
+    const bf16_t* rows = up + static_cast<int64_t>(p) * a.page * up_cols;
+    bf16_t* kdst = keys + (static_cast<int64_t>(p) * a.heads + h) * a.page * a.width;
+    for (int i = threadIdx.x; i < a.page * a.width; i += 256) {
+        const int slot = i / a.width, c = i % a.width;
+        bf16_t v = 0;
+        if (c < a.d) v = rows[slot * up_cols + static_cast<int64_t>(h) * a.d + c];
+        else if (c < a.d + a.rot) {
+            const bf16_t* src = cached_row(kcache, block_table, pg[0], pg[1] + slot, pg[2], a);
+            if (src) v = src[a.rank + c - a.d];
+        }
+        kdst[i] = v;
+    }
+    const int pitch = a.dv + 2;
+    for (int i = threadIdx.x; i < a.page * a.dv; i += 256) {
+        const int slot = i / a.dv, c = i % a.dv;
+        v_s[slot * pitch + c] = rows[slot * up_cols + static_cast<int64_t>(a.heads) * a.d + static_cast<int64_t>(h) * a.dv + c];
+    }
+    __syncthreads();
+    bf16_t* vdst = values + (static_cast<int64_t>(p) * a.heads + h) * a.page * a.width;
+    for (int i = threadIdx.x; i < a.page * a.width; i += 256) {
+        const int c = i / a.page, slot = i % a.page;
+        vdst[i] = c < a.dv ? v_s[slot * pitch + c] : static_cast<bf16_t>(0);
+    }
+}
+
+__global__ void latent_compact_kernel(const bf16_t* __restrict__ o, int64_t o_stride, int width, bf16_t* __restrict__ y,
+                                      int64_t y_stride, int dv, int n, float scale) {
+    const int t = blockIdx.x;
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const bf16_t v = o[static_cast<int64_t>(t) * o_stride + static_cast<int64_t>(i / dv) * width + i % dv];
+        y[static_cast<int64_t>(t) * y_stride + i] = scale == 1.f ? v : f32_to_bf16(bf16_to_f32(v) * scale);
     }
 }
 
@@ -199,7 +317,7 @@ __global__ __launch_bounds__(256) void heads_product_kernel(const TX* __restrict
 
 // x [tokens, x_stride]: queries from column q0 (heads x (d + rot), the turned part last); down_x [tokens, down_stride]:
 // the down projection from column c0 (rank + rot; the two may be one matrix; without `write` down_x is not read).  q [tokens, q_stride] receives, for head h at h * stored, the turned
-// part at rank .. rank + rot and zeros behind it (the first rank channels are pulse_latent_absorb's).  With `write`
+// part at rank .. rank + rot and zeros behind it (the first rank channels are pulse_latent_absorb's); null: no queries.  With `write`
 // the token's c and turned key part go to kcache [pages, 1, page, stored] and c to vcache [pages, 1, stored, page].
 extern "C" int pulse_latent_rows(const void* x, int64_t x_stride, int x_dtype, int q0, const void* down_x,
                                  int64_t down_stride, int c0, void* q, int64_t q_stride,
@@ -208,8 +326,8 @@ extern "C" int pulse_latent_rows(const void* x, int64_t x_stride, int x_dtype, i
                                  const int* block_table, int bt_width, int tokens, int heads, int d, int rot, int rank,
                                  int stored, int page_size, int num_pages, float eps, int write, hipStream_t stream) {
     PULSE_REQUIRE(tokens >= 0 && heads > 0 && d >= 0 && rank > 0 && rot > 0 && rot % 2 == 0, "latent_rows: bad sizes");
-    PULSE_REQUIRE(stored >= rank + rot && q_stride >= static_cast<int64_t>(heads) * stored, "latent_rows: stored rows too narrow");
-    PULSE_REQUIRE(x && q && cos_t && sin_t && positions && token_entry && (!write || (down_x && norm_w && kcache && vcache &&
+    PULSE_REQUIRE(stored >= rank + rot && (!q || q_stride >= static_cast<int64_t>(heads) * stored), "latent_rows: stored rows too narrow");
+    PULSE_REQUIRE(x && (q || write) && cos_t && sin_t && positions && token_entry && (!write || (down_x && norm_w && kcache && vcache &&
                   block_table)), "latent_rows: null pointer");
     PULSE_REQUIRE(pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype) && pulse_dtype_ok(c_dtype), "latent_rows: bad dtype tag");
     PULSE_REQUIRE(q0 >= 0 && c0 >= 0 && x_stride >= static_cast<int64_t>(q0) + static_cast<int64_t>(heads) * (d + rot) &&
@@ -297,11 +415,87 @@ extern "C" int pulse_heads_product(const void* x, int64_t x_stride, int x_head, 
     PULSE_REQUIRE(reinterpret_cast<uintptr_t>(x) % 16 == 0 && (x_stride * xb) % 16 == 0 && (static_cast<int64_t>(x_head) * xb) % 16 == 0 &&
                   reinterpret_cast<uintptr_t>(w) % 16 == 0, "heads_product: operands must be 16-byte aligned");
     if (tokens == 0) return 0;
-    const dim3 grid((tokens + 15) / 16, heads);
-    PULSE_DISPATCH_DTYPE(x_dtype, TX,
-        hipLaunchKernelGGL(heads_product_kernel<TX>, grid, dim3(256), 0, stream, static_cast<const TX*>(x), x_stride, x_head,
-                           static_cast<const bf16_t*>(w), static_cast<const bf16_t*>(gate), gate_stride,
-                           static_cast<bf16_t*>(y), y_stride, y_head, tokens, m_out, k_in, scale, gate_heads));
+#define PULSE_HEADS(TT_)                                                                                                 \
+    PULSE_DISPATCH_DTYPE(x_dtype, TX,                                                                                    \
+        hipLaunchKernelGGL((heads_product_kernel<TX, TT_>), dim3((tokens + 16 * TT_ - 1) / (16 * TT_), heads), dim3(256), 0, \
+                           stream, static_cast<const TX*>(x), x_stride, x_head, static_cast<const bf16_t*>(w),           \
+                           static_cast<const bf16_t*>(gate), gate_stride, static_cast<bf16_t*>(y), y_stride, y_head,     \
+                           tokens, m_out, k_in, scale, gate_heads))
+    if (tokens >= 256) PULSE_HEADS(4);
+    else PULSE_HEADS(1);
+#undef PULSE_HEADS
     PULSE_LAUNCH_CHECK("heads_product");
+    return 0;
+}
+
+// x [tokens, x_stride] holds the queries from column q0 (heads x (d + rot)); q [tokens, q_stride] receives heads of `width`
+// channels.
+extern "C" int pulse_latent_queries(const void* x, int64_t x_stride, int x_dtype, int q0, void* q, int64_t q_stride,
+                                    const float* cos_t, const float* sin_t, int pairing, int tokens, int heads, int d, int rot,
+                                    int width, hipStream_t stream) {
+    PULSE_REQUIRE(tokens >= 0 && heads > 0 && d > 0 && rot > 0 && rot % 2 == 0 && width >= d + rot && q0 >= 0, "latent_queries: bad sizes");
+    PULSE_REQUIRE(x && q && cos_t && sin_t && pulse_dtype_ok(x_dtype) && (pairing == 0 || pairing == 1), "latent_queries: bad arguments");
+    PULSE_REQUIRE(x_stride >= q0 + static_cast<int64_t>(heads) * (d + rot) && q_stride >= static_cast<int64_t>(heads) * width,
+                  "latent_queries: the rows are too short");
+    if (tokens == 0) return 0;
+    PULSE_DISPATCH_DTYPE(x_dtype, TX,
+        hipLaunchKernelGGL(latent_queries_kernel<TX>, dim3(tokens), dim3(256), 0, stream, static_cast<const TX*>(x), x_stride, q0,
+                           static_cast<TX*>(q), q_stride, cos_t, sin_t, heads, d, rot, width, pairing));
+    PULSE_LAUNCH_CHECK("latent_queries");
+    return 0;
+}
+
+static int expand_args(ExpandArgs& a, int heads, int d, int rot, int dv, int rank, int stored, int width, int page, int src_page,
+                       int src_pages, int bt_width) {
+    PULSE_REQUIRE(heads > 0 && heads < 65536 && d > 0 && rot > 0 && dv > 0 && rank > 0 && stored >= rank + rot && width >= d + rot &&
+                  width >= dv && page > 0 && src_page > 0 && src_pages > 0 && bt_width > 0, "latent expansion: bad sizes");
+    PULSE_REQUIRE(rank % 8 == 0 && stored % 8 == 0, "latent expansion: rows must keep 16-byte alignment");
+    a.heads = heads; a.d = d; a.rot = rot; a.dv = dv; a.rank = rank; a.stored = stored; a.width = width; a.page = page;
+    a.src_page = src_page; a.src_pages = src_pages; a.bt_width = bt_width;
+    return 0;
+}
+
+// kcache bfloat16 [src_pages, 1, src_page, stored]; pages int32 [n_pages, 4]: entry (row of block_table), first position, end
+// of the entry's tokens, 0.  rows bfloat16 [n_pages * page, rank]; a row that is not cached becomes zeros.
+extern "C" int pulse_latent_gather(const void* kcache, const int* block_table, int bt_width, const int* pages, int n_pages,
+                                   void* rows, int rank, int rot, int stored, int page, int src_page, int src_pages,
+                                   hipStream_t stream) {
+    ExpandArgs a;
+    if (expand_args(a, 1, 1, rot, 1, rank, stored, 1 + rot, page, src_page, src_pages, bt_width)) return 1;
+    PULSE_REQUIRE(kcache && block_table && pages && rows && n_pages >= 0 && reinterpret_cast<uintptr_t>(kcache) % 16 == 0 &&
+                  reinterpret_cast<uintptr_t>(rows) % 16 == 0, "latent_gather: bad arguments");
+    if (n_pages == 0) return 0;
+    hipLaunchKernelGGL(latent_gather_kernel, dim3(n_pages, (page + 3) / 4), dim3(256), 0, stream, static_cast<const bf16_t*>(kcache),
+                       block_table, pages, static_cast<bf16_t*>(rows), a);
+    PULSE_LAUNCH_CHECK("latent_gather");
+    return 0;
+}
+
+// up bfloat16 [n_pages * page, heads * d + heads * dv]: the rows' keys, then values, head by head.
+extern "C" int pulse_latent_pages(const void* kcache, const int* block_table, int bt_width, const int* pages, int n_pages,
+                                  const void* up, void* keys, void* values, int heads, int d, int rot, int dv, int rank,
+                                  int stored, int width, int page, int src_page, int src_pages, hipStream_t stream) {
+    ExpandArgs a;
+    if (expand_args(a, heads, d, rot, dv, rank, stored, width, page, src_page, src_pages, bt_width)) return 1;
+    PULSE_REQUIRE(kcache && block_table && pages && up && keys && values && n_pages >= 0, "latent_pages: bad arguments");
+    const size_t lds = sizeof(bf16_t) * static_cast<size_t>(page) * (dv + 2);
+    PULSE_REQUIRE(lds <= 60 * 1024, "latent_pages: a page of %d values of %d channels does not fit", page, dv);
+    if (n_pages == 0) return 0;
+    hipLaunchKernelGGL(latent_pages_kernel, dim3(n_pages, heads), dim3(256), lds, stream, static_cast<const bf16_t*>(kcache),
+                       block_table, pages, static_cast<const bf16_t*>(up), static_cast<bf16_t*>(keys),
+                       static_cast<bf16_t*>(values), a);
+    PULSE_LAUNCH_CHECK("latent_pages");
+    return 0;
+}
+
+// y[t, h * dv + e] = scale * o[t, h * width + e], bfloat16.
+extern "C" int pulse_latent_compact(const void* o, int64_t o_stride, int width, void* y, int64_t y_stride, int tokens, int heads,
+                                    int dv, float scale, hipStream_t stream) {
+    PULSE_REQUIRE(tokens >= 0 && heads > 0 && dv > 0 && width >= dv && o && y && o_stride >= static_cast<int64_t>(heads) * width &&
+                  y_stride >= static_cast<int64_t>(heads) * dv, "latent_compact: bad arguments");
+    if (tokens == 0) return 0;
+    hipLaunchKernelGGL(latent_compact_kernel, dim3(tokens), dim3(256), 0, stream, static_cast<const bf16_t*>(o), o_stride, width,
+                       static_cast<bf16_t*>(y), y_stride, dv, heads * dv, scale);
+    PULSE_LAUNCH_CHECK("latent_compact");
     return 0;
 }

@@ -686,7 +686,7 @@ def group_norm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], gate: Optio
          _i32(1 if weight is not None and weight.numel() != width else 0), _stream())
 
 
-def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight: Optional[torch.Tensor], cos: torch.Tensor,
+def latent_rows(x: torch.Tensor, q0: int, c0: int, q: Optional[torch.Tensor], norm_weight: Optional[torch.Tensor], cos: torch.Tensor,
                 sin: torch.Tensor, pairing: int, kcache: torch.Tensor, vcache: torch.Tensor, positions: torch.Tensor,
                 token_entry: torch.Tensor, block_table: torch.Tensor, heads: int, d: int, rot: int, rank: int,
                 stored: int, eps: float, write: bool = True, down: Optional[torch.Tensor] = None) -> None:
@@ -694,14 +694,14 @@ def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight:
     (keys [pages, 1, page, stored] = [c | turned | 0], values [pages, 1, stored, page] = [c | 0]) and the queries'
     turned parts into ``q`` [T, heads * stored] at rank .. rank + rot of every head (zeros behind).  The queries are
     columns q0 .. of ``x``, the down projection columns c0 .. of ``down`` (None: of ``x`` too); without ``write`` only the
-    queries are prepared."""
+    queries are prepared, with ``q`` None only the rows are written."""
     down = x if down is None else down
     _need(not write or (norm_weight is not None and down.dtype == x.dtype and down.dim() == 2 and down.stride(1) == 1
                         and down.shape[0] == x.shape[0]), "latent_rows: the down projection must be a matrix of x's type and rows")
     _gpu("latent_rows", x, down, q, norm_weight, cos, sin, kcache, vcache, positions, token_entry, block_table)
     tokens = x.shape[0]
-    _need(x.dim() == 2 and x.stride(1) == 1 and q.dim() == 2 and q.stride(1) == 1 and q.dtype == x.dtype
-          and q.shape[0] == tokens and q.shape[1] >= heads * stored, "latent_rows: x and q must be matrices of one type")
+    _need(x.dim() == 2 and x.stride(1) == 1 and (q is None or (q.dim() == 2 and q.stride(1) == 1 and q.dtype == x.dtype
+          and q.shape[0] == tokens and q.shape[1] >= heads * stored)), "latent_rows: x and q must be matrices of one type")
     pages, page_size = _check_cache("latent_rows", kcache, vcache, 1, stored)
     _int_vec("latent_rows: positions", positions, tokens)
     _int_vec("latent_rows: token_entry", token_entry, tokens)
@@ -713,7 +713,7 @@ def latent_rows(x: torch.Tensor, q0: int, c0: int, q: torch.Tensor, norm_weight:
               f"latent_rows: the tables must be contiguous float32 [{tokens}, {rot // 2}]")
     call("pulse_latent_rows", _ptr(x), _i64(x.stride(0) if tokens > 1 else x.shape[1]), _i32(_tag(x, "latent_rows")),
          _i32(q0), _ptr(down), _i64(down.stride(0) if tokens > 1 else down.shape[1]), _i32(c0), _ptr(q),
-         _i64(q.stride(0) if tokens > 1 else q.shape[1]), _ptr(norm_weight),
+         _i64(0 if q is None else (q.stride(0) if tokens > 1 else q.shape[1])), _ptr(norm_weight),
          _i32(_tag(norm_weight, "latent_rows") if norm_weight is not None else 0), _ptr(cos), _ptr(sin), _i32(pairing), _ptr(kcache), _ptr(vcache),
          _i32(_tag(kcache, "latent_rows")), _ptr(positions), _ptr(token_entry), _ptr(block_table),
          _i32(block_table.shape[1]), _i32(tokens), _i32(heads), _i32(d), _i32(rot), _i32(rank), _i32(stored),
@@ -765,6 +765,85 @@ def latent_expand(o: torch.Tensor, stored: int, w_uv: torch.Tensor, gate: Option
          _i32(_tag(w_uv, "latent_expand")), _ptr(gate), _i64(row(gate) if gate is not None else 0), _ptr(out),
          _i64(row(out)), _i32(_tag(out, "latent_expand")), _i32(tokens), _i32(heads), _i32(dv), _i32(rank), _f32(scale),
          _i32(1 if gate_heads else 0), _stream())
+
+
+EXPANDED_PAGE = 64      # slots of a page of expanded keys and values
+
+
+def latent_expand_pages(numbered, window: int):
+    """The pages of expanded keys and values that long portions need: ``numbered`` = (index in the step, entry) pairs.
+    Returns (flat quadruples entry, first position, end, 0 a page; {index: (number of the first position's page, first of
+    the entry's pages)})."""
+    flat, at = [], {}
+    for index, e in numbered:
+        end = e.start + e.count
+        low = max(0, e.start - window + 1) // EXPANDED_PAGE if window else 0
+        at[index] = (low, len(flat) // 4)
+        for p in range(low, (end + EXPANDED_PAGE - 1) // EXPANDED_PAGE):
+            flat.extend((index, p * EXPANDED_PAGE, end, 0))
+    return flat, at
+
+
+def latent_queries(x: torch.Tensor, q0: int, q: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor, pairing: int, heads: int,
+                   d: int, rot: int, width: int) -> None:
+    """q[t, h * width ..] = the head's plain channels as projected, its turned ones turned, zeros up to ``width``."""
+    _gpu("latent_queries", x, q, cos, sin)
+    tokens = x.shape[0]
+    _need(x.dim() == 2 and x.stride(1) == 1 and q.dim() == 2 and q.stride(1) == 1 and q.dtype == x.dtype and q.shape[0] == tokens
+          and q.shape[1] >= heads * width and x.shape[1] >= q0 + heads * (d + rot), "latent_queries: x or q too narrow")
+    for t in (cos, sin):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (tokens, rot // 2),
+              f"latent_queries: the tables must be contiguous float32 [{tokens}, {rot // 2}]")
+    row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
+    call("pulse_latent_queries", _ptr(x), _i64(row(x)), _i32(_tag(x, "latent_queries")), _i32(q0), _ptr(q), _i64(row(q)), _ptr(cos),
+         _ptr(sin), _i32(pairing), _i32(tokens), _i32(heads), _i32(d), _i32(rot), _i32(width), _stream())
+
+
+def _expand_common(what: str, kcache: torch.Tensor, block_table: torch.Tensor, pages: torch.Tensor, rank: int, rot: int) -> int:
+    _need(kcache.dim() == 4 and kcache.shape[1] == 1 and kcache.is_contiguous() and kcache.dtype == torch.bfloat16
+          and kcache.shape[3] >= rank + rot, f"{what}: cached rows must be bfloat16 [pages, 1, page, >= {rank + rot}]")
+    _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.is_contiguous(),
+          f"{what}: block_table must be contiguous int32 [entries, width]")
+    _need(pages.dtype == torch.int32 and pages.is_contiguous() and pages.numel() % 4 == 0, f"{what}: pages are int32 quadruples")
+    return pages.numel() // 4
+
+
+def latent_gather(kcache: torch.Tensor, block_table: torch.Tensor, pages: torch.Tensor, rows: torch.Tensor, rot: int) -> None:
+    """rows [pages * EXPANDED_PAGE, rank] bfloat16 = the cached latent rows of the listed pages (zeros where none is)."""
+    _gpu("latent_gather", kcache, block_table, pages, rows)
+    rank = rows.shape[1]
+    n = _expand_common("latent_gather", kcache, block_table, pages, rank, rot)
+    _need(rows.dtype == torch.bfloat16 and rows.is_contiguous() and rows.shape[0] == n * EXPANDED_PAGE and rank % 8 == 0,
+          f"latent_gather: rows must be contiguous bfloat16 [{n * EXPANDED_PAGE}, rank], rank a multiple of 8")
+    call("pulse_latent_gather", _ptr(kcache), _ptr(block_table), _i32(block_table.shape[1]), _ptr(pages), _i32(n), _ptr(rows),
+         _i32(rank), _i32(rot), _i32(kcache.shape[3]), _i32(EXPANDED_PAGE), _i32(kcache.shape[2]), _i32(kcache.shape[0]), _stream())
+
+
+def latent_pages(kcache: torch.Tensor, block_table: torch.Tensor, pages: torch.Tensor, up: torch.Tensor, keys: torch.Tensor,
+                 values: torch.Tensor, d: int, rot: int, dv: int, rank: int) -> None:
+    """keys [pages, heads, EXPANDED_PAGE, width] and values [pages, heads, width, EXPANDED_PAGE] from the rows' up
+    projections ``up`` [pages * EXPANDED_PAGE, heads * d + heads * dv] and the cached turned parts; zeros elsewhere."""
+    _gpu("latent_pages", kcache, block_table, pages, up, keys, values)
+    n = _expand_common("latent_pages", kcache, block_table, pages, rank, rot)
+    heads, width = keys.shape[1], keys.shape[3]
+    _need(all(t.dtype == torch.bfloat16 and t.is_contiguous() for t in (up, keys, values))
+          and tuple(up.shape) == (n * EXPANDED_PAGE, heads * (d + dv)) and tuple(keys.shape) == (n, heads, EXPANDED_PAGE, width)
+          and tuple(values.shape) == (n, heads, width, EXPANDED_PAGE) and width >= max(d + rot, dv),
+          "latent_pages: up, keys and values do not fit each other")
+    call("pulse_latent_pages", _ptr(kcache), _ptr(block_table), _i32(block_table.shape[1]), _ptr(pages), _i32(n), _ptr(up),
+         _ptr(keys), _ptr(values), _i32(heads), _i32(d), _i32(rot), _i32(dv), _i32(rank), _i32(kcache.shape[3]), _i32(width),
+         _i32(EXPANDED_PAGE), _i32(kcache.shape[2]), _i32(kcache.shape[0]), _stream())
+
+
+def latent_compact(o: torch.Tensor, width: int, out: torch.Tensor, heads: int, dv: int, scale: float = 1.0) -> None:
+    """out[t, h * dv + e] = scale * o[t, h * width + e], bfloat16; rows may be strided."""
+    _gpu("latent_compact", o, out)
+    tokens = o.shape[0]
+    _need(o.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and o.stride(1) == 1 and out.stride(1) == 1
+          and o.shape[1] >= heads * width and out.shape[0] == tokens and out.shape[1] >= heads * dv, "latent_compact: bad tensors")
+    row = lambda t: t.stride(0) if tokens > 1 else t.shape[1]
+    call("pulse_latent_compact", _ptr(o), _i64(row(o)), _i32(width), _ptr(out), _i64(row(out)), _i32(tokens), _i32(heads), _i32(dv),
+         _f32(scale), _stream())
 
 
 def heads_product_takes(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, x_head: int) -> bool:

@@ -22,20 +22,26 @@ Variations: ``query_dim``: the queries come from a latent of their own, q = W_uq
 them too (0: all of them).  ``reads_rows`` True: the part has no down projection; its run reads the latent rows and turned
 key parts that another run of the order caches (``RunSpec.cache_of``), with its own up projections.
 
+Where the rows are wider than the compiled attention kernels take, long portions of prompts go another way: the rows they
+see are gathered from the pages, expanded to every head's keys and values by one product with [W_uk; W_uv], and the
+prompt-portion kernel of ``attention`` runs on those (``EXPAND_MIN_TOKENS``; a third of the arithmetic at a latent row of
+512 and heads of 128, on a kernel that shares keys through LDS).  What is cached stays the same.
+
 Kernels: ``pulse_latent_rows`` (norm of the latent row, turns, page write), ``pulse_rms_rows``
 (norm of the queries' latent), ``pulse_heads_product`` (bfloat16: both
 products a head on the matrix cores) or ``pulse_latent_absorb`` / ``pulse_latent_expand`` (queries into the latent
-space, values out of it with the gate), and the attention kernels between them.  It answers the
+space, values out of it with the gate), and the attention kernels between them; ``pulse_latent_queries`` / ``gather`` /
+``pages`` / ``compact`` around the expanded form.  It answers the
 protocol of a branch of ``side_by_side``.
 """
 from __future__ import annotations
 
-from typing import Any, Dict
+from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 
 from ..cache.manager import PagedKVSpec
-from ..ops import kernels
+from ..ops import attention_mfma, kernels
 from ..weights.store import TensorSpec
 from .attention import PagedAttention
 from .base import MIXERS, BuildContext, PagedCacheView, Part, StepContext, StepCost, joined
@@ -145,8 +151,10 @@ class LatentAttention(PagedAttention):
         self.q_up = Linear(load.get(n["q_up"]), build.mode) if self.query_dim else None
         self.q_norm_weight = load.get(n["q_down_norm"]) if self.query_dim else None
         self.norm_weight = None if self.reads_rows else load.get(n["down_norm"])
-        self.w_uk = load.get(n["up_k"])
-        self.w_uv = load.get(n["up_v"])
+        up = load.get_concat([n["up_k"], n["up_v"]])
+        self.w_uk, self.w_uv = up[:self.nq * self.plain_dim], up[self.nq * self.plain_dim:]
+        self.up = Linear(up, build.mode)
+        self.expanded = (max(self.plain_dim + self.rot_dim, self.v_dim) + 15) // 16 * 16   # channels of an expanded head
         # for the matrix cores: a head's rows side by side ([heads, out, in]); w_uk transposed once, so that both
         # products walk their inner dimension along a row (a layout choice, not new maths)
         self.w_uk_t = self.w_uv_h = None
@@ -194,32 +202,50 @@ class LatentAttention(PagedAttention):
         if tables.rotary_dim != self.rot_dim:
             raise ValueError(f"latent attention turns {self.rot_dim} channels, its position encoding {tables.rotary_dim}")
         table = ctx.block_tables[cache.group]
-        q = ws.buffer("latent.q", tokens, self.nq * self.d, self.act_dtype)
-        kernels.latent_rows(raw, 0, self.down_col0, q, self.norm_weight, tables.cos, tables.sin, tables.pairing, cache.keys,
-                            cache.values, ctx.positions, ctx.token_entry, table, self.nq, self.plain_dim, self.rot_dim,
-                            self.rank, self.d, self.eps, write=cache.writable, down=y)
+        gate = y[:, self.gate_col0:self.gate_col0 + self.gate_cols] if self.gated else None
+        plan = self._expansion(ctx, cache)
+        runs = plan["others"] if plan is not None else [(0, tokens)]
+        q = ws.buffer("latent.q", tokens, self.nq * self.d, self.act_dtype) if runs else None
+        if runs or cache.writable:
+            kernels.latent_rows(raw, 0, self.down_col0, q, self.norm_weight, tables.cos, tables.sin, tables.pairing,
+                                cache.keys, cache.values, ctx.positions, ctx.token_entry, table, self.nq, self.plain_dim,
+                                self.rot_dim, self.rank, self.d, self.eps, write=cache.writable, down=y)
+        if runs:
+            self._absorbed(raw, q, gate, ctx, cache, table, out, runs, plan)
+        if plan is not None:
+            self._expanded(raw, gate, ctx, cache, table, tables, out, plan)
+
+    def _absorbed(self, raw, q, gate, ctx: StepContext, cache: PagedCacheView, table, out, runs: List[Tuple[int, int]],
+                  plan: Optional[Dict[str, Any]]) -> None:
+        """Attention in the latent space, of the rows in ``runs`` (all of them without a plan)."""
+        ws = ctx.workspace
+        tokens = q.shape[0]
         q_head = self.plain_dim + self.rot_dim
-        if self.w_uk_t is not None and kernels.heads_product_takes(raw, self.w_uk_t, q, q_head):
-            kernels.heads_product(raw, q_head, self.w_uk_t, None, q, self.d)
-        else:
-            kernels.latent_absorb(raw, 0, q_head, self.w_uk, q, self.d, self.nq, self.plain_dim, self.rank)
+        for a, b in runs:
+            if self.w_uk_t is not None and kernels.heads_product_takes(raw[a:b], self.w_uk_t, q[a:b], q_head):
+                kernels.heads_product(raw[a:b], q_head, self.w_uk_t, None, q[a:b], self.d)
+            else:
+                kernels.latent_absorb(raw[a:b], 0, q_head, self.w_uk, q[a:b], self.d, self.nq, self.plain_dim, self.rank)
         window = int(self.window) if self.window is not None else 0
         # the weighted latent rows: from the matrix-core kernels of ``attention`` where they are compiled for rows this
         # wide (the activations' type), else in float32 from the matrix-core kernel for wide values or the generic one
         if self.uses_matrix_cores(q, cache):
             o = ws.buffer("latent.rows", tokens, self.nq * self.d, self.act_dtype)
             self.attend(q, o, ctx, cache, table)
-        elif self.options.get("attention", "auto") != "generic" and kernels.attn_wide_takes(q, cache.keys, self.d):
+        elif self._wide(q, cache):
             o = ws.buffer("latent.rows", tokens, self.nq * self.d, torch.float32)
-            key = f"static:latent.wide_items:{self.nq}"
+            key = f"static:latent.wide_items:{self.nq}:{'some' if plan else 'all'}"
             if key not in ctx.extras:
                 row_tiles = kernels.attn_wide_row_tiles(ctx.num_tokens)
-                flat, hp = kernels.attn_wide_items(ctx.entries, self.nq, 1, row_tiles)
+                entries = [e for i, e in enumerate(ctx.entries) if plan is None or i not in plan["at"]]
+                flat, hp = kernels.attn_wide_items(entries, self.nq, 1, row_tiles)
                 ctx.extras[key] = (ctx.to_device(flat), hp, row_tiles)
             items, hp, row_tiles = ctx.extras[key]
             wv = (self.rank + 15) // 16 * 16
             seen = min(ctx.max_context, window + 32) if window else ctx.max_context
             splits = kernels.attn_wide_splits(items.numel() // 4, (wv + 255) // 256, seen) if row_tiles == 1 else 1
+            if plan is not None:
+                splits = 1     # (the merge of splits covers every row of the step)
             part = part_ml = None
             if splits > 1:
                 part = ws.buffer("attn_wide.part", tokens * self.nq * splits, self.d, torch.float32)
@@ -231,12 +257,91 @@ class LatentAttention(PagedAttention):
             o = ws.buffer("latent.rows", tokens, self.nq * self.d, torch.float32)
             kernels.attn_generic(q, o, self.nq, 1, self.d, cache.keys, cache.values, ctx.positions, ctx.token_entry,
                                  table, self.scale, window, sink=self.sink, softcap=self.score_cap)
-        gate = y[:, self.gate_col0:self.gate_col0 + self.gate_cols] if self.gated else None
-        if self.w_uv_h is not None and kernels.heads_product_takes(o, self.w_uv_h, out, self.d):
-            kernels.heads_product(o, self.d, self.w_uv_h, gate, out, self.v_dim, self.out_scale, self.gate_heads)
-        else:
-            kernels.latent_expand(o, self.d, self.w_uv, gate, out, self.nq, self.v_dim, self.rank, self.out_scale,
-                                  self.gate_heads)
+        for a, b in runs:
+            some = gate[a:b] if gate is not None else None
+            if self.w_uv_h is not None and kernels.heads_product_takes(o[a:b], self.w_uv_h, out[a:b], self.d):
+                kernels.heads_product(o[a:b], self.d, self.w_uv_h, some, out[a:b], self.v_dim, self.out_scale, self.gate_heads)
+            else:
+                kernels.latent_expand(o[a:b], self.d, self.w_uv, some, out[a:b], self.nq, self.v_dim, self.rank, self.out_scale,
+                                      self.gate_heads)
+
+    def _wide(self, q: torch.Tensor, cache: PagedCacheView) -> bool:
+        return self.options.get("attention", "auto") != "generic" and kernels.attn_wide_takes(q, cache.keys, self.d)
+
+    EXPAND_MIN_TOKENS = 64             # portions from here on attend to expanded keys and values
+    EXPAND_MAX_BYTES = 1 << 31         # of the expanded keys of a step, and of its values
+
+    def _expansion(self, ctx: StepContext, cache: PagedCacheView) -> Optional[Dict[str, Any]]:
+        """How this step's long portions attend to expanded keys and values; None: no portion does.  The lists depend on the
+        step's shape and positions; every layer with this window and these sizes shares them."""
+        if not any(e.count >= self.EXPAND_MIN_TOKENS for e in ctx.entries):
+            return None
+        form = self.options.get("latent", "auto")
+        if (form == "absorbed" or self.w_uk_t is None or self.options.get("attention", "auto") == "generic"
+                or not attention_mfma.supported(self.expanded, kernels.EXPANDED_PAGE, self.act_dtype, cache.keys.dtype)):
+            return None
+        if attention_mfma.supported(self.d, cache.page_size, self.act_dtype, cache.keys.dtype):
+            return None      # (narrow rows: the compiled kernels take them as they are)
+        window = int(self.window) if self.window is not None else 0
+        key = f"latent.expansion:{window}:{self.nq}:{self.expanded}"
+        if key not in ctx.extras:
+            ctx.extras[key] = self._plan(ctx, window)
+        return ctx.extras[key]
+
+    def _plan(self, ctx: StepContext, window: int) -> Optional[Dict[str, Any]]:
+        numbered = [(i, e) for i, e in enumerate(ctx.entries) if e.count >= self.EXPAND_MIN_TOKENS]
+        flat, at = kernels.latent_expand_pages(numbered, window)
+        n_pages = len(flat) // 4
+        if 2 * n_pages * self.nq * kernels.EXPANDED_PAGE * self.expanded > self.EXPAND_MAX_BYTES:
+            return None
+        width = max((e.start + e.count + kernels.EXPANDED_PAGE - 1) // kernels.EXPANDED_PAGE for _, e in numbered)
+        rows = [[-1] * width for _ in ctx.entries]
+        for (index, e) in numbered:
+            low, first = at[index]
+            last = (e.start + e.count + kernels.EXPANDED_PAGE - 1) // kernels.EXPANDED_PAGE
+            rows[index][low:last] = range(first, first + last - low)
+        others: List[Tuple[int, int]] = []     # the other entries' rows, neighbours together
+        for i, e in enumerate(ctx.entries):
+            if i in at:
+                continue
+            if others and others[-1][1] == e.first_row:
+                others[-1] = (others[-1][0], e.first_row + e.count)
+            else:
+                others.append((e.first_row, e.first_row + e.count))
+        portion = attention_mfma.portion_tokens(1, self.expanded)
+        split_size, splits = attention_mfma.choose_prefill_splits(numbered, portion, self.nq, 1, self.expanded, window)
+        return {"at": at, "n_pages": n_pages, "pages": ctx.to_device(flat), "others": others,
+                "table": ctx.to_device([p for row in rows for p in row]).view(len(rows), width),
+                "items": ctx.to_device(attention_mfma.build_items(numbered, portion)),
+                "spans": [(e.first_row, e.first_row + e.count) for _, e in numbered], "split_size": split_size, "splits": splits}
+
+    def _expanded(self, raw, gate, ctx: StepContext, cache: PagedCacheView, table, tables, out, plan: Dict[str, Any]) -> None:
+        """Attention of the long portions over keys and values expanded to every head."""
+        ws = ctx.workspace
+        tokens, w, page, n = raw.shape[0], self.expanded, kernels.EXPANDED_PAGE, plan["n_pages"]
+        bf16 = self.act_dtype
+        q = ws.buffer("latent.expanded_q", tokens, self.nq * w, bf16)
+        kernels.latent_queries(raw, 0, q, tables.cos, tables.sin, tables.pairing, self.nq, self.plain_dim, self.rot_dim, w)
+        rows = ws.buffer("latent.gathered", n * page, self.rank, bf16)
+        kernels.latent_gather(cache.keys, table, plan["pages"], rows, self.rot_dim)
+        up = self.up.forward(rows, ws.buffer("latent.up", n * page, self.up.out_features, bf16))
+        keys = ws.buffer("latent.expanded_k", n * self.nq * page, w, bf16).view(n, self.nq, page, w)
+        values = ws.buffer("latent.expanded_v", n * self.nq * w, page, bf16).view(n, self.nq, w, page)
+        kernels.latent_pages(cache.keys, table, plan["pages"], up, keys, values, self.plain_dim, self.rot_dim, self.v_dim, self.rank)
+        direct = w == self.v_dim and self.out_scale == 1.0
+        o = out if direct else ws.buffer("latent.expanded_o", tokens, self.nq * w, bf16)
+        part_o = part_ml = None
+        if plan["splits"] > 1:
+            part_o = ws.buffer("attention.portion_part_o", tokens * self.nq * plan["splits"], w, torch.float32)
+            part_ml = ws.buffer("attention.portion_part_ml", tokens * self.nq * plan["splits"], 2, torch.float32)
+        attention_mfma.attn_prefill(q, o, self.nq, self.nq, w, keys, values, ctx.positions, plan["table"], plan["items"],
+                                    self.scale, int(self.window) if self.window is not None else 0, plan["split_size"],
+                                    plan["splits"], part_o, part_ml, gate=gate,
+                                    gate_width=0 if self.gate_heads else (self.v_dim if gate is not None else 0),
+                                    sink=self.sink, softcap=self.score_cap)
+        if not direct:
+            for a, b in plan["spans"]:
+                kernels.latent_compact(o[a:b], w, out[a:b], self.nq, self.v_dim, self.out_scale)
 
     def forward(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView) -> torch.Tensor:
         if self._o is None:

@@ -696,6 +696,123 @@ def test_a_long_prompt_far_beyond_the_windows(runners, plain, dtype):
     agree(run_alone(runner, ids, [150, 190] + [1] * 60), want, dtype, "decoded tail", fragile, loose=name == "mixed")
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_portions_beside_single_tokens(runners, plain, dtype):
+    """Steps that hold portions of 64 tokens and more (which attend to keys and values expanded to every head, behind
+    windows of 64 and 100 tokens whose pages have gone back to the pool) beside short portions and single tokens of other
+    requests (which attend in the latent space), and a step of two long portions."""
+    from pulse_infer_amd.engine.runner import StepEntry
+
+    name = "wide"
+    vocab = CONFIGS[name]["vocab"]
+    lengths = {"a": 420, "b": 90, "c": 300}
+    ids = {k: token_ids(vocab, n, seed=30 + i) for i, (k, n) in enumerate(lengths.items())}
+    runner = runners(name, dtype, 16, tokens=1024)
+    steps = [{"a": 64, "b": 30}, {"a": 200, "b": 1}, {"b": 1, "a": 63, "c": 70}, {"c": 2, "b": 20, "a": 90}, {"c": 130, "a": 1},
+             {"a": 1, "c": 65, "b": 38}, {"a": 1, "c": 1}, {"c": 32}]
+    fed, got = {k: 0 for k in ids}, {k: [] for k in ids}
+    for k in ids:
+        runner.add_request(k)
+    for step in steps:
+        for k, n in step.items():
+            runner.reserve(k, fed[k] + n)
+        logits = runner.step([StepEntry(k, ids[k][fed[k]:fed[k] + n], list(range(n))) for k, n in step.items()])
+        row = 0
+        for k, n in step.items():
+            got[k].append(logits[row:row + n])
+            fed[k], row = fed[k] + n, row + n
+    assert fed == lengths
+    for k in ids:
+        runner.free_request(k)
+        agree(torch.cat(got[k]), plain(name, ids[k]), dtype, f"request {k}", plain.fragile(name, ids[k]))
+        agree(run_alone(runner, ids[k], [lengths[k]]), plain(name, ids[k]), dtype, f"request {k} whole", plain.fragile(name, ids[k]))
+
+
+@pytest.mark.parametrize("gate_heads", [True, False])
+@pytest.mark.parametrize("heads,d,dr,dv,rank,window", [(4, 64, 32, 64, 256, 0), (4, 64, 32, 64, 256, 70), (3, 16, 8, 24, 264, 33),
+                                                       (2, 128, 64, 128, 512, 64), (2, 96, 16, 112, 232, 1)])
+def test_latent_rows_expanded_to_every_head(heads, d, dr, dv, rank, window, gate_heads):
+    """Long portions over gathered and expanded pages against the plain mixer's attention: portions that start inside a
+    page and beyond the window, whose earlier pages are gone from the block table (and hold NaN), with a key planted just
+    inside the window of one query and another just outside."""
+    from types import SimpleNamespace
+
+    from pulse_infer_amd.ops import attention_mfma as M
+    from pulse_infer_amd.ops import kernels
+    from pulse_infer_amd.parts.latent import latent_stored_width
+
+    dtype, bs, scale = torch.bfloat16, 16, 0.2
+    D, w = latent_stored_width(rank, dr), (max(d + dr, dv) + 15) // 16 * 16
+    lens, counts = [300, 90, 131], [170, 90, 67]
+    up_w, up_ref = stored(rnd(heads * (d + dv), rank, seed=1, scale=rank ** -0.5), dtype)
+    sink = rnd(heads, seed=2)
+    entries = [SimpleNamespace(start=n - c, count=c, first_row=sum(counts[:i])) for i, (n, c) in enumerate(zip(lens, counts))]
+    per = [(n + bs - 1) // bs for n in lens]
+    kc = torch.full((sum(per) + 1, 1, bs, D), float("nan"), dtype=dtype, device=DEV)
+    perm = torch.randperm(sum(per) + 1, generator=torch.Generator().manual_seed(4)).tolist()
+    table = torch.full((3, max(per)), -1, dtype=torch.int32)
+    q, qref = stored(rnd(sum(counts), heads * (d + dr), seed=5), dtype)
+    gate_cols = heads * (1 if gate_heads else dv)
+    gate, gref = stored(rnd(sum(counts), gate_cols, seed=6), dtype)
+    wants, at = [], 0
+    for r, (n, e) in enumerate(zip(lens, entries)):
+        c, cref = stored(rnd(n, rank + dr, seed=10 + r), dtype)
+        if window > 1:     # one query's own direction as a key: seen by it, and by nobody `window` later
+            t = e.start + 40
+            row = qref[e.first_row + 40].view(heads, d + dr)[0]
+            far = torch.cat([up_ref[:d].T @ row[:d], row[d:]]) * 4.0
+            for j in (t - window + 1, t - window):
+                if j >= 0:
+                    c[j], cref[j] = stored(far.float(), dtype)
+        low = max(0, e.start - window + 1) if window else 0
+        for i in range(per[r]):
+            if (i + 1) * bs <= low:
+                continue                     # gone back to the pool
+            page = perm[at + i]
+            table[r, i] = page
+            here = c[i * bs:min(n, (i + 1) * bs)]
+            kc[page, 0, :here.shape[0]] = float("nan")
+            kc[page, 0, :here.shape[0], :rank + dr] = here
+        at += per[r]
+        k_plain = (cref[:, :rank] @ up_ref[:heads * d].T).view(n, heads, d)
+        v = (cref[:, :rank] @ up_ref[heads * d:].T).view(n, heads, dv)
+        mine = qref[e.first_row:e.first_row + e.count].view(e.count, heads, d + dr)
+        scores = torch.stack([mine[:, h, :d] @ k_plain[:, h].T + mine[:, h, d:] @ cref[:, rank:].T for h in range(heads)]) * scale
+        full = torch.full((heads, n, n), 0.0, dtype=F64)
+        full[:, e.start:] = scores
+        a = P.softmax_weights(full, P.visible(n, window or None), sink.to(F64))[:, e.start:]
+        o = torch.stack([a[h] @ v[:, h] for h in range(heads)], dim=1)
+        g = torch.sigmoid(gref[e.first_row:e.first_row + e.count]).view(e.count, heads, -1)
+        wants.append((o * g).reshape(e.count, heads * dv))
+    numbered = list(enumerate(entries))
+    flat, where = kernels.latent_expand_pages(numbered, window)
+    n_pages, page = len(flat) // 4, kernels.EXPANDED_PAGE
+    rows = torch.full((n_pages * page, rank), float("nan"), dtype=dtype, device=DEV)
+    kernels.latent_gather(kc, table.to(DEV), ints(flat), rows, dr)
+    assert torch.isfinite(rows).all()
+    up = (rows.float() @ up_w.float().t()).to(dtype)
+    keys = torch.full((n_pages, heads, page, w), float("nan"), dtype=dtype, device=DEV)
+    values = torch.full((n_pages, heads, w, page), float("nan"), dtype=dtype, device=DEV)
+    kernels.latent_pages(kc, table.to(DEV), ints(flat), up, keys, values, d, dr, dv, rank)
+    assert torch.isfinite(keys).all() and torch.isfinite(values).all()
+    wide_table = torch.full((3, max((n + page - 1) // page for n in lens)), -1, dtype=torch.int32)
+    for r, e in numbered:
+        low, first = where[r]
+        last = (lens[r] + page - 1) // page
+        wide_table[r, low:last] = torch.arange(first, first + last - low, dtype=torch.int32)
+    positions = [p for e in entries for p in range(e.start, e.start + e.count)]
+    cos, sin = torch.ones(len(positions), dr // 2, device=DEV), torch.zeros(len(positions), dr // 2, device=DEV)
+    qx = torch.full((len(positions), heads * w), float("nan"), dtype=dtype, device=DEV)
+    kernels.latent_queries(q, 0, qx, cos, sin, 1, heads, d, dr, w)
+    o = torch.full((len(positions), heads * w), float("nan"), dtype=dtype, device=DEV)
+    items = ints(M.build_items(numbered, M.portion_tokens(1, w)))
+    M.attn_prefill(qx, o, heads, heads, w, keys, values, ints(positions), wide_table.to(DEV), items, scale, window, gate=gate,
+                   gate_width=0 if gate_heads else dv, sink=sink.to(DEV))
+    out = torch.full((len(positions), heads * dv), float("nan"), dtype=dtype, device=DEV)
+    kernels.latent_compact(o, w, out, heads, dv)
+    near(out, torch.cat(wants), dtype)
+
+
 # ------------------------------------------------------------------------------------ seeded random configurations
 def random_config(rng):
     """Layers drawn one by one, in any order: head sizes that are no multiples of 16 or of 4, keys wider or narrower than
