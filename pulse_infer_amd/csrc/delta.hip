@@ -15,6 +15,7 @@
 // pulse_delta_prepare: convolutions, unit vectors, decays and strengths of a step's tokens, in float32 rows; a second
 //                      launch moves the ring on.
 // pulse_delta_walk:    the recurrence over prepared rows, token by token, entry by entry (portions, mixed batches).
+// pulse_delta_chunks:  the recurrence over prepared rows of long portions, 64 tokens at a time on the matrix cores (float32).
 // pulse_delta_decode:  a step of single tokens in one launch: convolution, ring, recurrence, the norm of every head's
 //                      result and its gate.
 // State, unit vectors, decays, strengths and all sums are float32 whatever the storage type of the rows.
@@ -143,7 +144,8 @@ __global__ __launch_bounds__(WALK_THREADS) void delta_walk_kernel(const float* _
                                                                   float* __restrict__ out, float* __restrict__ state,
                                                                   const int* __restrict__ entry_first_row,
                                                                   const int* __restrict__ entry_start,
-                                                                  const int* __restrict__ entry_slot, DeltaArgs a) {
+                                                                  const int* __restrict__ entry_slot,
+                                                                  const int* __restrict__ which, DeltaArgs a) {
     constexpr int TB = WALK_TOKENS;
     constexpr int CW = PULSE_WAVE / R, WC = 4 * CW, DR = D / R;
     constexpr int EQ = TB * D / WALK_THREADS, EV = TB * WC / WALK_THREADS;
@@ -153,7 +155,7 @@ __global__ __launch_bounds__(WALK_THREADS) void delta_walk_kernel(const float* _
     __shared__ __attribute__((aligned(16))) float k_s[TB][DP];
     __shared__ float v_s[TB][WC];
     __shared__ float gb_s[TB][2];
-    const int e = blockIdx.x, h = blockIdx.y;
+    const int e = which ? which[blockIdx.x] : blockIdx.x, h = blockIdx.y;
     const int tid = threadIdx.x, lane = tid % PULSE_WAVE, wave = tid / PULSE_WAVE;
     const int rg = lane % R, cl = lane / R;
     const int c = blockIdx.z * WC + wave * CW + cl;
@@ -254,6 +256,247 @@ __global__ __launch_bounds__(WALK_THREADS) void delta_walk_kernel(const float* _
         for (int j = 0; j < DR; ++j) {
             const int i = rg + R * j;
             if (i < a.d) S[static_cast<int64_t>(i) * a.dv + c] = s[j];
+        }
+    }
+}
+
+// ------------------------------------------------------------------ 64 tokens at a time
+// With G_i the sum of the logarithms of the decays of a chunk's tokens up to i and S the state before the chunk:
+//     u_i = beta_i v_i - beta_i e^(G_i) S^T k_i - sum_(j < i) A_ij u_j,      A_ij = beta_i e^(G_i - G_j) k_i . k_j
+// so U = Y - W S with (I + A) [Y | W] = [diag(beta) V | diag(beta e^G) K], a forward substitution that does not know S, and
+//     O = diag(e^G) Q S + P U,  P_ij = e^(G_i - G_j) q_i . k_j  (j <= i),      S <- e^(G_last) S + (diag(e^(G_last - G)) K)^T U.
+// A first kernel does what needs no state, a workgroup a (chunk, head), all chunks at the same time; a second one goes
+// through an entry's chunks in order, a workgroup a (entry, head, 16 columns of the state): three products of float32
+// matrix instructions a chunk.  No exponent is ever positive, so nothing overflows whatever the decays.
+constexpr int CHUNK = 64;
+typedef __attribute__((ext_vector_type(4))) float f32x4;
+
+// What the first kernel leaves for a (chunk, head), in floats from its place in the scratch (D: d rounded up):
+// W [64, D], e^G Q [64, D], (e^(G_last - G) K)^T [D, 64], P [64, 64], Y [64, dvp], e^(G_last).
+__host__ __device__ inline int64_t chunk_floats(int D, int dvp) { return CHUNK * (3ll * D + CHUNK + dvp) + 4; }
+
+__device__ __forceinline__ f32x4 load4(const float* p, bool ok) {
+    return ok ? *reinterpret_cast<const f32x4*>(p) : f32x4{0.f, 0.f, 0.f, 0.f};
+}
+
+template <int D>
+__global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const float* __restrict__ rows, const float* __restrict__ gates,
+                                                                  const int* __restrict__ chunks, float* __restrict__ scratch,
+                                                                  int dvp, DeltaArgs a) {
+    __shared__ __attribute__((aligned(16))) float A_s[CHUNK][CHUNK + 4];
+    __shared__ float G_s[CHUNK], beta_s[CHUNK], front_s[CHUNK], left_s[CHUNK];   // beta e^G, e^(G_last - G)
+    const int h = blockIdx.y, tid = threadIdx.x, lane = tid % PULSE_WAVE, wave = tid / PULSE_WAVE;
+    const int row0 = chunks[4 * blockIdx.x], n = chunks[4 * blockIdx.x + 1];
+    float* item = scratch + (static_cast<int64_t>(blockIdx.x) * a.heads + h) * chunk_floats(D, dvp);
+    float* W = item;
+    float* Qs = W + CHUNK * D;
+    float* KdT = Qs + CHUNK * D;
+    float* P = KdT + CHUNK * D;
+    float* Y = P + CHUNK * CHUNK;
+    const int grp = h / (a.heads / a.groups);
+    const int q0 = grp * a.d, k0 = (a.groups + grp) * a.d, v0 = 2 * a.groups * a.d + h * a.dv;
+    if (wave == 0) {
+        const float* gt = gates + static_cast<int64_t>(row0 + lane) * 2 * a.heads + h;
+        float g = lane < n ? gt[0] : 0.f;
+        const float beta = lane < n ? gt[a.heads] : 0.f;
+#pragma unroll
+        for (int off = 1; off < PULSE_WAVE; off <<= 1) {
+            const float up = __shfl_up(g, off, PULSE_WAVE);
+            if (lane >= off) g += up;
+        }
+        const float last = __shfl(g, PULSE_WAVE - 1, PULSE_WAVE);
+        G_s[lane] = g;
+        beta_s[lane] = beta;
+        front_s[lane] = beta * expf(g);
+        left_s[lane] = expf(last - g);
+        if (lane == 0) Y[CHUNK * dvp] = expf(last);
+    }
+    __syncthreads();
+    const int m = lane % 16, kq = lane / 16;
+    {
+        const int i = 16 * wave + m;
+        const float* row = rows + static_cast<int64_t>(row0 + i) * a.channels;
+        f32x4 ka[D / 16], qa[D / 16];
+        const float eg = expf(G_s[i]);
+#pragma unroll
+        for (int b = 0; b < D / 16; ++b) {
+            const int c = 16 * b + 4 * kq;
+            ka[b] = load4(row + k0 + c, i < n && c < a.d);
+            qa[b] = load4(row + q0 + c, i < n && c < a.d);
+            *reinterpret_cast<f32x4*>(Qs + i * D + c) = qa[b] * eg;
+        }
+        for (int jt = 0; jt <= wave; ++jt) {
+            const int j = 16 * jt + m;
+            const float* rj = rows + static_cast<int64_t>(row0 + j) * a.channels;
+            f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int b = 0; b < D / 16; ++b) {
+                const int c = 16 * b + 4 * kq;
+                const f32x4 kb = load4(rj + k0 + c, j < n && c < a.d);
+#pragma unroll
+                for (int u = 0; u < 4; ++u) {
+                    kk = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[b][u], kb[u], kk, 0, 0, 0);
+                    qk = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[b][u], kb[u], qk, 0, 0, 0);
+                }
+            }
+            // lane: rows 16 wave + 4 kq + u, column j
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int r = 16 * wave + 4 * kq + u;
+                const float e = j <= r ? expf(G_s[r] - G_s[j]) : 0.f;
+                A_s[r][j] = j < r ? beta_s[r] * e * kk[u] : 0.f;
+                P[r * CHUNK + j] = e * qk[u];
+            }
+        }
+    }
+    __syncthreads();
+    // forward substitution, a thread a column of [W | Y]
+    for (int col = tid; col < D + dvp; col += 256) {
+        const bool key = col < D;
+        const int c = key ? col : col - D;
+        const bool there = key ? c < a.d : c < a.dv;
+        const float* src = rows + static_cast<int64_t>(row0) * a.channels + (key ? k0 : v0) + c;
+        float x[CHUNK];
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) x[i] = (there && i < n) ? src[static_cast<int64_t>(i) * a.channels] : 0.f;
+        if (key) {
+#pragma unroll
+            for (int b = 0; b < CHUNK / 4; ++b) {
+                f32x4 t;
+#pragma unroll
+                for (int u = 0; u < 4; ++u) t[u] = x[4 * b + u] * left_s[4 * b + u];
+                *reinterpret_cast<f32x4*>(KdT + c * CHUNK + 4 * b) = t;
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) {
+            float s[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int b = 0; b < (i + 3) / 4; ++b) {
+                const f32x4 ar = *reinterpret_cast<const f32x4*>(&A_s[i][4 * b]);
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+                    if (4 * b + u < i) s[u] = fmaf(ar[u], x[4 * b + u], s[u]);
+            }
+            const float f = key ? front_s[i] : beta_s[i];
+            x[i] = f * x[i] - ((s[0] + s[1]) + (s[2] + s[3]));
+            asm volatile("" ::: "memory");   // (rows of A are read when their turn comes: all at once they need 500 registers)
+        }
+        float* dst = key ? W + c : Y + c;
+        const int pitch = key ? D : dvp;
+#pragma unroll
+        for (int i = 0; i < CHUNK; ++i) dst[i * pitch] = x[i];
+    }
+}
+
+template <int D>
+__global__ __launch_bounds__(256) void delta_chunk_walk_kernel(const float* __restrict__ scratch, const int* __restrict__ chunks,
+                                                               const int* __restrict__ runs, float* __restrict__ out,
+                                                               float* __restrict__ state, const int* __restrict__ entry_start,
+                                                               const int* __restrict__ entry_slot, int dvp, DeltaArgs a) {
+    constexpr int B = D / 16;                         // 16-channel tiles of the state
+    constexpr int TW = B >= 4 ? B / 4 : 1;            // of which a wavefront keeps
+    __shared__ __attribute__((aligned(16))) float S_s[16][D + 4];       // [column][channel]
+    __shared__ __attribute__((aligned(16))) float U_s[16][CHUNK + 4];   // [column][token]
+    const int e = runs[4 * blockIdx.x], first = runs[4 * blockIdx.x + 1], count = runs[4 * blockIdx.x + 2];
+    const int h = blockIdx.y, c0 = 16 * blockIdx.z;
+    const int lane = threadIdx.x % PULSE_WAVE, wave = threadIdx.x / PULSE_WAVE;
+    const int m = lane % 16, kq = lane / 16;
+    const int64_t size = chunk_floats(D, dvp);
+    float* S = state + static_cast<int64_t>(entry_slot[e]) * a.slot_stride + static_cast<int64_t>(h) * a.d * a.dv;
+    const bool fresh = entry_start[e] == 0;
+    // lane: columns c0 + 4 kq + u, channel 16 tile + m
+    f32x4 acc[TW];
+#pragma unroll
+    for (int t = 0; t < TW; ++t) {
+        const int ch = 16 * (wave * TW + t) + m;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int c = c0 + 4 * kq + u;
+            acc[t][u] = (!fresh && ch < a.d && c < a.dv) ? S[static_cast<int64_t>(ch) * a.dv + c] : 0.f;
+            if (wave * TW + t < B) S_s[4 * kq + u][ch] = acc[t][u];
+        }
+    }
+    f32x4 wv[B], qv[B], pv[4], kd[TW][4];
+    float yv[4], el = 1.f;
+    auto item_of = [&](int i) { return scratch + (static_cast<int64_t>(first + i) * a.heads + h) * size; };
+    auto load_wq = [&](int i) __attribute__((always_inline)) {
+        const float* W = item_of(i) + (16 * wave + m) * D + 4 * kq;
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            wv[b] = *reinterpret_cast<const f32x4*>(W + 16 * b);
+            qv[b] = *reinterpret_cast<const f32x4*>(W + CHUNK * D + 16 * b);
+        }
+    };
+    auto load_rest = [&](int i) __attribute__((always_inline)) {
+        const float* KdT = item_of(i) + 2 * CHUNK * D;
+        const float* P = KdT + CHUNK * D;
+        const float* Y = P + CHUNK * CHUNK;
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            pv[b] = load4(P + (16 * wave + m) * CHUNK + 16 * b + 4 * kq, b <= wave);
+#pragma unroll
+            for (int t = 0; t < TW; ++t)
+                kd[t][b] = load4(KdT + (16 * (wave * TW + t) + m) * CHUNK + 16 * b + 4 * kq, wave * TW + t < B);
+            yv[b] = Y[(16 * wave + 4 * kq + b) * dvp + c0 + m];
+        }
+        el = Y[CHUNK * dvp];
+    };
+    load_wq(0);
+    load_rest(0);
+    for (int i = 0; i < count; ++i) {
+        const int row0 = chunks[4 * (first + i)], n = chunks[4 * (first + i) + 1];
+        __syncthreads();     // S_s is whole, U_s has been read
+        f32x4 us = {0.f, 0.f, 0.f, 0.f}, os = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            const f32x4 sb = *reinterpret_cast<const f32x4*>(&S_s[m][16 * b + 4 * kq]);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                us = __builtin_amdgcn_mfma_f32_16x16x4f32(wv[b][u], sb[u], us, 0, 0, 0);
+                os = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[b][u], sb[u], os, 0, 0, 0);
+            }
+        }
+        if (i + 1 < count) load_wq(i + 1);
+        f32x4 uv;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) uv[u] = yv[u] - us[u];
+        *reinterpret_cast<f32x4*>(&U_s[m][16 * wave + 4 * kq]) = uv;
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < TW; ++t) acc[t] *= el;
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            const f32x4 ub = *reinterpret_cast<const f32x4*>(&U_s[m][16 * b + 4 * kq]);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                if (b <= wave) os = __builtin_amdgcn_mfma_f32_16x16x4f32(pv[b][u], ub[u], os, 0, 0, 0);
+#pragma unroll
+                for (int t = 0; t < TW; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ub[u], kd[t][b][u], acc[t], 0, 0, 0);
+            }
+        }
+        if (i + 1 < count) load_rest(i + 1);
+#pragma unroll
+        for (int t = 0; t < TW; ++t)
+            if (wave * TW + t < B) {
+#pragma unroll
+                for (int u = 0; u < 4; ++u) S_s[4 * kq + u][16 * (wave * TW + t) + m] = acc[t][u];
+            }
+        if (c0 + m < a.dv) {
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int r = 16 * wave + 4 * kq + u;
+                if (r < n) out[static_cast<int64_t>(row0 + r) * a.heads * a.dv + h * a.dv + c0 + m] = os[u];
+            }
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < TW; ++t) {
+        const int ch = 16 * (wave * TW + t) + m;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int c = c0 + 4 * kq + u;
+            if (wave * TW + t < B && ch < a.d && c < a.dv) S[static_cast<int64_t>(ch) * a.dv + c] = acc[t][u];
         }
     }
 }
@@ -426,11 +669,12 @@ extern "C" int pulse_delta_prepare(const void* x, int x_dtype, int64_t x_stride,
     return 0;
 }
 
-// row_groups: over how many lanes a column's rows are shared out (4, or 16 from 64 key channels a head on).
+// row_groups: over how many lanes a column's rows are shared out (4, or 16 from 64 key channels a head on).  which: the
+// `entries` entries that are walked (null: entries 0, 1, ...).
 extern "C" int pulse_delta_walk(const float* rows, const float* gates, float* out, float* state, int slots,
                                 int64_t slot_stride, const int* entry_first_row, const int* entry_start,
-                                const int* entry_slot, int entries, int heads, int groups, int d, int dv, int n_taps,
-                                int row_groups, hipStream_t stream) {
+                                const int* entry_slot, const int* which, int entries, int heads, int groups, int d, int dv,
+                                int n_taps, int row_groups, hipStream_t stream) {
     PULSE_REQUIRE(entries >= 0 && slots > 0 && heads < 65536 && dv < 65536 * 4, "delta_walk: bad sizes");
     PULSE_REQUIRE(rows && gates && out && state && entry_first_row && entry_start && entry_slot, "delta_walk: null pointer");
     DeltaArgs a;
@@ -438,7 +682,7 @@ extern "C" int pulse_delta_walk(const float* rows, const float* gates, float* ou
     if (entries == 0) return 0;
 #define PULSE_WALK(D_, R_)                                                                                              \
     hipLaunchKernelGGL((delta_walk_kernel<D_, R_>), dim3(entries, heads, (dv * R_ + 255) / 256), dim3(WALK_THREADS), 0,  \
-                       stream, rows, gates, out, state, entry_first_row, entry_start, entry_slot, a)
+                       stream, rows, gates, out, state, entry_first_row, entry_start, entry_slot, which, a)
     if (d <= 16) PULSE_WALK(16, 4);
     else if (d <= 32) PULSE_WALK(32, 4);
     else if (d <= 64) { if (row_groups >= 16) PULSE_WALK(64, 16); else PULSE_WALK(64, 4); }
@@ -446,6 +690,45 @@ extern "C" int pulse_delta_walk(const float* rows, const float* gates, float* ou
     else { if (row_groups >= 16) PULSE_WALK(256, 16); else PULSE_WALK(256, 4); }
 #undef PULSE_WALK
     PULSE_LAUNCH_CHECK("delta_walk");
+    return 0;
+}
+
+static int chunk_channels(int d) { return d <= 32 ? 32 : (d <= 64 ? 64 : 128); }
+
+// Whether pulse_delta_chunks takes heads of these sizes.
+extern "C" int pulse_delta_chunks_takes(int d, int dv) { return d >= 4 && d <= 128 && d % 4 == 0 && dv >= 4 && dv % 4 == 0; }
+
+// Float32 values of scratch that one chunk of one head needs.
+extern "C" int64_t pulse_delta_chunk_floats(int d, int dv) { return chunk_floats(chunk_channels(d), (dv + 15) / 16 * 16); }
+
+// chunks int32 [n_chunks, 4]: first row, tokens (1 to 64), 0, 0, an entry's chunks in order and next to each other; runs int32
+// [n_runs, 4]: entry, its first chunk, its number of chunks, 0.  scratch float32 [n_chunks, heads, pulse_delta_chunk_floats].
+extern "C" int pulse_delta_chunks(const float* rows, const float* gates, float* out, float* state, int slots, int64_t slot_stride,
+                                  const int* entry_start, const int* entry_slot, const int* chunks, int n_chunks,
+                                  const int* runs, int n_runs, float* scratch, int heads, int groups, int d, int dv, int n_taps,
+                                  hipStream_t stream) {
+    PULSE_REQUIRE(n_chunks >= 0 && n_runs >= 0 && slots > 0 && heads < 65536, "delta_chunks: bad sizes");
+    PULSE_REQUIRE(rows && gates && out && state && entry_start && entry_slot && chunks && runs && scratch, "delta_chunks: null pointer");
+    PULSE_REQUIRE(pulse_delta_chunks_takes(d, dv), "delta_chunks: heads of %d x %d are not a size it takes", d, dv);
+    DeltaArgs a;
+    if (fill_args(a, heads, groups, d, dv, n_taps, 0, 0, 0, 0, slot_stride)) return 1;
+    PULSE_REQUIRE(reinterpret_cast<uintptr_t>(rows) % 16 == 0 && reinterpret_cast<uintptr_t>(scratch) % 16 == 0,
+                  "delta_chunks: rows and scratch must be 16-byte aligned");
+    if (n_chunks == 0 || n_runs == 0) return 0;
+    const int dvp = (dv + 15) / 16 * 16;
+#define PULSE_CHUNKS(D_)                                                                                                \
+    do {                                                                                                                \
+        hipLaunchKernelGGL((delta_chunk_prepare_kernel<D_>), dim3(n_chunks, heads), dim3(256), 0, stream, rows, gates,  \
+                           chunks, scratch, dvp, a);                                                                    \
+        PULSE_LAUNCH_CHECK("delta_chunks (prepare)");                                                                   \
+        hipLaunchKernelGGL((delta_chunk_walk_kernel<D_>), dim3(n_runs, heads, dvp / 16), dim3(256), 0, stream, scratch, \
+                           chunks, runs, out, state, entry_start, entry_slot, dvp, a);                                  \
+    } while (0)
+    if (d <= 32) PULSE_CHUNKS(32);
+    else if (d <= 64) PULSE_CHUNKS(64);
+    else PULSE_CHUNKS(128);
+#undef PULSE_CHUNKS
+    PULSE_LAUNCH_CHECK("delta_chunks");
     return 0;
 }
 

@@ -1353,11 +1353,13 @@ def delta_row_groups(entries: int, heads: int, d: int, dv: int) -> int:
 
 def delta_walk(rows: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, state: torch.Tensor, entry_first_row: torch.Tensor,
                entry_start: torch.Tensor, entry_slot: torch.Tensor, heads: int, groups: int, d: int, dv: int,
-               n_taps: int, row_groups: int) -> None:
-    """For every entry, token by token over prepared rows: S <- e^g S, u = beta (v - S^T k), S <- S + k u^T, out = S^T q, per
+               n_taps: int, row_groups: int, which: Optional[torch.Tensor] = None) -> None:
+    """For every entry (or those whose numbers ``which`` lists, int32), token by token over prepared rows: S <- e^g S, u = beta (v - S^T k), S <- S + k u^T, out = S^T q, per
     head, in float32; S is the front of the entry's slot, zero when the entry starts at position 0."""
-    _gpu("delta_walk", rows, gates, out, state, entry_first_row, entry_start, entry_slot)
+    _gpu("delta_walk", rows, gates, out, state, entry_first_row, entry_start, entry_slot, which)
     tokens, entries = rows.shape[0], entry_start.numel()
+    if which is not None:
+        _int_vec("delta_walk: which", which)
     channels = 2 * groups * d + heads * dv
     _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2
           and state.shape[1] >= delta_slot_floats(heads, groups, d, dv, n_taps), "delta_walk: the slots are too small")
@@ -1368,8 +1370,61 @@ def delta_walk(rows: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, state
                        ("entry_slot", entry_slot, entries)):
         _int_vec(f"delta_walk: {name}", t, n)
     call("pulse_delta_walk", _ptr(rows), _ptr(gates), _ptr(out), _ptr(state), _i32(state.shape[0]), _i64(state.shape[1]),
-         _ptr(entry_first_row), _ptr(entry_start), _ptr(entry_slot), _i32(entries), _i32(heads), _i32(groups), _i32(d), _i32(dv),
-         _i32(n_taps), _i32(row_groups), _stream())
+         _ptr(entry_first_row), _ptr(entry_start), _ptr(entry_slot), _ptr(which),
+         _i32(entries if which is None else which.numel()), _i32(heads), _i32(groups), _i32(d), _i32(dv), _i32(n_taps),
+         _i32(row_groups), _stream())
+
+
+DELTA_CHUNK = 64
+
+
+def delta_chunks_takes(d: int, dv: int) -> bool:
+    """Whether ``delta_chunks`` takes heads of these sizes (as pulse_delta_chunks_takes)."""
+    return 4 <= d <= 128 and d % 4 == 0 and dv >= 4 and dv % 4 == 0
+
+
+def delta_chunk_floats(d: int, dv: int) -> int:
+    """Float32 values of scratch a (chunk, head) of ``delta_chunks``."""
+    channels, columns = (32 if d <= 32 else 64 if d <= 64 else 128), (dv + 15) // 16 * 16
+    return DELTA_CHUNK * (3 * channels + DELTA_CHUNK + columns) + 4
+
+
+def delta_chunk_lists(entries, min_tokens: int):
+    """(chunks, runs, the other entries' numbers) for a step: entries of at least ``min_tokens`` tokens are cut into chunks
+    (flat quadruples first row, tokens, 0, 0; runs: entry, first chunk, chunks, 0)."""
+    chunks, runs, others = [], [], []
+    for index, e in enumerate(entries):
+        if e.count < min_tokens:
+            others.append(index)
+            continue
+        first = len(chunks) // 4
+        for at in range(0, e.count, DELTA_CHUNK):
+            chunks.extend((e.first_row + at, min(DELTA_CHUNK, e.count - at), 0, 0))
+        runs.extend((index, first, len(chunks) // 4 - first, 0))
+    return chunks, runs, others
+
+
+def delta_chunks(rows: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, state: torch.Tensor, entry_start: torch.Tensor,
+                 entry_slot: torch.Tensor, chunks: torch.Tensor, runs: torch.Tensor, scratch: torch.Tensor, heads: int,
+                 groups: int, d: int, dv: int, n_taps: int) -> None:
+    """``delta_walk`` of the entries in ``runs``, 64 tokens at a time on the matrix cores (float32 throughout)."""
+    _gpu("delta_chunks", rows, gates, out, state, entry_start, entry_slot, chunks, runs, scratch)
+    tokens = rows.shape[0]
+    channels = 2 * groups * d + heads * dv
+    _need(delta_chunks_takes(d, dv), f"delta_chunks: heads of {d} x {dv} are not a size it takes")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and state.dim() == 2
+          and state.shape[1] >= delta_slot_floats(heads, groups, d, dv, n_taps), "delta_chunks: the slots are too small")
+    _need(all(t.dtype == torch.float32 and t.is_contiguous() for t in (rows, gates, out, scratch)) and tuple(rows.shape) == (tokens, channels)
+          and tuple(gates.shape) == (tokens, 2 * heads) and tuple(out.shape) == (tokens, heads * dv),
+          f"delta_chunks: float32 rows [T, {channels}], gates [T, {2 * heads}] and out [T, {heads * dv}] are needed")
+    for name, t in (("entry_start", entry_start), ("entry_slot", entry_slot), ("chunks", chunks), ("runs", runs)):
+        _int_vec(f"delta_chunks: {name}", t)
+    n_chunks, n_runs = chunks.numel() // 4, runs.numel() // 4
+    _need(chunks.numel() == 4 * n_chunks and runs.numel() == 4 * n_runs
+          and scratch.numel() >= n_chunks * heads * delta_chunk_floats(d, dv), "delta_chunks: bad lists or too little scratch")
+    call("pulse_delta_chunks", _ptr(rows), _ptr(gates), _ptr(out), _ptr(state), _i32(state.shape[0]), _i64(state.shape[1]),
+         _ptr(entry_start), _ptr(entry_slot), _ptr(chunks), _i32(n_chunks), _ptr(runs), _i32(n_runs), _ptr(scratch), _i32(heads),
+         _i32(groups), _i32(d), _i32(dv), _i32(n_taps), _stream())
 
 
 def delta_decode_takes(d: int, dv: int) -> bool:

@@ -13,7 +13,8 @@ silu(Wg x); the heads side by side are projected by Wo.
 
 The six input projections are one product with the row-stacked weight.  A step of single tokens runs everything between
 that product and the output projection in one kernel; other steps prepare float32 rows (convolutions, unit vectors,
-decays), run the recurrence over them and norm and gate the heads (``csrc/delta.hip``).  A request's slot holds one
+decays), run the recurrence over them (portions of 64 tokens and more in chunks on the matrix cores, in float32; the
+others token by token) and norm and gate the heads (``csrc/delta.hip``).  A request's slot holds one
 float32 row: the states and the last ``conv`` inputs of the convolutions, which are kept as projected.
 
 Parameters: ``hidden_size``, ``num_heads``, ``num_groups``, ``head_dim``, ``value_dim``, ``conv``, ``norm_eps``, ``names``
@@ -110,10 +111,12 @@ class GatedDelta(Part):
         self._o = None
         self.mode = build.mode
         self.act_dtype = build.act_dtype
-        self.options = build.options
         self.inner_width = self.heads * self.dv
-        self.decodes = kernels.delta_decode_takes(self.d, self.dv)
+        walk_only = build.options.get("delta", "auto") == "walk"
+        self.decodes = not walk_only and kernels.delta_decode_takes(self.d, self.dv)
+        self.chunked = not walk_only and kernels.delta_chunks_takes(self.d, self.dv)
 
+    CHUNKED_MIN_TOKENS = 64  # portions from here on go through the recurrence in chunks
     records_cleanly = True   # slots, starts, positions and rows are read on the device
 
     def cache_spec(self) -> StateSpec:
@@ -131,7 +134,7 @@ class GatedDelta(Part):
         self.proj.forward(x, y)
         if "static:delta.single_tokens" not in ctx.extras:
             ctx.extras["static:delta.single_tokens"] = all(e.count == 1 for e in ctx.entries)
-        if self.decodes and ctx.extras["static:delta.single_tokens"] and self.options.get("delta", "auto") != "walk":
+        if self.decodes and ctx.extras["static:delta.single_tokens"]:
             kernels.delta_decode(y, self.gate0, self.beta0, self.decay0, self.conv, self.a_log, self.dt_bias,
                                  self.norm_weight, cache.state, out, ctx.positions, ctx.token_entry, ctx.entry_slot,
                                  self.heads, self.groups, self.d, self.dv, self.eps, self.out_scale)
@@ -142,9 +145,25 @@ class GatedDelta(Part):
                               ctx.positions, ctx.token_entry, ctx.entry_start, ctx.entry_first_row, ctx.entry_slot,
                               self.heads, self.groups, self.d, self.dv)
         o = ws.buffer("delta.heads", tokens, self.heads * self.dv, torch.float32)
-        groups = kernels.delta_row_groups(len(ctx.entries), self.heads, self.d, self.dv)
-        kernels.delta_walk(rows, gates, o, cache.state, ctx.entry_first_row, ctx.entry_start, ctx.entry_slot,
-                           self.heads, self.groups, self.d, self.dv, self.taps, groups)
+        # long portions 64 tokens at a time on the matrix cores, the other entries token by token (the lists depend on the
+        # step's shape alone)
+        key = "static:delta.chunks"
+        if key not in ctx.extras:
+            chunks, runs, others = kernels.delta_chunk_lists(ctx.entries, self.CHUNKED_MIN_TOKENS)
+            dev = lambda flat: ctx.to_device(flat) if flat else None
+            ctx.extras[key] = (dev(chunks), dev(runs), dev(others), len(others))
+        chunks, runs, others, walkers = ctx.extras[key]
+        if chunks is not None and self.chunked:
+            scratch = ws.buffer("delta.chunks", chunks.numel() // 4 * self.heads, kernels.delta_chunk_floats(self.d, self.dv),
+                                torch.float32)
+            kernels.delta_chunks(rows, gates, o, cache.state, ctx.entry_start, ctx.entry_slot, chunks, runs, scratch, self.heads,
+                                 self.groups, self.d, self.dv, self.taps)
+        else:
+            others, walkers = None, len(ctx.entries)
+        if walkers:
+            kernels.delta_walk(rows, gates, o, cache.state, ctx.entry_first_row, ctx.entry_start, ctx.entry_slot, self.heads,
+                               self.groups, self.d, self.dv, self.taps,
+                               kernels.delta_row_groups(walkers, self.heads, self.d, self.dv), which=others)
         kernels.group_norm_gate(o, self.norm_weight, y[:, self.gate0:self.gate0 + self.heads * self.dv], out, self.heads,
                                 self.eps, self.out_scale, "silu")
 

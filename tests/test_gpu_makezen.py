@@ -271,12 +271,15 @@ def test_blended_rotation_tables():
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_short_convolution_ring_and_recurrence(dtype):
     """The gated delta rule from its projections on against the plain mixer with identity projections: earlier portions,
-    then one step that holds a long portion, a fresh prompt in a slot full of NaN, two tokens and single tokens, then a
-    step of single tokens through the one-launch kernel and through prepared rows."""
+    then one step that holds a long portion, a fresh prompt in a slot full of NaN, two tokens and single tokens (token by
+    token, with the rows of the state shared out over 4 and over 16 lanes, and the longer ones in chunks), then a step of
+    single tokens through the one-launch kernel and through prepared rows."""
+    from types import SimpleNamespace
+
     from pulse_infer_amd.ops import kernels
 
     for heads, groups, d, dv, taps in [(4, 2, 16, 32, 4), (3, 1, 24, 20, 2), (2, 2, 40, 10, 3), (2, 2, 64, 64, 1),
-                                       (6, 3, 128, 128, 4), (2, 1, 256, 256, 5), (1, 1, 8, 4, 16), (2, 2, 33, 12, 4)]:
+                                       (6, 3, 128, 128, 4), (2, 1, 256, 256, 5), (1, 1, 8, 4, 16), (2, 2, 33, 12, 4), (2, 1, 100, 52, 4)]:
         eps, scale = 1e-5, 1.3
         gd, hv = groups * d, heads * dv
         channels = 2 * gd + hv
@@ -291,7 +294,7 @@ def test_short_convolution_ring_and_recurrence(dtype):
              "m.a": eye[a0:], "m.q.conv": taps_ref[:gd], "m.k.conv": taps_ref[gd:2 * gd], "m.v.conv": taps_ref[2 * gd:],
              "m.A_log": a_log.to(F64), "m.dt_bias": dt.to(F64), "m.norm": norm_w.to(F64), "m.o": torch.eye(hv, dtype=F64)}
         sizes = {"heads": heads, "kv_heads": groups, "dim": d, "vdim": dv}
-        counts, starts, slots = [70, 19, 2, 1, 1], [33, 0, 5, 17, 0], [3, 0, 4, 1, 6]
+        counts, starts, slots = [150, 64, 2, 1, 1], [33, 0, 5, 17, 0], [3, 0, 4, 1, 6]
         y_of, wants = [], []
         for r in range(5):
             y, ref = stored(rnd(starts[r] + counts[r] + 3, width, seed=40 + r), dtype)
@@ -321,13 +324,24 @@ def test_short_convolution_ring_and_recurrence(dtype):
             kernels.delta_prepare(x, b0, a0, conv, a_log, dt, state, rows, gates, positions, entry, start, first, slot, heads,
                                   groups, d, dv)
             o = torch.full((n, hv), float("nan"), dtype=torch.float32, device=DEV)
-            kernels.delta_walk(rows, gates, o, state, first, start, slot, heads, groups, d, dv, taps,
-                               row_groups or kernels.delta_row_groups(len(which), heads, d, dv))
+            others = None
+            if row_groups == "chunks":
+                entries = [SimpleNamespace(first_row=firsts[i], count=lens[r]) for i, r in enumerate(which)]
+                chunks, runs, others = kernels.delta_chunk_lists(entries, 2)
+                scratch = torch.full((len(chunks) // 4 * heads, kernels.delta_chunk_floats(d, dv)), float("nan"),
+                                     dtype=torch.float32, device=DEV)
+                kernels.delta_chunks(rows, gates, o, state, start, slot, ints(chunks), ints(runs), scratch, heads, groups, d, dv,
+                                     taps)
+                others = ints(others)
+            if others is None or others.numel():
+                kernels.delta_walk(rows, gates, o, state, first, start, slot, heads, groups, d, dv, taps,
+                                   row_groups if isinstance(row_groups, int) else kernels.delta_row_groups(len(which), heads, d, dv),
+                                   which=others)
             kernels.group_norm_gate(o, norm_w, x[:, g0:g0 + hv], out, heads, eps, scale, "silu")
             return out
 
         ends = {}
-        for row_groups in (4, 16):
+        for row_groups in (4, 16) + ("chunks",) * kernels.delta_chunks_takes(d, dv):
             state = torch.full((7, slot_floats), float("nan"), dtype=torch.float32, device=DEV)
             earlier = [r for r in range(5) if starts[r]]
             step(state, earlier, {r: 0 for r in earlier}, {r: starts[r] for r in earlier}, row_groups=row_groups)
@@ -335,6 +349,9 @@ def test_short_convolution_ring_and_recurrence(dtype):
             want = torch.cat([wants[r][starts[r]:starts[r] + counts[r]] for r in range(5)])
             near(got, want, dtype, (heads, groups, d, dv, taps, row_groups))
             ends[row_groups] = state
+            if row_groups != 4:       # the states and the convolutions' inputs that are left behind
+                used = [s for s in slots]
+                assert torch.allclose(state[used], ends[4][used], atol=1e-4, rtol=1e-4, equal_nan=True), (heads, d, dv, row_groups)
         one_launch = [True] if kernels.delta_decode_takes(d, dv) else []
         for fused in [False] + one_launch:
             state = ends[4].clone()
