@@ -101,6 +101,112 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(const TX* __restrict
     }
 }
 
+// The same for many tokens and few taps: a wavefront takes a unit of channels (a head of q or k, or 128 channels of v) for
+// RUN neighbouring tokens, two channels a lane, with the taps and the last inputs in registers: every input is read once.
+constexpr int RUN = 8;
+
+template <typename TX> __device__ __forceinline__ float2 load2(const TX* p);
+template <> __device__ __forceinline__ float2 load2<float>(const float* p) { return *reinterpret_cast<const float2*>(p); }
+template <> __device__ __forceinline__ float2 load2<bf16_t>(const bf16_t* p) {
+    const uint32_t two = *reinterpret_cast<const uint32_t*>(p);
+    return make_float2(__uint_as_float(two << 16), __uint_as_float(two & 0xffff0000u));
+}
+
+// (bfloat16 rows: the hardware's exponential and reciprocal, a few units in the last place of float32)
+template <typename TX> __device__ __forceinline__ float conv_silu(float v) {
+    if constexpr (sizeof(TX) == 4) return silu_f(v);
+    else return v * __builtin_amdgcn_rcpf(1.0f + __expf(-v));
+}
+
+template <typename TX, int TAPS, int PASSES>
+__global__ __launch_bounds__(256) void delta_prepare_runs_kernel(const TX* __restrict__ x, const float* __restrict__ taps,
+                                                                 const float* __restrict__ a_log, const float* __restrict__ dt_bias,
+                                                                 const float* __restrict__ state, float* __restrict__ rows,
+                                                                 float* __restrict__ gates, const int* __restrict__ positions,
+                                                                 const int* __restrict__ token_entry,
+                                                                 const int* __restrict__ entry_start,
+                                                                 const int* __restrict__ entry_first_row,
+                                                                 const int* __restrict__ entry_slot, int tokens, int units,
+                                                                 DeltaArgs a) {
+    const int lane = threadIdx.x % PULSE_WAVE, wave = threadIdx.x / PULSE_WAVE;
+    const int t0 = blockIdx.x * RUN, t1 = min(tokens, t0 + RUN);
+    if (blockIdx.y == 0) {
+        for (int i = threadIdx.x; i < (t1 - t0) * a.heads; i += 256) {
+            const int t = t0 + i / a.heads, h = i % a.heads;
+            const TX* row = x + static_cast<int64_t>(t) * a.x_stride;
+            gates[static_cast<int64_t>(t) * 2 * a.heads + h] = -expf(a_log[h]) * softplus_f(to_f32<TX>(row[a.a0 + h]) + dt_bias[h]);
+            gates[static_cast<int64_t>(t) * 2 * a.heads + a.heads + h] = sigmoid_f(to_f32<TX>(row[a.b0 + h]));
+        }
+    }
+    const int unit = blockIdx.y * 4 + wave;
+    if (unit >= units) return;
+    const bool qk = unit < 2 * a.groups;
+    const int first = qk ? unit * a.d : 2 * a.groups * a.d + (unit - 2 * a.groups) * 128;
+    const int width = qk ? a.d : min(128, a.channels - first);
+    float2 w[PASSES][TAPS], in[PASSES][TAPS];
+    bool ok[PASSES];
+#pragma unroll
+    for (int p = 0; p < PASSES; ++p) {
+        const int c = 128 * p + 2 * lane;
+        ok[p] = c < width;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+            w[p][j] = ok[p] ? *reinterpret_cast<const float2*>(taps + j * a.channels + first + c) : make_float2(0.f, 0.f);
+            in[p][j] = make_float2(0.f, 0.f);
+        }
+    }
+    int entry = -1;
+    for (int t = t0; t < t1; ++t) {
+        const int e = token_entry[t], pos = positions[t];
+        const bool fresh = e != entry;        // the inputs before this token are another sequence's
+        const int start = entry_start[e], row0 = entry_first_row[e];
+        entry = e;
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            const int c = first + 128 * p + 2 * lane;
+            if (fresh) {
+                const float* ring = state + static_cast<int64_t>(entry_slot[e]) * a.slot_stride + a.ring0;
+#pragma unroll
+                for (int j = 1; j < TAPS; ++j) {      // places 1 .. TAPS - 1 become 0 .. TAPS - 2 below
+                    const int q = pos - TAPS + j;
+                    in[p][j] = make_float2(0.f, 0.f);
+                    if (ok[p]) {
+                        if (q >= start) in[p][j] = load2<TX>(x + static_cast<int64_t>(row0 + q - start) * a.x_stride + c);
+                        else if (q >= 0) in[p][j] = *reinterpret_cast<const float2*>(ring + static_cast<int64_t>(q % TAPS) * a.channels + c);
+                    }
+                }
+            }
+#pragma unroll
+            for (int j = 0; j + 1 < TAPS; ++j) in[p][j] = in[p][j + 1];
+            in[p][TAPS - 1] = ok[p] ? load2<TX>(x + static_cast<int64_t>(t) * a.x_stride + c) : make_float2(0.f, 0.f);
+        }
+        float2 v[PASSES];
+        float ss = 0.f;
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p) {
+            v[p] = make_float2(0.f, 0.f);
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) {
+                v[p].x = fmaf(w[p][j].x, in[p][j].x, v[p].x);
+                v[p].y = fmaf(w[p][j].y, in[p][j].y, v[p].y);
+            }
+            v[p].x = conv_silu<TX>(v[p].x);
+            v[p].y = conv_silu<TX>(v[p].y);
+            ss = fmaf(v[p].x, v[p].x, fmaf(v[p].y, v[p].y, ss));
+        }
+        float f = 1.f;
+        if (qk) {
+            f = 1.0f / sqrtf(wave_sum(ss) + UNIT_EPS);
+            if (unit < a.groups) f *= 1.0f / sqrtf(static_cast<float>(a.d));
+        }
+#pragma unroll
+        for (int p = 0; p < PASSES; ++p)
+            if (ok[p])
+                *reinterpret_cast<float2*>(rows + static_cast<int64_t>(t) * a.channels + first + 128 * p + 2 * lane) =
+                    make_float2(v[p].x * f, v[p].y * f);
+    }
+}
+
 // The ring moves on to the end of every entry's portion: the last min(count, K) inputs go to their places.
 template <typename TX>
 __global__ __launch_bounds__(256) void delta_ring_kernel(const TX* __restrict__ x, float* __restrict__ state,
@@ -390,7 +496,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const float* _
 }
 
 template <int D>
-__global__ __launch_bounds__(256) void delta_chunk_walk_kernel(const float* __restrict__ scratch, const int* __restrict__ chunks,
+__global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* __restrict__ scratch, const int* __restrict__ chunks,
                                                                const int* __restrict__ runs, float* __restrict__ out,
                                                                float* __restrict__ state, const int* __restrict__ entry_start,
                                                                const int* __restrict__ entry_slot, int dvp, DeltaArgs a) {
@@ -417,34 +523,33 @@ __global__ __launch_bounds__(256) void delta_chunk_walk_kernel(const float* __re
             if (wave * TW + t < B) S_s[4 * kq + u][ch] = acc[t][u];
         }
     }
-    f32x4 wv[B], qv[B], pv[4], kd[TW][4];
-    float yv[4], el = 1.f;
-    auto item_of = [&](int i) { return scratch + (static_cast<int64_t>(first + i) * a.heads + h) * size; };
-    auto load_wq = [&](int i) __attribute__((always_inline)) {
-        const float* W = item_of(i) + (16 * wave + m) * D + 4 * kq;
+    // What a chunk's products read is asked for a whole chunk ahead, into one of two sets of registers.
+    struct Operands {
+        f32x4 wv[B], qv[B], pv[4], kd[TW][4];
+        float yv[4], el;
+    };
+    auto load = [&](int i, Operands& o) __attribute__((always_inline)) {
+        const float* W = scratch + (static_cast<int64_t>(first + i) * a.heads + h) * size;
+        const float* mine = W + (16 * wave + m) * D + 4 * kq;
 #pragma unroll
         for (int b = 0; b < B; ++b) {
-            wv[b] = *reinterpret_cast<const f32x4*>(W + 16 * b);
-            qv[b] = *reinterpret_cast<const f32x4*>(W + CHUNK * D + 16 * b);
+            o.wv[b] = *reinterpret_cast<const f32x4*>(mine + 16 * b);
+            o.qv[b] = *reinterpret_cast<const f32x4*>(mine + CHUNK * D + 16 * b);
         }
-    };
-    auto load_rest = [&](int i) __attribute__((always_inline)) {
-        const float* KdT = item_of(i) + 2 * CHUNK * D;
+        const float* KdT = W + 2 * CHUNK * D;
         const float* P = KdT + CHUNK * D;
         const float* Y = P + CHUNK * CHUNK;
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
-            pv[b] = load4(P + (16 * wave + m) * CHUNK + 16 * b + 4 * kq, b <= wave);
+            o.pv[b] = load4(P + (16 * wave + m) * CHUNK + 16 * b + 4 * kq, b <= wave);
 #pragma unroll
             for (int t = 0; t < TW; ++t)
-                kd[t][b] = load4(KdT + (16 * (wave * TW + t) + m) * CHUNK + 16 * b + 4 * kq, wave * TW + t < B);
-            yv[b] = Y[(16 * wave + 4 * kq + b) * dvp + c0 + m];
+                o.kd[t][b] = load4(KdT + (16 * (wave * TW + t) + m) * CHUNK + 16 * b + 4 * kq, wave * TW + t < B);
+            o.yv[b] = Y[(16 * wave + 4 * kq + b) * dvp + c0 + m];
         }
-        el = Y[CHUNK * dvp];
+        o.el = Y[CHUNK * dvp];
     };
-    load_wq(0);
-    load_rest(0);
-    for (int i = 0; i < count; ++i) {
+    auto chunk = [&](int i, const Operands& o) __attribute__((always_inline)) {
         const int row0 = chunks[4 * (first + i)], n = chunks[4 * (first + i) + 1];
         __syncthreads();     // S_s is whole, U_s has been read
         f32x4 us = {0.f, 0.f, 0.f, 0.f}, os = {0.f, 0.f, 0.f, 0.f};
@@ -453,29 +558,27 @@ __global__ __launch_bounds__(256) void delta_chunk_walk_kernel(const float* __re
             const f32x4 sb = *reinterpret_cast<const f32x4*>(&S_s[m][16 * b + 4 * kq]);
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                us = __builtin_amdgcn_mfma_f32_16x16x4f32(wv[b][u], sb[u], us, 0, 0, 0);
-                os = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[b][u], sb[u], os, 0, 0, 0);
+                us = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wv[b][u], sb[u], us, 0, 0, 0);
+                os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qv[b][u], sb[u], os, 0, 0, 0);
             }
         }
-        if (i + 1 < count) load_wq(i + 1);
         f32x4 uv;
 #pragma unroll
-        for (int u = 0; u < 4; ++u) uv[u] = yv[u] - us[u];
+        for (int u = 0; u < 4; ++u) uv[u] = o.yv[u] - us[u];
         *reinterpret_cast<f32x4*>(&U_s[m][16 * wave + 4 * kq]) = uv;
         __syncthreads();
 #pragma unroll
-        for (int t = 0; t < TW; ++t) acc[t] *= el;
+        for (int t = 0; t < TW; ++t) acc[t] *= o.el;
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             const f32x4 ub = *reinterpret_cast<const f32x4*>(&U_s[m][16 * b + 4 * kq]);
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                if (b <= wave) os = __builtin_amdgcn_mfma_f32_16x16x4f32(pv[b][u], ub[u], os, 0, 0, 0);
+                if (b <= wave) os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pv[b][u], ub[u], os, 0, 0, 0);
 #pragma unroll
-                for (int t = 0; t < TW; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ub[u], kd[t][b][u], acc[t], 0, 0, 0);
+                for (int t = 0; t < TW; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ub[u], o.kd[t][b][u], acc[t], 0, 0, 0);
             }
         }
-        if (i + 1 < count) load_rest(i + 1);
 #pragma unroll
         for (int t = 0; t < TW; ++t)
             if (wave * TW + t < B) {
@@ -488,6 +591,16 @@ __global__ __launch_bounds__(256) void delta_chunk_walk_kernel(const float* __re
                 const int r = 16 * wave + 4 * kq + u;
                 if (r < n) out[static_cast<int64_t>(row0 + r) * a.heads * a.dv + h * a.dv + c0 + m] = os[u];
             }
+        }
+    };
+    Operands even, odd;
+    load(0, even);
+    for (int i = 0; i < count; i += 2) {
+        if (i + 1 < count) load(i + 1, odd);
+        chunk(i, even);
+        if (i + 1 < count) {
+            if (i + 2 < count) load(i + 2, even);
+            chunk(i + 1, odd);
         }
     }
 #pragma unroll
@@ -655,10 +768,34 @@ extern "C" int pulse_delta_prepare(const void* x, int x_dtype, int64_t x_stride,
     PULSE_REQUIRE(b0 >= 0 && a0 >= 0 && x_stride >= a.channels && x_stride >= b0 + heads && x_stride >= a0 + heads,
                   "delta_prepare: the rows are too short");
     if (tokens == 0 || entries == 0) return 0;
-    PULSE_DISPATCH_DTYPE(x_dtype, TX,
-        hipLaunchKernelGGL(delta_prepare_kernel<TX>, dim3(tokens), dim3(256), 0, stream, static_cast<const TX*>(x), taps,
-                           a_log, dt_bias, state, rows, gates, positions, token_entry, entry_start, entry_first_row,
-                           entry_slot, a));
+    const int xb = x_dtype == PULSE_F32 ? 4 : 2;
+    const bool runs = tokens >= 64 && n_taps >= 2 && n_taps <= 4 && d % 2 == 0 && a.channels % 2 == 0 && x_stride % 2 == 0 &&
+                      slot_stride % 2 == 0 && a.ring0 % 2 == 0 && reinterpret_cast<uintptr_t>(x) % (2 * xb) == 0 &&
+                      reinterpret_cast<uintptr_t>(taps) % 8 == 0 && reinterpret_cast<uintptr_t>(state) % 8 == 0 &&
+                      reinterpret_cast<uintptr_t>(rows) % 8 == 0;
+    if (runs) {
+        const int units = 2 * groups + (heads * dv + 127) / 128;
+#define PULSE_RUNS(TAPS_, PASSES_)                                                                                        \
+    PULSE_DISPATCH_DTYPE(x_dtype, TX,                                                                                     \
+        hipLaunchKernelGGL((delta_prepare_runs_kernel<TX, TAPS_, PASSES_>), dim3((tokens + RUN - 1) / RUN, (units + 3) / 4), \
+                           dim3(256), 0, stream, static_cast<const TX*>(x), taps, a_log, dt_bias, state, rows, gates,     \
+                           positions, token_entry, entry_start, entry_first_row, entry_slot, tokens, units, a))
+        if (d <= 128) {
+            if (n_taps == 2) PULSE_RUNS(2, 1);
+            else if (n_taps == 3) PULSE_RUNS(3, 1);
+            else PULSE_RUNS(4, 1);
+        } else {
+            if (n_taps == 2) PULSE_RUNS(2, 2);
+            else if (n_taps == 3) PULSE_RUNS(3, 2);
+            else PULSE_RUNS(4, 2);
+        }
+#undef PULSE_RUNS
+    } else {
+        PULSE_DISPATCH_DTYPE(x_dtype, TX,
+            hipLaunchKernelGGL(delta_prepare_kernel<TX>, dim3(tokens), dim3(256), 0, stream, static_cast<const TX*>(x), taps,
+                               a_log, dt_bias, state, rows, gates, positions, token_entry, entry_start, entry_first_row,
+                               entry_slot, a));
+    }
     PULSE_LAUNCH_CHECK("delta_prepare");
     if (n_taps > 1) {
         PULSE_DISPATCH_DTYPE(x_dtype, TX,

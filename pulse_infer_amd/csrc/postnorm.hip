@@ -54,6 +54,32 @@ __global__ void activation_kernel(const T* __restrict__ x, T* __restrict__ y, in
     y[i] = from_f32<T>(r);
 }
 
+// bfloat16, eight neighbouring elements a thread; gelu as z sigmoid(2 u), the same as 0.5 z (1 + tanh(u)), with the
+// hardware's exponential and reciprocal (a few units in the last place of float32, rounded to bfloat16).
+__global__ __launch_bounds__(256) void activation_bf16x8_kernel(const bf16_t* __restrict__ x, bf16_t* __restrict__ y, int64_t n8,
+                                                                int act) {
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+    if (i >= n8) return;
+    const uint4 raw = reinterpret_cast<const uint4*>(x)[i];
+    const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
+    uint32_t out[4];
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+        float z[2] = {__uint_as_float(in[w] << 16), __uint_as_float(in[w] & 0xffff0000u)};
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const float v = z[u];
+            if (act == 1) { const float p = fmaxf(v, 0.f); z[u] = p * p; }
+            else {
+                const float e = act == 2 ? 1.5957691216057308f * (v + 0.044715f * v * v * v) : v;
+                z[u] = v * __builtin_amdgcn_rcpf(1.0f + __expf(-e));
+            }
+        }
+        out[w] = static_cast<uint32_t>(f32_to_bf16(z[0])) | (static_cast<uint32_t>(f32_to_bf16(z[1])) << 16);
+    }
+    reinterpret_cast<uint4*>(y)[i] = make_uint4(out[0], out[1], out[2], out[3]);
+}
+
 __global__ void softcap_kernel(float* __restrict__ x, int64_t n, float cap) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (i < n) x[i] = cap * tanhf(x[i] / cap);
@@ -92,6 +118,12 @@ extern "C" int pulse_activation(const void* x, void* y, int dtype, int64_t n, in
     if (n == 0) return 0;
     const int64_t blocks = (n + 255) / 256;
     PULSE_REQUIRE(blocks < (1ll << 31), "activation: too many elements");
+    if (dtype == PULSE_BF16 && n % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0) {
+        hipLaunchKernelGGL(activation_bf16x8_kernel, dim3(static_cast<unsigned>((n / 8 + 255) / 256)), dim3(256), 0, stream,
+                           static_cast<const bf16_t*>(x), static_cast<bf16_t*>(y), n / 8, act);
+        PULSE_LAUNCH_CHECK("activation");
+        return 0;
+    }
     PULSE_DISPATCH_DTYPE(dtype, T, hipLaunchKernelGGL(activation_kernel<T>, dim3(static_cast<unsigned>(blocks)), dim3(256),
                                                       0, stream, static_cast<const T*>(x), static_cast<T*>(y), n, act));
     PULSE_LAUNCH_CHECK("activation");

@@ -40,7 +40,7 @@ constexpr int NDT = D / 16;            // 16-channel tiles of the output
 constexpr int WAVES = 4;
 constexpr int BLOCK_KEYS = 32;
 // Column tiles a wavefront takes in the prompt-portion kernel: two while the accumulators of both fit the registers.
-#define PULSE_WIDE (PULSE_HEAD_DIM == 32 || PULSE_HEAD_DIM == 64 || PULSE_HEAD_DIM == 128)
+#define PULSE_WIDE (PULSE_HEAD_DIM == 32 || PULSE_HEAD_DIM == 64 || PULSE_HEAD_DIM == 128 || PULSE_HEAD_DIM == 192)
 #ifndef PULSE_WIDE_CT
 #define PULSE_WIDE_CT 2
 #endif
@@ -962,7 +962,8 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
 //      which eight neighbouring lanes read for one c lie in eight different 16-byte places of an LDS cycle;
 //   V: a tile of 16 keys is D channel rows of 32 bytes; the piece (channel ch, half h) sits at slot
 //      (ch / 16) * 32 + h * 16 + ch % 16, so the 16 channel rows of one half are 256 contiguous bytes.
-// Needs D in {32, 64, 128} (P a power of two, whole 1 KB chunks a tile).
+// Needs D in {32, 64, 128, 192} (whole 1 KB chunks a tile; P a power of two or a multiple of the 8 pieces that LDS serves
+// in a cycle, so that the rotation alone decides where in a cycle's 128 bytes a piece lies).
 //
 // The loads are written in assembly: the compiler knows nothing of them (it would wait for every one before any LDS
 // read), so the waits for them are written here too.  Its own vector loads inside the loop (the block table) only
@@ -990,7 +991,7 @@ __device__ __forceinline__ void load_to_lds(const void* from, uint32_t lds_base)
     asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" : : "s"(lds_base), "v"(from) : "memory", "m0");
 }
 
-#if PULSE_WIDE_CT > 2
+#if PULSE_WIDE_CT > 2 || PULSE_HEAD_DIM > 128   // (the accumulators take most of the registers, the stages most of LDS)
 #define PULSE_WIDE_WAVES_PER_EU __attribute__((amdgpu_waves_per_eu(1, 1)))
 #else
 #define PULSE_WIDE_WAVES_PER_EU PULSE_ATTN_WAVES_PER_EU
@@ -1000,7 +1001,7 @@ __global__ __launch_bounds__(NW* PULSE_WAVE) PULSE_WIDE_WAVES_PER_EU void attn_p
     using Shape = WideShape<CT, KT, NW>;
     constexpr int BK = Shape::BK;
     static_assert(KT % 2 == 0, "the second product takes pairs of key tiles");
-    static_assert(D == 32 || D == 64 || D == 128, "whole 1 KB chunks and a power of two of pieces a key");
+    static_assert(D == 32 || D == 64 || D == 128 || D == 192, "whole 1 KB chunks, and key rows that start at the same place of 128 bytes or divide them");
     constexpr int P = Shape::P;
     __shared__ __attribute__((aligned(1024))) bf16_t s_kv[2 * Shape::STAGE];  // stage: K block, then V block
 
@@ -1382,6 +1383,7 @@ __global__ __launch_bounds__(PR_THREADS) void attn_prefill_reduce_kernel(const f
     if (tok >= ntok) return;
     if (positions[row0 + ntok - 1] < split_size) return;   // the item was finished by its only split
     const int64_t row = row0 + tok;
+    if (threadIdx.x / PR_QUADS >= PR_HEADS) return;
     const int head = blockIdx.y * PR_HEADS + threadIdx.x / PR_QUADS;
     const int quad = threadIdx.x % PR_QUADS;
     if (head >= nq) return;

@@ -74,12 +74,13 @@ def tokens_per_item(group: int) -> int:
 
 PORTION_MIN_TOKENS = 16   # entries with at least this many tokens go to the kernel that shares keys through LDS
 PORTION_WAVES = 4         # wavefronts of its workgroup
+WIDE_HEAD_DIMS = (32, 64, 128, 192)   # head sizes its wide variant takes
 
 
 def portion_tokens(group: int, head_dim: int) -> int:
     """Tokens of one work item of the prompt-portion kernel: its four wavefronts take one or two column tiles of
     ``tokens_per_item`` tokens each (two for the head sizes its wide variant takes)."""
-    return tokens_per_item(group) * PORTION_WAVES * (2 if head_dim in (32, 64, 128) else 1)
+    return tokens_per_item(group) * PORTION_WAVES * (2 if head_dim in WIDE_HEAD_DIMS else 1)
 
 
 ITEM_INTS = 4
@@ -251,7 +252,7 @@ def _live(live_context: Optional[torch.Tensor]) -> None:
 
 
 PREFILL_SPLIT_KEYS = 64        # a split of the prompt-portion kernel is a whole number of its 64-key blocks
-PREFILL_SPLIT_HEAD_DIMS = (32, 64, 128)
+PREFILL_SPLIT_HEAD_DIMS = WIDE_HEAD_DIMS
 PREFILL_MAX_SPLITS = 64
 PREFILL_SCRATCH_BYTES = 1 << 30
 TAIL_SPLIT_MIN_BLOCKS = 64     # walks from here on (4,096 keys) are worth a cut at three quarters on a full chip
