@@ -377,19 +377,47 @@ __global__ __launch_bounds__(WALK_THREADS) void delta_walk_kernel(const float* _
 constexpr int CHUNK = 64;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
-// What the first kernel leaves for a (chunk, head), in floats from its place in the scratch (D: d rounded up):
-// W [64, D], e^G Q [64, D], (e^(G_last - G) K)^T [D, 64], P [64, 64], Y [64, dvp], e^(G_last).
+// What the first kernel leaves for a (chunk, head), in floats from its place in the scratch (D: d rounded up): W [64, D],
+// e^G Q [64, D], (e^(G_last - G) K)^T [D, 64], P [64, 64], Y [64, dvp], e^(G_last), 3 spare.  All matrices lie in tiles of
+// 16 x 16 in the order in which the second kernel's operands want them: the four numbers of lane l of a wavefront at
+// 4 l of the tile (a load is 1 KB in a row; row by row a load of 64 lanes would touch 64 pieces of 16 bytes).
+//   W, Q, P:  tile (row / 16, column / 16), lane = row % 16 + 16 (column % 16 / 4), number column % 4
+//   K^T:      tile (channel / 16, token / 16), lane = channel % 16 + 16 (token % 16 / 4), number token % 4
+//   Y:        tile (column / 16, token / 16), lane = column % 16 + 16 (token % 16 / 4), number token % 4
 __host__ __device__ inline int64_t chunk_floats(int D, int dvp) { return CHUNK * (3ll * D + CHUNK + dvp) + 4; }
 
 __device__ __forceinline__ f32x4 load4(const float* p, bool ok) {
     return ok ? *reinterpret_cast<const f32x4*>(p) : f32x4{0.f, 0.f, 0.f, 0.f};
 }
 
+// A 4 x 4 block turned around inside every quad of lanes: lane i of a quad brings v[0 .. 3] and leaves with what lanes
+// 0 .. 3 brought as their number i.
+__device__ __forceinline__ f32x4 quad_transpose(f32x4 v, int lane) {
+    f32x4 out;
+    const int q = lane & 3;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        // what goes to lane q ^ k (and comes from there): the number with that lane's place
+        const int to = q ^ k;
+        float send = to == 0 ? v[0] : to == 1 ? v[1] : to == 2 ? v[2] : v[3];
+        if (k == 1) send = lane_move<0xB1>(send);        // quad_perm [1, 0, 3, 2]
+        else if (k == 2) send = lane_move<0x4E>(send);   // quad_perm [2, 3, 0, 1]
+        else if (k == 3) send = lane_move<0x1B>(send);   // quad_perm [3, 2, 1, 0]
+        if (to == 0) out[0] = send;
+        else if (to == 1) out[1] = send;
+        else if (to == 2) out[2] = send;
+        else out[3] = send;
+    }
+    return out;
+}
+
 template <int D>
-__global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const float* __restrict__ rows, const float* __restrict__ gates,
+__global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(const float* __restrict__ rows, const float* __restrict__ gates,
                                                                   const int* __restrict__ chunks, float* __restrict__ scratch,
                                                                   int dvp, DeltaArgs a) {
+    constexpr int B = D / 16;
     __shared__ __attribute__((aligned(16))) float A_s[CHUNK][CHUNK + 4];
+    __shared__ __attribute__((aligned(16))) float K_s[CHUNK][D + 4];     // q first, then k
     __shared__ float G_s[CHUNK], beta_s[CHUNK], front_s[CHUNK], left_s[CHUNK];   // beta e^G, e^(G_last - G)
     const int h = blockIdx.y, tid = threadIdx.x, lane = tid % PULSE_WAVE, wave = tid / PULSE_WAVE;
     const int row0 = chunks[4 * blockIdx.x], n = chunks[4 * blockIdx.x + 1];
@@ -417,28 +445,41 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const float* _
         left_s[lane] = expf(last - g);
         if (lane == 0) Y[CHUNK * dvp] = expf(last);
     }
-    __syncthreads();
-    const int m = lane % 16, kq = lane / 16;
-    {
-        const int i = 16 * wave + m;
-        const float* row = rows + static_cast<int64_t>(row0 + i) * a.channels;
-        f32x4 ka[D / 16], qa[D / 16];
-        const float eg = expf(G_s[i]);
+    auto stage = [&](int col0) __attribute__((always_inline)) {
 #pragma unroll
-        for (int b = 0; b < D / 16; ++b) {
-            const int c = 16 * b + 4 * kq;
-            ka[b] = load4(row + k0 + c, i < n && c < a.d);
-            qa[b] = load4(row + q0 + c, i < n && c < a.d);
-            *reinterpret_cast<f32x4*>(Qs + i * D + c) = qa[b] * eg;
+        for (int u = 0; u < CHUNK * D / 4 / 256; ++u) {
+            const int idx = u * 256 + tid, i = idx / (D / 4), c = 4 * (idx % (D / 4));
+            *reinterpret_cast<f32x4*>(&K_s[i][c]) =
+                load4(rows + static_cast<int64_t>(row0 + i) * a.channels + col0 + c, i < n && c < a.d);
         }
+    };
+    const int m = lane % 16, kq = lane / 16;
+    stage(q0);
+    __syncthreads();
+    f32x4 qa[B];
+    {
+        const float eg = expf(G_s[16 * wave + m]);
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            qa[b] = *reinterpret_cast<const f32x4*>(&K_s[16 * wave + m][16 * b + 4 * kq]);
+            *reinterpret_cast<f32x4*>(Qs + ((wave * B + b) * PULSE_WAVE + lane) * 4) = qa[b] * eg;
+        }
+    }
+    __syncthreads();
+    stage(k0);
+    __syncthreads();
+    {
+        f32x4 ka[B];
+#pragma unroll
+        for (int b = 0; b < B; ++b) ka[b] = *reinterpret_cast<const f32x4*>(&K_s[16 * wave + m][16 * b + 4 * kq]);
+        for (int jt = wave + 1; jt < 4; ++jt)
+            *reinterpret_cast<f32x4*>(P + ((wave * 4 + jt) * PULSE_WAVE + lane) * 4) = f32x4{0.f, 0.f, 0.f, 0.f};
         for (int jt = 0; jt <= wave; ++jt) {
             const int j = 16 * jt + m;
-            const float* rj = rows + static_cast<int64_t>(row0 + j) * a.channels;
             f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int b = 0; b < D / 16; ++b) {
-                const int c = 16 * b + 4 * kq;
-                const f32x4 kb = load4(rj + k0 + c, j < n && c < a.d);
+            for (int b = 0; b < B; ++b) {
+                const f32x4 kb = *reinterpret_cast<const f32x4*>(&K_s[j][16 * b + 4 * kq]);
 #pragma unroll
                 for (int u = 0; u < 4; ++u) {
                     kk = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[b][u], kb[u], kk, 0, 0, 0);
@@ -446,57 +487,72 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(const float* _
                 }
             }
             // lane: rows 16 wave + 4 kq + u, column j
+            f32x4 p;
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
                 const int r = 16 * wave + 4 * kq + u;
                 const float e = j <= r ? expf(G_s[r] - G_s[j]) : 0.f;
                 A_s[r][j] = j < r ? beta_s[r] * e * kk[u] : 0.f;
-                P[r * CHUNK + j] = e * qk[u];
+                p[u] = e * qk[u];
             }
+            // rows 4 kq .. + 3 of column m become columns 4 (m / 4) .. + 3 of row 4 kq + m % 4
+            p = quad_transpose(p, lane);
+            *reinterpret_cast<f32x4*>(P + ((wave * 4 + jt) * PULSE_WAVE + 16 * (m / 4) + 4 * kq + m % 4) * 4) = p;
         }
     }
     __syncthreads();
-    // forward substitution, a thread a column of [W | Y]
+    // forward substitution, a thread a column of [W | Y] (whole wavefronts: the stores of W exchange numbers inside quads)
     for (int col = tid; col < D + dvp; col += 256) {
         const bool key = col < D;
         const int c = key ? col : col - D;
-        const bool there = key ? c < a.d : c < a.dv;
-        const float* src = rows + static_cast<int64_t>(row0) * a.channels + (key ? k0 : v0) + c;
         float x[CHUNK];
-#pragma unroll
-        for (int i = 0; i < CHUNK; ++i) x[i] = (there && i < n) ? src[static_cast<int64_t>(i) * a.channels] : 0.f;
         if (key) {
+#pragma unroll
+            for (int i = 0; i < CHUNK; ++i) x[i] = K_s[i][c];
 #pragma unroll
             for (int b = 0; b < CHUNK / 4; ++b) {
                 f32x4 t;
 #pragma unroll
                 for (int u = 0; u < 4; ++u) t[u] = x[4 * b + u] * left_s[4 * b + u];
-                *reinterpret_cast<f32x4*>(KdT + c * CHUNK + 4 * b) = t;
+                *reinterpret_cast<f32x4*>(KdT + (((c / 16) * 4 + b / 4) * PULSE_WAVE + 16 * (b % 4) + c % 16) * 4) = t;
             }
+        } else {
+            const float* src = rows + static_cast<int64_t>(row0) * a.channels + v0 + c;
+#pragma unroll
+            for (int i = 0; i < CHUNK; ++i) x[i] = (c < a.dv && i < n) ? src[static_cast<int64_t>(i) * a.channels] : 0.f;
         }
+        int place = 0;
 #pragma unroll
         for (int i = 0; i < CHUNK; ++i) {
+            // a row of A is read when the row before the last has been used: all at once they need 2000 registers
+            if (i > 1) asm volatile("" : "+v"(place), "+v"(x[i - 2]));
             float s[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int b = 0; b < (i + 3) / 4; ++b) {
-                const f32x4 ar = *reinterpret_cast<const f32x4*>(&A_s[i][4 * b]);
+                const f32x4 ar = *reinterpret_cast<const f32x4*>(&A_s[i][4 * b + place]);
 #pragma unroll
                 for (int u = 0; u < 4; ++u)
                     if (4 * b + u < i) s[u] = fmaf(ar[u], x[4 * b + u], s[u]);
             }
             const float f = key ? front_s[i] : beta_s[i];
             x[i] = f * x[i] - ((s[0] + s[1]) + (s[2] + s[3]));
-            asm volatile("" ::: "memory");   // (rows of A are read when their turn comes: all at once they need 500 registers)
         }
-        float* dst = key ? W + c : Y + c;
-        const int pitch = key ? D : dvp;
 #pragma unroll
-        for (int i = 0; i < CHUNK; ++i) dst[i * pitch] = x[i];
+        for (int b = 0; b < CHUNK / 4; ++b) {
+            f32x4 t = {x[4 * b], x[4 * b + 1], x[4 * b + 2], x[4 * b + 3]};
+            if (key) {   // a row's four neighbouring columns
+                t = quad_transpose(t, lane);
+                const int r = 4 * b + c % 4;
+                *reinterpret_cast<f32x4*>(W + (((r / 16) * B + c / 16) * PULSE_WAVE + 16 * ((c % 16) / 4) + r % 16) * 4) = t;
+            } else {     // a column's four neighbouring rows
+                *reinterpret_cast<f32x4*>(Y + (((c / 16) * 4 + b / 4) * PULSE_WAVE + 16 * (b % 4) + c % 16) * 4) = t;
+            }
+        }
     }
 }
 
 template <int D>
-__global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* __restrict__ scratch, const int* __restrict__ chunks,
+__global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(float* __restrict__ scratch, const int* __restrict__ chunks,
                                                                const int* __restrict__ runs, float* __restrict__ out,
                                                                float* __restrict__ state, const int* __restrict__ entry_start,
                                                                const int* __restrict__ entry_slot, int dvp, DeltaArgs a) {
@@ -523,29 +579,30 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* _
             if (wave * TW + t < B) S_s[4 * kq + u][ch] = acc[t][u];
         }
     }
-    // What a chunk's products read is asked for a whole chunk ahead, into one of two sets of registers.
+    // What a chunk's products read is asked for a whole chunk ahead, into one of two sets of registers.  Loads and stores
+    // stand outside every branch (addresses are clamped, results that nobody may see go to a spare place behind the item's
+    // last number): the compiler then knows how many are in flight and waits for the older set alone.
     struct Operands {
-        f32x4 wv[B], qv[B], pv[4], kd[TW][4];
-        float yv[4], el;
+        f32x4 wv[B], qv[B], pv[4], kd[TW][4], yv;
+        float el;
     };
     auto load = [&](int i, Operands& o) __attribute__((always_inline)) {
         const float* W = scratch + (static_cast<int64_t>(first + i) * a.heads + h) * size;
-        const float* mine = W + (16 * wave + m) * D + 4 * kq;
-#pragma unroll
-        for (int b = 0; b < B; ++b) {
-            o.wv[b] = *reinterpret_cast<const f32x4*>(mine + 16 * b);
-            o.qv[b] = *reinterpret_cast<const f32x4*>(mine + CHUNK * D + 16 * b);
-        }
         const float* KdT = W + 2 * CHUNK * D;
         const float* P = KdT + CHUNK * D;
         const float* Y = P + CHUNK * CHUNK;
+        auto tile = [&](const float* from, int t) { return *reinterpret_cast<const f32x4*>(from + (t * PULSE_WAVE + lane) * 4); };
+#pragma unroll
+        for (int b = 0; b < B; ++b) {
+            o.wv[b] = tile(W, wave * B + b);
+            o.qv[b] = tile(W + CHUNK * D, wave * B + b);
+        }
+        o.yv = tile(Y, blockIdx.z * 4 + wave);
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
-            o.pv[b] = load4(P + (16 * wave + m) * CHUNK + 16 * b + 4 * kq, b <= wave);
+            o.pv[b] = tile(P, wave * 4 + b);
 #pragma unroll
-            for (int t = 0; t < TW; ++t)
-                o.kd[t][b] = load4(KdT + (16 * (wave * TW + t) + m) * CHUNK + 16 * b + 4 * kq, wave * TW + t < B);
-            o.yv[b] = Y[(16 * wave + 4 * kq + b) * dvp + c0 + m];
+            for (int t = 0; t < TW; ++t) o.kd[t][b] = tile(KdT, min(wave * TW + t, B - 1) * 4 + b);
         }
         o.el = Y[CHUNK * dvp];
     };
@@ -553,13 +610,16 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* _
         const int row0 = chunks[4 * (first + i)], n = chunks[4 * (first + i) + 1];
         __syncthreads();     // S_s is whole, U_s has been read
         f32x4 us = {0.f, 0.f, 0.f, 0.f}, os = {0.f, 0.f, 0.f, 0.f};
+        f32x4 sb[B];
+#pragma unroll
+        for (int b = 0; b < B; ++b) sb[b] = *reinterpret_cast<const f32x4*>(&S_s[m][16 * b + 4 * kq]);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int b = 0; b < B; ++b) {
-            const f32x4 sb = *reinterpret_cast<const f32x4*>(&S_s[m][16 * b + 4 * kq]);
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                us = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wv[b][u], sb[u], us, 0, 0, 0);
-                os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qv[b][u], sb[u], os, 0, 0, 0);
+                us = __builtin_amdgcn_mfma_f32_16x16x4f32(o.wv[b][u], sb[b][u], us, 0, 0, 0);
+                os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.qv[b][u], sb[b][u], os, 0, 0, 0);
             }
         }
         f32x4 uv;
@@ -569,14 +629,18 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* _
         __syncthreads();
 #pragma unroll
         for (int t = 0; t < TW; ++t) acc[t] *= o.el;
+        f32x4 ub[4];
+#pragma unroll
+        for (int b = 0; b < 4; ++b) ub[b] = *reinterpret_cast<const f32x4*>(&U_s[m][16 * b + 4 * kq]);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
-            const f32x4 ub = *reinterpret_cast<const f32x4*>(&U_s[m][16 * b + 4 * kq]);
 #pragma unroll
             for (int u = 0; u < 4; ++u) {
-                if (b <= wave) os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pv[b][u], ub[u], os, 0, 0, 0);
+                os = __builtin_amdgcn_mfma_f32_16x16x4f32(o.pv[b][u], ub[b][u], os, 0, 0, 0);
 #pragma unroll
-                for (int t = 0; t < TW; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ub[u], o.kd[t][b][u], acc[t], 0, 0, 0);
+                for (int t = 0; t < TW; ++t)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ub[b][u], o.kd[t][b][u], acc[t], 0, 0, 0);
             }
         }
 #pragma unroll
@@ -585,23 +649,23 @@ __global__ __launch_bounds__(256, 1) void delta_chunk_walk_kernel(const float* _
 #pragma unroll
                 for (int u = 0; u < 4; ++u) S_s[4 * kq + u][16 * (wave * TW + t) + m] = acc[t][u];
             }
-        if (c0 + m < a.dv) {
+        float* spare = scratch + (static_cast<int64_t>(first + i) * a.heads + h + 1) * size - 1;
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                const int r = 16 * wave + 4 * kq + u;
-                if (r < n) out[static_cast<int64_t>(row0 + r) * a.heads * a.dv + h * a.dv + c0 + m] = os[u];
-            }
+        for (int u = 0; u < 4; ++u) {
+            const int r = 16 * wave + 4 * kq + u;
+            float* dst = out + static_cast<int64_t>(row0 + r) * a.heads * a.dv + h * a.dv + c0 + m;
+            *(r < n && c0 + m < a.dv ? dst : spare) = os[u];
         }
     };
     Operands even, odd;
     load(0, even);
-    for (int i = 0; i < count; i += 2) {
-        if (i + 1 < count) load(i + 1, odd);
+    for (int i = 0;;) {
+        load(min(i + 1, count - 1), odd);
         chunk(i, even);
-        if (i + 1 < count) {
-            if (i + 2 < count) load(i + 2, even);
-            chunk(i + 1, odd);
-        }
+        if (++i == count) break;
+        load(min(i + 1, count - 1), even);
+        chunk(i, odd);
+        if (++i == count) break;
     }
 #pragma unroll
     for (int t = 0; t < TW; ++t) {
