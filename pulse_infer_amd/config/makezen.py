@@ -6,8 +6,9 @@ mixer), the mixer's sizes and constants (``mixer``) and its feed-forward (``mlp`
 constant is taken from there.  Tensors: ``embed``, ``embed.norm``, ``l<i>.norm1`` / ``norm1b`` / ``norm2`` / ``norm2b``,
 ``l<i>.mix.*``, ``l<i>.mlp.up`` / ``down``, ``final.norm``; the logits are a product with ``embed``.
 
-The model: x = norm(embed[token]); per layer x <- x + norm1b(mixer(norm1(x))), then x <- x + norm2b(ff(norm2(x))); all
-these norms are layer norms with a weight and no bias.  logits = embed final.norm(x).
+The model: the token's row of ``embed`` through ``embed.norm``; every sublayer f (a layer's mixer, then its
+feed-forward) adds post(f(pre(x))), with ``norm1`` and ``norm1b`` around the mixer, ``norm2`` and ``norm2b`` around the
+feed-forward; all these norms are layer norms with a weight and no bias.  logits = embed final.norm(x).
 
 Mixers.  ``delta``: the gated delta rule behind convolutions of ``conv`` taps (``heads`` x ``dim`` x ``vdim`` states,
 ``kv_heads`` heads of q and k).  ``parallel``: half the sum of two mixers on the same input, each result divided by its

@@ -6,7 +6,7 @@
 //     x_t <- silu(sum_j taps[j] raw_(t - (K - 1) + j))                  zeros before the sequence's start
 // then q and k become unit vectors, x / sqrt(sum(x^2) + 1e-6), q times d^(-1/2), and per head
 //     beta = sigmoid(b)      g = exp(-exp(A_log) softplus(a + dt_bias))
-//     S <- g S               u = beta (v - S^T k)        S <- S + k u^T        o = S^T q
+//     D = g S                r = v - D^T k               S = D + beta k r^T    o = S^T q
 //
 // A request's slot holds one float32 row: S [heads, d, dv], then the last raw inputs of the convolutions as a ring
 // [K, channels], the input at position p in place p % K.  A decoded token then writes a place that no other workgroup

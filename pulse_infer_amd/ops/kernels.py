@@ -1354,7 +1354,8 @@ def delta_row_groups(entries: int, heads: int, d: int, dv: int) -> int:
 def delta_walk(rows: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, state: torch.Tensor, entry_first_row: torch.Tensor,
                entry_start: torch.Tensor, entry_slot: torch.Tensor, heads: int, groups: int, d: int, dv: int,
                n_taps: int, row_groups: int, which: Optional[torch.Tensor] = None) -> None:
-    """For every entry (or those whose numbers ``which`` lists, int32), token by token over prepared rows: S <- e^g S, u = beta (v - S^T k), S <- S + k u^T, out = S^T q, per
+    """For every entry (or those whose numbers ``which`` lists, int32), token by token over prepared rows: with the
+    decayed state D = e^g S the error r = v - D^T k is written back, S = D + beta k r^T, and read, out = S^T q, per
     head, in float32; S is the front of the entry's slot, zero when the entry starts at position 0."""
     _gpu("delta_walk", rows, gates, out, state, entry_first_row, entry_start, entry_slot, which)
     tokens, entries = rows.shape[0], entry_start.numel()

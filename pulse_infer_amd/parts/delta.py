@@ -2,11 +2,11 @@
 
 For a token with input x: q = Wq x and k = Wk x (``num_groups`` x dim), v = Wv x (``num_heads`` x vdim); each passes a
 causal convolution along the sequence (``conv`` taps a channel, no bias, zeros before a sequence's start) and silu; then
-q and k are made unit vectors per head, x / sqrt(sum(x^2) + 1e-6), and q is multiplied by dim^(-1/2).  Query head h uses q
-and k of group h // (num_heads // num_groups).  With beta = sigmoid(Wb x) and g = exp(-exp(A_log) softplus(Wa x + dt_bias)),
+every head of q and k is divided by its length (with 1e-6 added to the sum of squares), and q multiplied by dim^(-1/2).
+Query head h uses q and k of group h // (num_heads // num_groups).  With beta = sigmoid(Wb x) and g = exp(-exp(A_log) softplus(Wa x + dt_bias)),
 one of each a head, every head keeps a state S [dim, vdim] per request, zero at the request's start:
 
-    S <- g S          u = beta (v - S^T k)          S <- S + k u^T          o = S^T q
+    D = g S           r = v - D^T k           S = D + beta k r^T           o = S^T q
 
 Every head's o is divided by its own root mean square, multiplied by a weight [vdim] that the heads share and by
 silu(Wg x); the heads side by side are projected by Wo.

@@ -149,7 +149,7 @@ def unit_vector(x: torch.Tensor) -> torch.Tensor:
 
 
 def delta_walk(q, k, v, beta, log_decay) -> torch.Tensor:
-    """Per head, token by token: S <- e^a S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.  q, k [T, H, d],
+    """Per head, token by token: D = e^a S; r = v - D^T k; S = D + beta k r^T; o = S^T q.  q, k [T, H, d],
     v [T, H, dv], beta and log_decay [T, H]."""
     t, heads, d = q.shape
     out = torch.zeros(t, heads, v.shape[2], dtype=q.dtype)
