@@ -4,12 +4,12 @@
     llm = LLM.from_pretrained("model_dir", dtype="bfloat16")
     out = llm.generate([[1, 2, 3]], max_new_tokens=16)
 """
-from .config import (ConfigError, DirozenConfig, FosupelConfig, KesovikConfig, MakezenConfig, Qwen3Config, TipidraConfig, load_config,
-                     register_architecture)
+from .config import (ConfigError, DirozenConfig, FosupelConfig, KesovikConfig, MakezenConfig, Qwen3Config,
+                     SosuvikConfig, TipidraConfig, load_config, register_architecture)
 from .sampling.params import SamplingParams
 
-__all__ = ["ConfigError", "DirozenConfig", "FosupelConfig", "KesovikConfig", "MakezenConfig", "Qwen3Config", "TipidraConfig", "load_config", "register_architecture", "SamplingParams", "LLM",
-           "ContinuousBatchEngine"]
+__all__ = ["ConfigError", "DirozenConfig", "FosupelConfig", "KesovikConfig", "MakezenConfig", "Qwen3Config",
+           "SosuvikConfig", "TipidraConfig", "load_config", "register_architecture", "SamplingParams", "LLM", "ContinuousBatchEngine"]
 
 
 def __getattr__(name):  # the engine pulls in torch.cuda pieces; load it on first use

@@ -76,11 +76,19 @@ class CacheGroup:
     def window(self) -> Optional[int]:
         return getattr(self.spec, "window", None)
 
+    @property
+    def forgets(self) -> bool:
+        """Whether pages go back to the pool while their request still runs."""
+        return self.window is not None or bool(getattr(self.spec, "chunk", None))
+
     def pages_for(self, length: int) -> int:
         return (length + self.page_size - 1) // self.page_size
 
     def first_needed_token(self, computed: int) -> int:
         """The lowest key position that a token at position >= computed can still read."""
+        chunk = getattr(self.spec, "chunk", None)
+        if chunk:
+            return computed // chunk * chunk
         if self.window is None:
             return 0
         return max(0, computed - self.window + 1)
@@ -248,7 +256,7 @@ class CacheManager:
             raise CacheError(f"request {request!r} computed {computed} tokens but pages are reserved for {req.reserved}")
         req.computed = computed
         for g in self.groups:
-            if g.window is None:
+            if not g.forgets:
                 continue
             table = g.tables[request]
             dead = min(g.first_needed_token(computed) // g.page_size, len(table))

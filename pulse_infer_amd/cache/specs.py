@@ -10,7 +10,9 @@ A spec is a small hashable object that the cache manager asks, never inspects:
   tokens are ever read, so pages wholly below the window go back to the pool
   while the request still runs.  ``keep_first`` (optional, default 0): the first
   tokens of a request that stay readable whatever the window; the pages that hold
-  them are kept.
+  them are kept.  ``chunk`` (optional, in place of a window): positions fall into
+  chunks of that many, counted from 0, and a token reads keys of its own chunk
+  only, so pages wholly in chunks that are over go back.
 * ``bytes_per_token(element_size)`` (per-token specs) — what one token costs one
   run, for sizing pools and pricing steps.
 * ``allocate(runs, units, page_size, device, dtype)`` — the storage of all runs of
@@ -67,6 +69,7 @@ class PagedKVSpec:
     head_dim: int
     window: Optional[int] = None  # None: all keys
     keep_first: int = 0           # with a window: the first tokens stay readable, so their pages are never given back
+    chunk: Optional[int] = None   # in place of a window: a token reads the keys of its own chunk of positions only
 
     per_token = True
 

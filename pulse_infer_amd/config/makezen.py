@@ -85,13 +85,13 @@ class Rotation:
             out["scaling"] = dict(self.scaling)
         return out
 
-    def position(self, head_dim: int, positions: Dict[str, PartSpec]) -> Optional[str]:
+    def position(self, head_dim: int, positions: Dict[str, PartSpec], pairing: str = "half") -> Optional[str]:
         """The name under which the model lists this rotation (listed on the way); None without one."""
         if not self.dims:
             return None
         scaled = "" if self.scaling is None else ":" + ":".join(repr(self.scaling[key]) for key in SCALING_KEYS)
-        name = f"rope:{self.base!r}:{self.dims}{scaled}"
-        params: Dict[str, Any] = {"theta": self.base, "rotary_dim": self.dims, "head_dim": max(head_dim, self.dims), "pairing": "half"}
+        name = f"rope:{self.base!r}:{self.dims}{scaled}" + ("" if pairing == "half" else f":{pairing}")
+        params: Dict[str, Any] = {"theta": self.base, "rotary_dim": self.dims, "head_dim": max(head_dim, self.dims), "pairing": pairing}
         if self.scaling is not None:
             params["yarn"] = dict(self.scaling)
         positions.setdefault(name, PartSpec("rope", params))

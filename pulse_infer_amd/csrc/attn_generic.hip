@@ -2,7 +2,7 @@
 // wavefront per (token, query head), float32 arithmetic throughout.
 //
 // A token at position p sees keys lo..p of its own request through the block
-// table, lo = max(0, p - window + 1) when a window is set, else 0.  Keys are
+// table, lo = max(0, p - window + 1) when a window is set, p - p mod chunk when chunks are, else 0.  Keys are
 // taken 64 at a time (one per lane); the softmax is the running-maximum form
 // (reference: src/ops/kernels/cuda/paged_attention.cu:88-137), the scale is a
 // parameter (the reference fixes rsqrt(head_size), paged_attention.cu:108), and
@@ -35,6 +35,7 @@ struct AttnArgs {
     int page_size, num_pages, bt_width;
     float scale;
     int window;  // 0: all keys
+    int chunk;   // > 0 (without a window): the keys of the token's own chunk of this many positions
     float cap;   // > 0: a score s becomes cap * tanh(s / cap); 0: scores as they are
     int gate_per_channel;   // 0: one gate logit a head; 1: one a channel (gate [T, nq * gate_width])
     int gate_width;         // channels of a head that have a gate logit (the others are stored ungated)
@@ -64,7 +65,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const TX* __restrict__
     const int kvh = h / group;
     const int pos = positions[t];
     const int* bt = block_table + static_cast<int64_t>(token_entry[t]) * a.bt_width;
-    const int lo = (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
+    const int lo = a.chunk > 0 ? pos - pos % a.chunk : (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
     const int n_first = min(a.keep_first, lo);        // kept keys below the window
     const int total = n_first + pos - lo + 1;         // keys this token sees
     const int width = a.all_values ? a.nkv * d : d;   // values accumulated for this query head
@@ -171,7 +172,8 @@ extern "C" int pulse_attn_generic_ex(const void* q, int64_t q_stride, void* out,
                                      const int* token_entry, const int* block_table, int bt_width, int tokens, int nq,
                                      int nkv, int d, int page_size, int num_pages, float scale, int window,
                                      const void* gate, int64_t gate_stride, int gate_width, const float* sink,
-                                     float softcap, int keep_first, int all_values, int out_f32, hipStream_t stream) {
+                                     float softcap, int keep_first, int all_values, int out_f32, int chunk,
+                                     hipStream_t stream) {
     const int width = all_values ? nkv * d : d;
     PULSE_REQUIRE(tokens >= 0 && nq > 0 && nkv > 0 && d > 0, "attn_generic: bad sizes");
     PULSE_REQUIRE(nq % nkv == 0, "attn_generic: %d query heads are not a multiple of %d kv heads", nq, nkv);
@@ -180,6 +182,7 @@ extern "C" int pulse_attn_generic_ex(const void* q, int64_t q_stride, void* out,
     PULSE_REQUIRE(nq < 65536, "attn_generic: at most 65535 query heads, got %d", nq);
     PULSE_REQUIRE(page_size > 0 && num_pages > 0 && bt_width > 0, "attn_generic: bad cache geometry");
     PULSE_REQUIRE(window >= 0 && keep_first >= 0, "attn_generic: negative window or kept keys");
+    PULSE_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "attn_generic: a window and chunks at once");
     PULSE_REQUIRE(!all_values || (out_f32 && !gate), "attn_generic: all values side by side come out in float32, ungated");
     PULSE_REQUIRE(q_stride >= static_cast<int64_t>(nq) * d && o_stride >= static_cast<int64_t>(nq) * width,
                   "attn_generic: row strides too small");
@@ -192,7 +195,7 @@ extern "C" int pulse_attn_generic_ex(const void* q, int64_t q_stride, void* out,
     if (tokens == 0) return 0;
     AttnArgs a;
     a.nq = nq; a.nkv = nkv; a.d = d; a.q_stride = q_stride; a.o_stride = o_stride;
-    a.page_size = page_size; a.num_pages = num_pages; a.bt_width = bt_width; a.scale = scale; a.window = window;
+    a.page_size = page_size; a.num_pages = num_pages; a.bt_width = bt_width; a.scale = scale; a.window = window; a.chunk = chunk;
     a.cap = softcap; a.gate_per_channel = gate_width > 0 ? 1 : 0; a.gate_width = gate_width;
     a.keep_first = window > 0 ? keep_first : 0; a.all_values = all_values ? 1 : 0;
     const size_t lds = static_cast<size_t>(d) * sizeof(float) + PULSE_WAVE * sizeof(float) + PULSE_WAVE * sizeof(long long);
@@ -214,5 +217,5 @@ extern "C" int pulse_attn_generic(const void* q, int64_t q_stride, void* out, in
                                   float softcap, hipStream_t stream) {
     return pulse_attn_generic_ex(q, q_stride, out, o_stride, x_dtype, kcache, vcache, c_dtype, positions, token_entry,
                                  block_table, bt_width, tokens, nq, nkv, d, page_size, num_pages, scale, window, gate,
-                                 gate_stride, gate_width, sink, softcap, 0, 0, 0, stream);
+                                 gate_stride, gate_width, sink, softcap, 0, 0, 0, 0, stream);
 }

@@ -18,7 +18,9 @@
 // scores as they are.  `in_weight` (gate/up kernels): the expert is fed weight * x, i.e. both products are multiplied
 // by the pair's weight before the activation (the products are linear), and the down kernels are then handed no
 // weight.  `act_kind` 1 is the clamped form g' = min(g, limit), u' = clamp(u, -limit, limit),
-// act = g' * sigmoid(1.702 g') * (u' + 1).
+// act = g' * sigmoid(1.702 g') * (u' + 1).  `groups` > 1: the outputs form that many equal groups of neighbours, a group's
+// mark is the sum of its two largest s + correction, and only outputs of the `keep` groups with the largest marks (the
+// lower group among equals) can be chosen.  `wscale` multiplies the weights behind everything else.
 #include "common.h"
 
 #include <math.h>
@@ -27,11 +29,47 @@ namespace {
 
 constexpr int ROUTE_PER_LANE = 16;   // router outputs <= 64 * 16
 
+struct RouteForm {
+    int score_fn, renorm;
+    int groups, keep;        // groups <= 1: no groups
+    float wscale;
+};
+
+// Which groups stay, as a bit mask: lane g forms the mark of group g from the choice scores `c` of all lanes (lane + 64 r
+// holds output lane + 64 r), which go through `c_s` (LDS, one wavefront's).
+__device__ __forceinline__ unsigned long long kept_groups(const float (&c)[ROUTE_PER_LANE], float* c_s, int n, int groups,
+                                                          int keep, int lane) {
+#pragma unroll
+    for (int r = 0; r < ROUTE_PER_LANE; ++r) {
+        const int j = lane + r * PULSE_WAVE;
+        if (j < n) c_s[j] = c[r];
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");   // (one wavefront writes and reads: order is all it needs)
+    __builtin_amdgcn_wave_barrier();
+    const int size = n / groups;
+    float first = -INFINITY, second = -INFINITY;
+    if (lane < groups) {
+        for (int i = 0; i < size; ++i) {
+            const float v = c_s[lane * size + i];
+            second = fmaxf(second, fminf(first, v));
+            first = fmaxf(first, v);
+        }
+    }
+    const float mark = lane < groups ? (size > 1 ? first + second : first) : -INFINITY;
+    int before = 0;
+    for (int g = 0; g < groups; ++g) {
+        const float other = __shfl(mark, g, PULSE_WAVE);
+        before += (other > mark || (other == mark && g < lane)) ? 1 : 0;
+    }
+    return __ballot(lane < groups && before < keep);
+}
+
 // One wavefront routes one token: `row` holds its n router logits (in global memory or in LDS).
 template <typename TW>
 __device__ __forceinline__ void route_row(const float* row, const TW* __restrict__ correction, int* __restrict__ idx,
                                           float* __restrict__ weight, int n, int top, int t, int lane,
-                                          int score_fn, int renorm) {
+                                          const RouteForm& form, float* c_s) {
+    const int score_fn = form.score_fn, renorm = form.renorm;
     float s[ROUTE_PER_LANE], c[ROUTE_PER_LANE];
     float m = -INFINITY;
 #pragma unroll
@@ -55,6 +93,15 @@ __device__ __forceinline__ void route_row(const float* row, const TW* __restrict
         const int j = lane + r * PULSE_WAVE;
         s[r] = s[r] / sum;
         c[r] = j < n ? s[r] + (correction ? to_f32<TW>(correction[j]) : 0.f) : -INFINITY;
+    }
+    if (form.groups > 1) {
+        const unsigned long long kept = kept_groups(c, c_s, n, form.groups, form.keep, lane);
+        const int size = n / form.groups;
+#pragma unroll
+        for (int r = 0; r < ROUTE_PER_LANE; ++r) {
+            const int j = lane + r * PULSE_WAVE;
+            if (j < n && !((kept >> (j / size)) & 1ull)) c[r] = -INFINITY;
+        }
     }
     float total = 0.f;
     float mine = 0.f;   // lane k keeps the score of choice k (top <= 64)
@@ -86,16 +133,17 @@ __device__ __forceinline__ void route_row(const float* row, const TW* __restrict
     }
     if (lane < top) {
         idx[static_cast<int64_t>(t) * top + lane] = mine_idx;
-        weight[static_cast<int64_t>(t) * top + lane] = renorm ? mine / (total + 1e-20f) : mine;
+        weight[static_cast<int64_t>(t) * top + lane] = (renorm ? mine / (total + 1e-20f) : mine) * form.wscale;
     }
 }
 
 template <typename TW>
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, const TW* __restrict__ correction,
                                                        int* __restrict__ idx, float* __restrict__ weight, int n, int top,
-                                                       int score_fn, int renorm) {
+                                                       RouteForm form) {
+    __shared__ float c_s[PULSE_WAVE * ROUTE_PER_LANE];
     route_row<TW>(z + static_cast<int64_t>(blockIdx.x) * n, correction, idx, weight, n, top, blockIdx.x, threadIdx.x,
-                  score_fn, renorm);
+                  form, c_s);
 }
 
 // The router's product and the routing in one: a workgroup a token holds the token's row in LDS, its wavefronts
@@ -105,8 +153,8 @@ template <typename TX, typename TW>
 __global__ __launch_bounds__(1024) void moe_router_kernel(const TX* __restrict__ x, const TW* __restrict__ w,
                                                          const TW* __restrict__ correction, int* __restrict__ idx,
                                                          float* __restrict__ weight, int hidden, int n, int top,
-                                                         int score_fn, int renorm) {
-    extern __shared__ float x_s[];          // [hidden] then [n]
+                                                         RouteForm form) {
+    extern __shared__ float x_s[];          // [hidden], then [n] logits, then [n] choice scores
     float* z_s = x_s + hidden;
     const int t = blockIdx.x;
 #pragma unroll 4
@@ -136,7 +184,7 @@ __global__ __launch_bounds__(1024) void moe_router_kernel(const TX* __restrict__
         if (lane == 0) z_s[o] = sum;
     }
     __syncthreads();
-    if (wave == 0) route_row<TW>(z_s, correction, idx, weight, n, top, t, lane, score_fn, renorm);
+    if (wave == 0) route_row<TW>(z_s, correction, idx, weight, n, top, t, lane, form, z_s + n);
 }
 
 template <typename TX, typename TW>
@@ -213,8 +261,17 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const TX* __restrict__ x,
 
 }  // namespace
 
+static int check_groups(const char* what, int n, int top, int groups, int keep) {
+    PULSE_REQUIRE(groups >= 0 && groups <= PULSE_WAVE, "%s: at most %d groups of outputs, got %d", what, PULSE_WAVE, groups);
+    PULSE_REQUIRE(groups <= 1 || (n % groups == 0 && keep >= 1 && keep <= groups && keep * (n / groups) >= top),
+                  "%s: %d of %d groups of %d outputs cannot give %d choices", what, keep, groups, n, top);
+    return 0;
+}
+
 extern "C" int pulse_moe_route(const float* z, const void* correction, int c_dtype, int* idx, float* weight, int tokens,
-                               int n, int top, int score_fn, int renorm, hipStream_t stream) {
+                               int n, int top, int score_fn, int renorm, int groups, int keep, float wscale,
+                               hipStream_t stream) {
+    if (check_groups("moe_route", n, top, groups, keep)) return 1;
     PULSE_REQUIRE(score_fn == 0 || score_fn == 1, "moe_route: unknown score function %d", score_fn);
     PULSE_REQUIRE(tokens >= 0 && n > 0 && top > 0 && top <= n && z && idx && weight, "moe_route: bad arguments");
     PULSE_REQUIRE(n <= PULSE_WAVE * ROUTE_PER_LANE && top <= PULSE_WAVE,
@@ -223,28 +280,29 @@ extern "C" int pulse_moe_route(const float* z, const void* correction, int c_dty
     if (tokens == 0) return 0;
     PULSE_DISPATCH_DTYPE(c_dtype, TW, hipLaunchKernelGGL(moe_route_kernel<TW>, dim3(tokens), dim3(64), 0, stream, z,
                                                          static_cast<const TW*>(correction), idx, weight, n, top,
-                                                         score_fn, renorm));
+                                                         RouteForm{score_fn, renorm, groups, keep, wscale}));
     PULSE_LAUNCH_CHECK("moe_route");
     return 0;
 }
 
 extern "C" int pulse_moe_router(const void* x, int x_dtype, const void* w, const void* correction, int w_dtype, int* idx,
                                 float* weight, int tokens, int hidden, int n, int top, int score_fn, int renorm,
-                                hipStream_t stream) {
+                                int groups, int keep, float wscale, hipStream_t stream) {
+    if (check_groups("moe_router", n, top, groups, keep)) return 1;
     PULSE_REQUIRE(score_fn == 0 || score_fn == 1, "moe_router: unknown score function %d", score_fn);
     PULSE_REQUIRE(tokens >= 0 && hidden > 0 && n > 0 && top > 0 && top <= n && x && w && idx && weight,
                   "moe_router: bad arguments");
     PULSE_REQUIRE(n <= PULSE_WAVE * ROUTE_PER_LANE && top <= PULSE_WAVE,
                   "moe_router: at most %d router outputs and %d choices", PULSE_WAVE * ROUTE_PER_LANE, PULSE_WAVE);
     PULSE_REQUIRE(pulse_dtype_ok(x_dtype) && pulse_dtype_ok(w_dtype), "moe_router: bad dtype tag");
-    const size_t lds = sizeof(float) * (static_cast<size_t>(hidden) + n);
+    const size_t lds = sizeof(float) * (static_cast<size_t>(hidden) + 2 * n);
     PULSE_REQUIRE(lds <= 60 * 1024, "moe_router: rows of %d values do not fit the workgroup's memory", hidden);
     if (tokens == 0) return 0;
     PULSE_DISPATCH_DTYPE(x_dtype, TX, PULSE_DISPATCH_DTYPE(w_dtype, TW,
         hipLaunchKernelGGL((moe_router_kernel<TX, TW>), dim3(tokens), dim3(tokens <= 256 ? 1024 : 256), lds, stream,
                            static_cast<const TX*>(x),
                            static_cast<const TW*>(w), static_cast<const TW*>(correction), idx, weight, hidden, n, top,
-                           score_fn, renorm)));
+                           RouteForm{score_fn, renorm, groups, keep, wscale})));
     PULSE_LAUNCH_CHECK("moe_router");
     return 0;
 }

@@ -5,7 +5,7 @@
 //     h = v / sqrt(mean(v^2) + eps) * w       float32, in place
 //     copy = h rounded to the activations' type (optional)
 // pulse_activation: y = act(x) element by element (1: relu squared, 2: gelu with tanh, 3: silu).
-// pulse_softcap: x <- cap * tanh(x / cap) in place on float32.
+// pulse_softcap: x <- cap * tanh(x / cap) in place on float32; pulse_scale_values: x <- s * x.
 // pulse_round_rows: a float32 matrix once more in the activations' type.
 #include "common.h"
 
@@ -85,6 +85,11 @@ __global__ void softcap_kernel(float* __restrict__ x, int64_t n, float cap) {
     if (i < n) x[i] = cap * tanhf(x[i] / cap);
 }
 
+__global__ void scale_values_kernel(float* __restrict__ x, int64_t n, float s) {
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+    if (i < n) x[i] *= s;
+}
+
 template <typename TY>
 __global__ void round_rows_kernel(const float* __restrict__ x, TY* __restrict__ y, int64_t n) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
@@ -137,6 +142,16 @@ extern "C" int pulse_softcap(float* x, int64_t n, float cap, hipStream_t stream)
     PULSE_REQUIRE(blocks < (1ll << 31), "softcap: too many elements");
     hipLaunchKernelGGL(softcap_kernel, dim3(static_cast<unsigned>(blocks)), dim3(256), 0, stream, x, n, cap);
     PULSE_LAUNCH_CHECK("softcap");
+    return 0;
+}
+
+extern "C" int pulse_scale_values(float* x, int64_t n, float s, hipStream_t stream) {
+    PULSE_REQUIRE(n >= 0 && x, "scale_values: bad arguments");
+    if (n == 0) return 0;
+    const int64_t blocks = (n + 255) / 256;
+    PULSE_REQUIRE(blocks < (1ll << 31), "scale_values: too many elements");
+    hipLaunchKernelGGL(scale_values_kernel, dim3(static_cast<unsigned>(blocks)), dim3(256), 0, stream, x, n, s);
+    PULSE_LAUNCH_CHECK("scale_values");
     return 0;
 }
 

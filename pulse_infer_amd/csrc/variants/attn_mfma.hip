@@ -84,6 +84,7 @@ struct MfmaArgs {
     int page_shift;   // log2(page_size) when it is a power of two, else -1
     float scale_log2e;
     int window;
+    int chunk;       // > 0: a token sees the keys of its own chunk of this many positions (counted from 0) only; then no window
     int split_size;  // multiple of 32
     int n_splits;
     // The longest context of the step as it is now, or null.  The launch (and a recording of it) is made for contexts
@@ -133,10 +134,25 @@ struct PulseAttnExtras {
     int v_head0;           // < 0: nq + nkv
     float temp_coef;
     int temp_every;
-    const void* sink;      // float32 [nq], or null (not taken by pulse_attn_decode)
-    float softcap;         // 0: none (not taken by pulse_attn_decode)
+    const void* sink;      // float32 [nq], or null
+    float softcap;         // 0: none
     int gate_width;        // see MfmaArgs
+    int chunk;             // > 0: keys of the token's own chunk of positions only (then window must be 0)
 };
+
+// The lowest key that a token at position `pos` sees: its window's or its chunk's first, else 0.  It never falls as
+// the position grows, which is what the walks rely on.  (Without a window pos may be -1, a column of no token.)
+__device__ __forceinline__ int low_key(int window, int chunk, int pos) {
+    if (chunk > 0) {
+        const int p = max(pos, 0);
+        return p - p % chunk;
+    }
+    return (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+}
+
+// Where the splits of an item of decoded tokens start to count: with chunks at the block of the item's lowest key, so
+// that all of them lie among the keys that are seen, else at key 0.
+__device__ __forceinline__ int splits_from(int chunk, int lo_item) { return chunk > 0 ? lo_item / 32 * 32 : 0; }
 
 // 1 / l of a column and its head's gate in one factor (a gate a channel is applied channel by channel instead).
 __device__ __forceinline__ float gated(float inv, const bf16_t* gate, int64_t gate_stride, int64_t row, int head,
@@ -331,7 +347,6 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     const int split_size = a.plan ? a.plan[1 + a.n_items * a.n_splits + item]
                            : (a.live_context && a.n_splits > 1)
                                ? live_split_size(uniform(*a.live_context), a.n_splits, a.split_size) : a.split_size;
-    const int split_begin = split * split_size;
     int split_end = 0;                              // set once hi has arrived
 
     // this lane's column: a token of the item and a head of the group
@@ -341,10 +356,11 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     const int col_row = row0 + (col_ok ? tc : 0);
     const int col_head = g * a.group + (col_ok ? hc : 0);
     const int pos_c = col_ok ? a.positions[col_row] : -1;
-    const int lo_c = (a.window > 0 && pos_c - a.window + 1 > 0) ? pos_c - a.window + 1 : 0;
+    const int lo_c = low_key(a.window, a.chunk, pos_c);
     // lowest key any column needs (the first token's window)
     const int pos_first = a.positions[row0];
-    const int lo_item = (a.window > 0 && pos_first - a.window + 1 > 0) ? pos_first - a.window + 1 : 0;
+    const int lo_item = low_key(a.window, a.chunk, pos_first);
+    const int split_begin = splits_from(a.chunk, lo_item) + split * split_size;
 
     // Q^T operand: column r, contraction elements ch*32 + kg*8 ..; loaded below, after the first keys are asked for
     bf16x8 bq[NCHUNK];
@@ -595,7 +611,7 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     // from the split alone: its loads go out before the positions have arrived.
     {
         BlockRegs xa, xb;
-        const bool early = a.window == 0;
+        const bool early = a.window == 0 && a.chunk == 0;
         int b = split_begin / BLOCK_KEYS + wave;
         // Results come back in the order asked for.  Plain: the keys first, q behind them (it is needed only when
         // the first keys are there).  FUSED: q, the token's raw key and what their preparation needs go out between
@@ -726,7 +742,7 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     const int ntok = uniform(a.items[4 * item + 1]);         // at most WAVES * per
     const int hi = uniform(a.positions[row0 + ntok - 1]);    // last key of the workgroup
     const int pos_first = uniform(a.positions[row0]);
-    const int lo_item = (a.window > 0 && pos_first - a.window + 1 > 0) ? pos_first - a.window + 1 : 0;
+    const int lo_item = low_key(a.window, a.chunk, pos_first);
     const int* bt = a.block_table + static_cast<int64_t>(uniform(a.items[4 * item + 2])) * a.bt_width;
 
     // this wavefront's tokens and this lane's column
@@ -738,11 +754,11 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     const int col_row = row0 + (col_ok ? wtok0 + tc : 0);
     const int col_head = g * a.group + (col_ok ? hc : 0);
     const int pos_c = col_ok ? a.positions[col_row] : -1;
-    const int lo_c = (a.window > 0 && pos_c - a.window + 1 > 0) ? pos_c - a.window + 1 : 0;
+    const int lo_c = low_key(a.window, a.chunk, pos_c);
     // keys this wavefront needs at all
     const int whi = uniform(wntok > 0 ? a.positions[row0 + wtok0 + wntok - 1] : -1);
     const int wpos0 = uniform(wntok > 0 ? a.positions[row0 + wtok0] : 0);
-    const int wlo = (a.window > 0 && wpos0 - a.window + 1 > 0) ? wpos0 - a.window + 1 : 0;
+    const int wlo = low_key(a.window, a.chunk, wpos0);
 
     bf16x8 bq[NCHUNK];
     {
@@ -823,7 +839,7 @@ __global__ __launch_bounds__(WAVES* PULSE_WAVE) PULSE_ATTN_WAVES_PER_EU void att
     // lowest position among this wavefront's columns: blocks wholly at or below it (and above every window's
     // start) need no mask at all
     const int wmin_pos = wpos0;
-    const int whi_lo = (a.window > 0 && whi - a.window + 1 > 0) ? whi - a.window + 1 : 0;  // highest window start
+    const int whi_lo = low_key(a.window, a.chunk, whi);  // highest window start
     const float c2 = a.scale_log2e;
 
     auto compute = [&](int b, int stage) {
@@ -1030,7 +1046,7 @@ __global__ __launch_bounds__(NW* PULSE_WAVE) PULSE_WIDE_WAVES_PER_EU void attn_p
     const int split_last = splits ? min(hi, split_begin + a.split_size - 1) : hi;
     const bool direct = !splits || hi < a.split_size;
     const int pos_first = uniform(a.positions[row0]);
-    const int lo_item = (a.window > 0 && pos_first - a.window + 1 > 0) ? pos_first - a.window + 1 : 0;
+    const int lo_item = low_key(a.window, a.chunk, pos_first);
     const int* bt = a.block_table + static_cast<int64_t>(uniform(a.items[4 * item + 2])) * a.bt_width;
 
     // this wavefront's column tiles and this lane's column in each
@@ -1049,11 +1065,11 @@ __global__ __launch_bounds__(NW* PULSE_WAVE) PULSE_WIDE_WAVES_PER_EU void attn_p
         col_ok[ct] = tc < wntok && hc < a.group;
         col_row[ct] = row0 + (col_ok[ct] ? wtok0 + tc : 0);
         pos_c[ct] = col_ok[ct] ? a.positions[col_row[ct]] : -1;
-        lo_c[ct] = (a.window > 0 && pos_c[ct] - a.window + 1 > 0) ? pos_c[ct] - a.window + 1 : 0;
+        lo_c[ct] = low_key(a.window, a.chunk, pos_c[ct]);
         t_hi[ct] = uniform(wntok > 0 ? a.positions[row0 + wtok0 + wntok - 1] : -1);
         t_pos0[ct] = uniform(wntok > 0 ? a.positions[row0 + wtok0] : 0);
-        t_lo[ct] = (a.window > 0 && t_pos0[ct] - a.window + 1 > 0) ? t_pos0[ct] - a.window + 1 : 0;
-        t_hi_lo[ct] = (a.window > 0 && t_hi[ct] - a.window + 1 > 0) ? t_hi[ct] - a.window + 1 : 0;
+        t_lo[ct] = low_key(a.window, a.chunk, t_pos0[ct]);
+        t_hi_lo[ct] = low_key(a.window, a.chunk, t_hi[ct]);
     }
     if (hc < a.group) col_head += hc;
     // keys this wavefront needs at all: from its first tile's window to its last tile's diagonal
@@ -1433,7 +1449,8 @@ __global__ __launch_bounds__(REDUCE_THREADS) void attn_mfma_reduce_kernel(const 
                                                                          const int* __restrict__ live_context,
                                                                          const int* __restrict__ plan, int n_items,
                                                                          const bf16_t* __restrict__ gate, int64_t gate_stride,
-                                                                         int gate_width, const float* __restrict__ sink) {
+                                                                         int gate_width, const float* __restrict__ sink,
+                                                                         int chunk) {
     __shared__ float s_w[MAX_SPLITS];      // hpw * n_splits <= MAX_SPLITS (hpw > 1 only with few splits)
     __shared__ float s_l[MAX_SPLITS];
     __shared__ f32x4 s_acc[REDUCE_GROUPS][REDUCE_QUADS];
@@ -1451,6 +1468,7 @@ __global__ __launch_bounds__(REDUCE_THREADS) void attn_mfma_reduce_kernel(const 
     const int head0 = blockIdx.y * hpw;
     const int pos_row = positions[row];
     const int pos_last = positions[row0 + ntok - 1];
+    const int from = chunk > 0 ? splits_from(chunk, low_key(0, chunk, positions[row0])) : 0;
     constexpr int ML_PER = MAX_SPLITS / REDUCE_THREADS;
     f32x2 ml[ML_PER];
 #pragma unroll
@@ -1484,7 +1502,7 @@ __global__ __launch_bounds__(REDUCE_THREADS) void attn_mfma_reduce_kernel(const 
                                            : f32x4{0.f, 0.f, 0.f, 0.f};
     }
     if (plan && pos_last < split_size) return;   // the item was finished by its only split
-    const int valid = min(n_splits, pos_row / split_size + 1);
+    const int valid = min(n_splits, (pos_row - from) / split_size + 1);
 #pragma unroll
     for (int j = 0; j < ML_PER; ++j) {
         const int i = threadIdx.x + j * REDUCE_THREADS;
@@ -1658,10 +1676,12 @@ struct Preparation {
 // The gate of `ex` into the kernels' arguments, checked; the other extras are pulse_attn_decode's.
 int take_gate(MfmaArgs& a, const PulseAttnExtras* ex, int nq, float scale = 0.f) {
     a.gate = nullptr; a.gate_stride = 0; a.gate_width = 0;
-    a.sink = nullptr; a.cap_in = 0.f; a.cap_out = 0.f;
+    a.sink = nullptr; a.cap_in = 0.f; a.cap_out = 0.f; a.chunk = 0;
     a.plain_norm = 0; a.v_head0 = a.nq + a.nkv; a.temp_coef = 0.f; a.temp_every = 0;
     if (!ex) return 0;
     a.sink = static_cast<const float*>(ex->sink);
+    PULSE_REQUIRE(ex->chunk >= 0 && (ex->chunk == 0 || a.window == 0), "attention: a window and chunks at once");
+    a.chunk = ex->chunk;
     PULSE_REQUIRE(ex->softcap >= 0.f, "attention: a negative score cap");
     if (ex->softcap > 0.f) {
         PULSE_REQUIRE(scale > 0.f, "attention: a score cap needs a positive scale (and a kernel that takes one)");
@@ -1692,8 +1712,11 @@ int launch_attn_mfma(const void* q, int64_t q_stride, void* out, int64_t o_strid
                   (reinterpret_cast<uintptr_t>(vcache) % 16) == 0, "attn_mfma: pointers must be 16-byte aligned");
     PULSE_REQUIRE(window >= 0 && n_splits >= 1 && split_size >= BLOCK_KEYS && split_size % BLOCK_KEYS == 0,
                   "attn_mfma: split size %d must be a positive multiple of %d", split_size, BLOCK_KEYS);
-    PULSE_REQUIRE(static_cast<int64_t>(n_splits) * split_size >= max_context,
-                  "attn_mfma: %d splits of %d keys do not cover a context of %d", n_splits, split_size, max_context);
+    // (with chunks the splits lie among an item's keys: a chunk's, those that a second token's adds, a block's rounding)
+    const int most_keys = (ex && ex->chunk > 0 && ex->chunk < max_context - 48) ? ex->chunk + 48 : max_context;
+    PULSE_REQUIRE(static_cast<int64_t>(n_splits) * split_size >= most_keys,
+                  "attn_mfma: %d splits of %d keys do not cover a context of %d", n_splits, split_size, most_keys);
+    PULSE_REQUIRE(!plan || !ex || ex->chunk == 0, "attn_mfma: a plan of uneven contexts has no chunks");
     PULSE_REQUIRE(n_splits == 1 || (part_o && part_ml && (reinterpret_cast<uintptr_t>(part_o) % 16) == 0),
                   "attn_mfma: scratch is missing or not 16-byte aligned");
     PULSE_REQUIRE(n_splits <= MAX_SPLITS, "attn_mfma: at most %d splits, got %d", MAX_SPLITS, n_splits);
@@ -1746,7 +1769,7 @@ int launch_attn_mfma(const void* q, int64_t q_stride, void* out, int64_t o_strid
         while (hpw * 2 * n_splits <= REDUCE_GROUPS && hpw * 2 <= nq) { hpw *= 2; ++hpw_log2; }
         hipLaunchKernelGGL(attn_mfma_reduce_kernel, dim3(n_items * per, (nq + hpw - 1) / hpw), dim3(REDUCE_THREADS), 0, stream,
                            part_o, part_ml, positions, items, per, a.out, o_stride, nq, n_splits, split_size, hpw_log2,
-                           a.live_context, a.plan, n_items, a.gate, a.gate_stride, a.gate_width, a.sink);
+                           a.live_context, a.plan, n_items, a.gate, a.gate_stride, a.gate_width, a.sink, a.chunk);
         PULSE_LAUNCH_CHECK("attn_mfma_reduce");
     }
     return 0;

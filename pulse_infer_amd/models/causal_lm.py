@@ -15,6 +15,7 @@ import torch
 
 from ..parts.base import (BLOCKS, EMBEDDINGS, HEADS, NORMS, POSITIONS, BuildContext, EntryMeta, ResidualStream,
                           StepContext, Workspace, joined, says)
+from ..parts.rejoin import OriginRejoin
 from ..weights.store import TensorSpec, WeightLoader
 from .spec import ModelSpec
 
@@ -33,10 +34,14 @@ def expected_tensors(spec: ModelSpec) -> Dict[str, TensorSpec]:
         out.setdefault(name, ts)
     for name, rows in spec.offsets.items():
         out[name] = TensorSpec((rows, spec.hidden_size), kind="linear", fan_in=4)
+    for name in spec.rejoins:
+        out.update(OriginRejoin.weight_specs({"hidden_size": spec.hidden_size, "name": name}))
     return out
 
 
 class CausalLM:
+    rejoins: Dict[str, OriginRejoin] = {}
+
     def __init__(self, spec: ModelSpec, source: Any, mode: str = "bfloat16", device: Any = "cuda:0",
                  strict: bool = False, options: Optional[Dict[str, Any]] = None):
         if mode not in ACT_DTYPES:
@@ -61,6 +66,7 @@ class CausalLM:
         self.final_norm = NORMS.get(spec.final_norm.kind)(spec.final_norm.params, spec.final_norm_prefix, build)
         self.head = HEADS.get(spec.head.kind)(spec.head.params, build, self.embedding)
         self.offsets = {name: loader.get(name) for name in spec.offsets}
+        self.rejoins = {name: OriginRejoin({"hidden_size": spec.hidden_size, "name": name}, build) for name in spec.rejoins}
         self.vocab_size = spec.vocab_size
         self.hidden_size = spec.hidden_size
         self._clean: Optional[bool] = None
@@ -84,7 +90,7 @@ class CausalLM:
         if self._clean is None:
             parts: List[Any] = [self.embedding, self.final_norm, self.head]
             parts += [self.blocks[run.layer] for run in self.spec.order]
-            parts += list(self.positions.values())
+            parts += list(self.positions.values()) + list(self.rejoins.values())
             self._clean = all(says(part, "records_cleanly") for part in parts)
         return self._clean
 
@@ -100,13 +106,18 @@ class CausalLM:
         h = ws.buffer("model.residual", ctx.num_tokens, self.hidden_size * self.spec.streams, torch.float32)
         self.embedding.forward(ctx.token_ids, h)
         stream = ResidualStream(h)
+        if self.rejoins:
+            OriginRejoin.keep_origin(h, ctx, self.act_dtype)
         order = self.spec.order
         for index, run in enumerate(order):
             # who reads the residual once this block is through: the block behind it (the final norm after the last
             # one gathers the wanted rows and stays a kernel of its own)
             follower = self.blocks[order[index + 1].layer] if index + 1 < len(order) else None
             stream.after_block = follower.entry_norm() if hasattr(follower, "entry_norm") else None
-            if run.offset is not None:
+            if run.rejoin is not None:
+                row = self.offsets[run.offset[0]][run.offset[1]] if run.offset is not None else None
+                self.rejoins[run.rejoin].forward(stream, ctx, row)
+            elif run.offset is not None:
                 # (a sum: it may go in while an update is still pending; what was known about the rows no longer holds)
                 from ..ops import kernels
                 kernels.residual_add_row(stream.h, self.offsets[run.offset[0]][run.offset[1]])

@@ -7,6 +7,7 @@ from __future__ import annotations
 from typing import List, Tuple
 
 from ..parts.base import BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, StepCost
+from ..parts.rejoin import OriginRejoin
 from .spec import ModelSpec
 
 
@@ -19,6 +20,9 @@ def step_cost(spec: ModelSpec, entries: List[Tuple[int, int]], wanted: int, weig
     table counts its gathered rows only; the head counts its whole matrix and the arithmetic of the wanted rows."""
     cost = EMBEDDINGS.get(spec.embedding.kind).step_cost(spec.embedding.params, entries, weight_bytes, cache_bytes)
     for run in spec.order:
+        if run.rejoin is not None:
+            cost = cost + OriginRejoin.step_cost({"hidden_size": spec.hidden_size, "name": run.rejoin}, entries, weight_bytes,
+                                                 cache_bytes)
         layer = spec.layers[run.layer]
         block = BLOCKS.get(layer.block.kind)
         mixer = MIXERS.get(layer.mixer.kind).step_cost(layer.mixer.params, entries, weight_bytes, cache_bytes)
@@ -27,6 +31,8 @@ def step_cost(spec: ModelSpec, entries: List[Tuple[int, int]], wanted: int, weig
             cost = cost + FEED_FORWARDS.get(layer.ffn.kind).step_cost(layer.ffn.params, entries, weight_bytes,
                                                                       cache_bytes)
         for place in getattr(block, "NORM_PLACES", ()):
+            if place == "ffn_norm" and layer.ffn is None:
+                continue
             norm = layer.norm(place)
             cost = cost + NORMS.get(norm.kind).step_cost(norm.params, entries, weight_bytes, cache_bytes)
     cost = cost + NORMS.get(spec.final_norm.kind).step_cost(spec.final_norm.params, [(0, wanted)], weight_bytes,

@@ -63,11 +63,14 @@ class RunSpec:
     order) of an earlier run whose cache this run reads instead of owning one.
     ``offset`` = (tensor, row): that row of a tensor listed in ``ModelSpec.offsets`` is added to the residual of every
     token right before the run (the marker of a pass over layers that run several times).
+    ``rejoin``: a tensor W listed in ``ModelSpec.rejoins``; before the run (and before its offset) the residual x becomes
+    W [x; x0], x0 the residual as the embedding left it.
     """
 
     layer: int
     cache_of: Optional[int] = None
     offset: Optional[Tuple[str, int]] = None
+    rejoin: Optional[str] = None
 
 
 @dataclass
@@ -89,6 +92,9 @@ class ModelSpec:
     streams: int = 1
     # tensors [rows, hidden_size] whose rows runs add to the residual (``RunSpec.offset``): name -> rows
     offsets: Dict[str, int] = field(default_factory=dict)
+    # tensors [hidden_size, 2 hidden_size] through which runs bring the embedding's output back into the residual
+    # (``RunSpec.rejoin``)
+    rejoins: List[str] = field(default_factory=list)
 
     def validate(self) -> None:
         if not self.layers:
@@ -104,6 +110,11 @@ class ModelSpec:
                     raise ValueError(f"order[{index}].offset names row {row} of '{name}', the model lists {self.offsets}")
                 if self.streams != 1:
                     raise ValueError("offsets are added to a residual of one stream")
+            if run.rejoin is not None:
+                if run.rejoin not in self.rejoins:
+                    raise ValueError(f"order[{index}].rejoin names '{run.rejoin}', the model lists {self.rejoins}")
+                if self.streams != 1:
+                    raise ValueError("the embedding's output is brought back into a residual of one stream")
             if run.cache_of is not None:
                 if not 0 <= run.cache_of < index:
                     raise ValueError(f"order[{index}].cache_of must name an earlier run, got {run.cache_of}")

@@ -24,20 +24,23 @@ class _Extras(ctypes.Structure):
     # as PulseAttnExtras of the kernel source
     _fields_ = [("gate", ctypes.c_void_p), ("gate_stride", ctypes.c_int64), ("plain_norm", ctypes.c_int),
                 ("v_head0", ctypes.c_int), ("temp_coef", ctypes.c_float), ("temp_every", ctypes.c_int),
-                ("sink", ctypes.c_void_p), ("softcap", ctypes.c_float), ("gate_width", ctypes.c_int)]
+                ("sink", ctypes.c_void_p), ("softcap", ctypes.c_float), ("gate_width", ctypes.c_int),
+                ("chunk", ctypes.c_int)]
 
 
 def _extras(what: str, tokens: int, nq: int, gate: Optional[torch.Tensor] = None, plain_norm: bool = False,
             v_head0: int = -1, q_temperature: Optional[Tuple[float, int]] = None, gate_width: int = 0,
-            sink: Optional[torch.Tensor] = None, softcap: float = 0.0):
+            sink: Optional[torch.Tensor] = None, softcap: float = 0.0, chunk: int = 0):
     """What the entry points take besides their lists, or a null pointer when there is none of it.  ``gate``: bfloat16
     [tokens, nq] (rows may be strided), the logits of an output gate: head h of token t leaves the kernel multiplied
     by sigmoid(gate[t, h]).  The rest is for ``attn_decode``: a norm of q and k without weights, the head number at
     which the raw values start in a row of the projection output, and a query temperature (coef, every):
     q *= 1 + coef * ln(floor((position + 1) / every) + 1).  ``gate_width`` > 0: the gate holds a logit for each of the
     first ``gate_width`` channels of every head ([tokens, nq * gate_width]).  ``sink`` float32 [nq]: exp(sink[h]) is one
-    more term of head h's softmax denominator; ``softcap`` > 0: scaled scores become cap * tanh(score / cap)."""
-    if gate is None and not plain_norm and v_head0 < 0 and q_temperature is None and sink is None and not softcap:
+    more term of head h's softmax denominator; ``softcap`` > 0: scaled scores become cap * tanh(score / cap); ``chunk`` > 0:
+    a token sees only the keys of its own chunk of that many positions, counted from 0."""
+    if (gate is None and not plain_norm and v_head0 < 0 and q_temperature is None and sink is None and not softcap
+            and not chunk):
         return None
     ex = _Extras()
     if gate is not None:
@@ -55,6 +58,8 @@ def _extras(what: str, tokens: int, nq: int, gate: Optional[torch.Tensor] = None
         ex.sink = sink.data_ptr()
     _need(softcap >= 0.0, f"{what}: a score cap must not be negative")
     ex.softcap = float(softcap)
+    _need(chunk >= 0, f"{what}: a chunk must not be negative")
+    ex.chunk = int(chunk)
     ex.plain_norm = 1 if plain_norm else 0
     ex.v_head0 = int(v_head0)
     if q_temperature is not None:
@@ -162,7 +167,7 @@ def attn_mfma(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, kca
               part_o: Optional[torch.Tensor], part_ml: Optional[torch.Tensor],
               live_context: Optional[torch.Tensor] = None, plan: Optional[torch.Tensor] = None,
               gate: Optional[torch.Tensor] = None, gate_width: int = 0, sink: Optional[torch.Tensor] = None,
-              softcap: float = 0.0) -> None:
+              softcap: float = 0.0, chunk: int = 0) -> None:
     """Attention of decoded tokens and short portions.  ``split_size`` x ``n_splits`` is what the launch is made for
     (contexts up to ``max_context``); ``live_context`` (one int32 on the device: the longest context among the step's
     entries as it is now) lets the kernel cut the keys that are there evenly into the same number of splits;
@@ -193,7 +198,8 @@ def attn_mfma(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, kca
             _ptr(vcache), _ptr(positions), _ptr(block_table), _i32(block_table.shape[1]),
             _ptr(items), _i32(n_items), _i32(tokens), _i32(nq), _i32(nkv), _i32(page_size), _i32(pages), _f32(scale),
             _i32(window), _i32(split_size), _i32(n_splits), _i32(max_context), _ptr(part_o), _ptr(part_ml),
-            _ptr(live_context), _ptr(plan), _extras("attn_mfma", tokens, nq, gate, gate_width=gate_width, sink=sink, softcap=softcap), _stream())
+            _ptr(live_context), _ptr(plan), _extras("attn_mfma", tokens, nq, gate, gate_width=gate_width, sink=sink, softcap=softcap,
+            chunk=chunk), _stream())
 
 
 PLAN_MIN_KEYS = 256      # no split of a plan is shorter (what a workgroup costs beside its walk, in keys walked)
@@ -258,6 +264,15 @@ PREFILL_SCRATCH_BYTES = 1 << 30
 TAIL_SPLIT_MIN_BLOCKS = 64     # walks from here on (4,096 keys) are worth a cut at three quarters on a full chip
 
 
+CHUNK_SLACK = 48     # keys that the splits of an item cover beside its chunk: a block's rounding, its other tokens'
+
+
+def split_span(max_context: int, chunk: int) -> int:
+    """The keys that the splits of an item of decoded tokens must cover: the context, or with chunks what an item can see
+    of it (there the splits count from the item's lowest key)."""
+    return min(max_context, chunk + CHUNK_SLACK) if chunk else max_context
+
+
 def choose_prefill_splits(entries: Sequence, portion: int, nkv: int, group: int, d: int, window: int,
                           target_groups: Optional[int] = None, min_blocks: int = 8) -> Tuple[int, int]:
     """(split_size, n_splits) for the prompt-portion kernel over these (index, entry) pairs.
@@ -312,7 +327,7 @@ def attn_prefill(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, 
                  items: torch.Tensor, scale: float, window: int, split_size: int = 0, n_splits: int = 1,
                  part_o: Optional[torch.Tensor] = None, part_ml: Optional[torch.Tensor] = None,
                  gate: Optional[torch.Tensor] = None, gate_width: int = 0, sink: Optional[torch.Tensor] = None,
-                 softcap: float = 0.0) -> None:
+                 softcap: float = 0.0, chunk: int = 0) -> None:
     """Attention for prompt portions: items of up to portion_tokens(group, d) tokens, keys shared through LDS.
     With ``n_splits > 1`` the keys are walked in splits of ``split_size`` (a multiple of 64) by workgroups of their
     own and merged by a second kernel; ``part_o`` / ``part_ml`` are float32 scratch of tokens * nq * n_splits * d
@@ -344,7 +359,8 @@ def attn_prefill(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, 
             _ptr(items), _i32(items.numel() // ITEM_INTS), _i32(tokens), _i32(nq), _i32(nkv), _i32(page_size), _i32(pages),
             _f32(scale), _i32(window), _i32(split_size if n_splits > 1 else 0), _i32(n_splits),
             _ptr(part_o if n_splits > 1 else None), _ptr(part_ml if n_splits > 1 else None),
-            _extras("attn_prefill", tokens, nq, gate, gate_width=gate_width, sink=sink, softcap=softcap), _stream())
+            _extras("attn_prefill", tokens, nq, gate, gate_width=gate_width, sink=sink, softcap=softcap,
+            chunk=chunk), _stream())
 
 
 def decode_takes(d: int, rotary_dim: int, pairing: int) -> bool:
@@ -361,11 +377,12 @@ def attn_decode(qkv: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int,
                 k_w: Optional[torch.Tensor], eps: float, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
                 rotary_dim: int, pairing: int, new_key: bool, live_context: Optional[torch.Tensor] = None,
                 plan: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, plain_norm: bool = False,
-                v_head0: int = -1, q_temperature: Optional[Tuple[float, int]] = None) -> None:
+                v_head0: int = -1, q_temperature: Optional[Tuple[float, int]] = None, sink: Optional[torch.Tensor] = None,
+                softcap: float = 0.0, chunk: int = 0) -> None:
     """Attention for decoded tokens from the raw projection output ``qkv`` [tokens, (nq + 2 nkv) d]: per-head norm
     and rotation of q and of the token's own key happen inside the kernel; with ``new_key`` key and value are also
     written to the token's page.  ``plain_norm``: the norm has no weights; ``v_head0``: the raw values start at head
-    number ``v_head0`` of a row instead of nq + nkv; ``q_temperature``, ``gate``: see ``_extras``.  Every item must hold one token; ``items`` None says that item i is token i with row
+    number ``v_head0`` of a row instead of nq + nkv; ``q_temperature``, ``gate``, ``sink``, ``softcap``, ``chunk``: see ``_extras``.  Every item must hold one token; ``items`` None says that item i is token i with row
     i of the block table (a step of decoded tokens in the order of its requests), which spares every workgroup the
     trip to memory for its item.  ``live_context``, ``plan``: as for ``attn_mfma``."""
     _gpu("attn_decode", qkv, out, kcache, vcache, positions, block_table, items, part_o, part_ml, q_w, k_w, cos, sin,
@@ -410,4 +427,5 @@ def attn_decode(qkv: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int,
             _i32(split_size), _i32(n_splits), _i32(max_context), _ptr(part_o), _ptr(part_ml), _ptr(q_w), _ptr(k_w),
             _f32(eps), _ptr(cos), _ptr(sin), _i32(rotary_dim if cos is not None else 0), _i32(pairing),
             _i32(1 if new_key else 0), _ptr(live_context), _ptr(plan),
-            _extras("attn_decode", tokens, nq, gate, plain_norm, v_head0, q_temperature), _stream())
+            _extras("attn_decode", tokens, nq, gate, plain_norm, v_head0, q_temperature, sink=sink, softcap=softcap,
+                    chunk=chunk), _stream())

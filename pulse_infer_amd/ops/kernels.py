@@ -125,6 +125,68 @@ def residual_add(h: torch.Tensor, delta: torch.Tensor, scale: float = 1.0) -> No
          _f32(scale), _stream())
 
 
+def residual_norms(h: torch.Tensor, terms: list, experts: Optional[tuple] = None, row: Optional[torch.Tensor] = None,
+                   outs: list = (), rows: Optional[torch.Tensor] = None) -> None:
+    """v = h + the terms + row + the chosen experts' weighted results; h keeps v unless rows are gathered; then the outputs.
+
+    ``terms``: at most two updates [T, H] (float32 or bfloat16; the first may be float32 [parts, T, H]); ``experts`` = (y
+    float32 [T * top, H], idx int32 [T, top], weight float32 [T, top] or None, number of experts); ``outs``: at most two
+    (out, weight or None, eps): out[r] = v / sqrt(mean(v^2) + eps) * weight, or v as it is without a weight, of row
+    ``rows[r]`` or r; the outputs' rows may be strided."""
+    what = "residual_norms"
+    _need(len(terms) <= 2 and len(outs) <= 2, f"{what}: at most two updates and two outputs")
+    _need(h.dtype == torch.float32 and h.dim() == 2 and h.is_contiguous(), f"{what}: h must be contiguous float32 [T, H]")
+    _gpu(what, h, row, rows, *terms, *[t for o in outs for t in o[:2]])
+    tokens, hidden = h.shape
+    n_out = tokens
+    if rows is not None:
+        _int_vec(f"{what}: rows", rows)
+        n_out = rows.numel()
+    parts = 1
+    for i, term in enumerate(terms):
+        if term.dim() == 3 and i == 0:
+            parts = term.shape[0]
+            _need(term.dtype == torch.float32 and term.shape[1:] == h.shape and term.is_contiguous(),
+                  f"{what}: an update in parts must be contiguous float32 [parts, T, H]")
+        else:
+            _need(term.shape == h.shape and term.is_contiguous(), f"{what}: an update must be a contiguous [{tokens}, {hidden}]")
+    a, b = (list(terms) + [None, None])[:2]
+    y = idx = weight = None
+    n_experts = top = 0
+    if experts is not None:
+        y, idx, weight, n_experts = experts
+        _gpu(what, y, idx, weight)
+        top = idx.shape[1]
+        _need(idx.dtype == torch.int32 and idx.is_contiguous() and idx.shape[0] == tokens, f"{what}: idx must be int32 [{tokens}, top]")
+        _need(y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (tokens * top, hidden),
+              f"{what}: the experts' results must be float32 [{tokens * top}, {hidden}]")
+        _need(weight is None or (weight.dtype == torch.float32 and weight.is_contiguous() and weight.shape == idx.shape),
+              f"{what}: the weights must be float32 [{tokens}, {top}]")
+    _need(row is None or (row.numel() == hidden and row.is_contiguous()), f"{what}: row must hold {hidden} values")
+    o_tag = w_tag = None
+    args = []
+    for out, w, eps in list(outs) + [(None, None, 0.0)] * (2 - len(outs)):
+        stride = hidden
+        if out is not None:
+            _need(out.dim() == 2 and tuple(out.shape) == (n_out, hidden) and out.stride(1) == 1,
+                  f"{what}: an output must be [{n_out}, {hidden}] with contiguous rows")
+            stride = out.stride(0) if n_out > 1 else hidden
+            tag = _tag(out, what)
+            _need(o_tag in (None, tag), f"{what}: both outputs must be of one storage type")
+            o_tag = tag
+        if w is not None:
+            _need(w.numel() == hidden and w.is_contiguous(), f"{what}: a weight must hold {hidden} values")
+            tag = _tag(w, what)
+            _need(w_tag in (None, tag), f"{what}: both weights must be of one storage type")
+            w_tag = tag
+        args += [_ptr(out), _i64(stride), _ptr(w), _f32(eps)]
+    tag_of = lambda t: _i32(_tag(t, what) if t is not None else 0)
+    changes = bool(terms) or experts is not None or row is not None
+    call("pulse_residual_norms", _ptr(h), _ptr(rows), _ptr(a), tag_of(a), _i32(parts), _i64(h.numel()), _ptr(b), tag_of(b),
+         _ptr(row), tag_of(row), _ptr(y), _ptr(idx), _ptr(weight), _i32(n_experts), _i32(top), *args, _i32(o_tag or 0),
+         _i32(w_tag or 0), _i32(n_out), _i32(hidden), _i32(1 if (changes and rows is None) else 0), _stream())
+
+
 def residual_add_row(h: torch.Tensor, row: torch.Tensor) -> None:
     """h[t] += row for every row t of h [T, H]; ``row`` holds H values."""
     _gpu("residual_add_row", h, row)
@@ -485,10 +547,11 @@ def attn_generic(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, 
                  vcache: torch.Tensor, positions: torch.Tensor, token_entry: torch.Tensor, block_table: torch.Tensor,
                  scale: float, window: int = 0, gate: Optional[torch.Tensor] = None, gate_width: int = 0,
                  sink: Optional[torch.Tensor] = None, softcap: float = 0.0, keep_first: int = 0,
-                 all_values: bool = False) -> None:
+                 all_values: bool = False, chunk: int = 0) -> None:
     """Paged causal attention, one wavefront per (token, head), float32 arithmetic.
 
     ``keep_first`` > 0 (with a window): the request's first ``keep_first`` keys stay visible below the window.
+    ``chunk`` > 0 (without a window): a token sees the keys of its own chunk of that many positions, counted from 0.
     ``all_values``: every query head's weights are applied to the values of all kv heads; ``out`` is then float32
     [T, nq * nkv * d] (head h, value head c at (h * nkv + c) * d).  ``out`` may be float32 in any case.
 
@@ -510,6 +573,7 @@ def attn_generic(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, 
     out_width = nq * d * (nkv if all_values else 1)
     _need(q.shape[1] >= nq * d and out.shape[1] >= out_width and out.shape[0] == tokens, "attn_generic: q/out too narrow")
     _need(keep_first >= 0, "attn_generic: negative number of kept keys")
+    _need(chunk >= 0 and not (chunk and window), "attn_generic: a window and chunks at once")
     pages, page_size = _check_cache("attn_generic", kcache, vcache, nkv, d)
     _int_vec("attn_generic: positions", positions, tokens)
     _int_vec("attn_generic: token_entry", token_entry, tokens)
@@ -532,7 +596,7 @@ def attn_generic(q: torch.Tensor, out: torch.Tensor, nq: int, nkv: int, d: int, 
          _ptr(block_table), _i32(block_table.shape[1]), _i32(tokens), _i32(nq), _i32(nkv), _i32(d), _i32(page_size),
          _i32(pages), _f32(scale), _i32(window), _ptr(gate), _i64(gate_stride),
          _i32(gate_width if gate is not None else 0), _ptr(sink), _f32(softcap), _i32(keep_first),
-         _i32(1 if all_values else 0), _i32(1 if out.dtype == torch.float32 else 0), _stream())
+         _i32(1 if all_values else 0), _i32(1 if out.dtype == torch.float32 else 0), _i32(chunk), _stream())
 
 
 def attn_wide_takes(q: torch.Tensor, kcache: torch.Tensor, d: int) -> bool:
@@ -1054,6 +1118,13 @@ def softcap(x: torch.Tensor, cap: float) -> None:
     call("pulse_softcap", _ptr(x), _i64(x.numel()), _f32(cap), _stream())
 
 
+def scale_values(x: torch.Tensor, s: float) -> None:
+    """x <- s * x, in place on float32."""
+    _gpu("scale_values", x)
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "scale_values: a contiguous float32 tensor")
+    call("pulse_scale_values", _ptr(x), _i64(x.numel()), _f32(s), _stream())
+
+
 def round_rows(x: torch.Tensor, out: torch.Tensor) -> None:
     """out = x (float32) in out's storage type."""
     _gpu("round_rows", x, out)
@@ -1471,7 +1542,8 @@ EXPERT_ACTIVATIONS = {"silu": 0, "clamped_swish": 1}
 
 
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, idx: torch.Tensor,
-              weight: torch.Tensor, score: str = "softmax", renormalize: bool = True) -> None:
+              weight: torch.Tensor, score: str = "softmax", renormalize: bool = True, groups: tuple = (0, 0),
+              weight_scale: float = 1.0) -> None:
     """Softmax over a row of router logits, the ``top`` outputs with the largest score + correction, and their scores
     divided by their sum: idx int32 [T, top], weight float32 [T, top]."""
     _gpu("moe_route", logits, correction, idx, weight)
@@ -1484,13 +1556,16 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
           f"moe_route: idx int32 and weight float32 must be [{tokens}, {top}]")
     call("pulse_moe_route", _ptr(logits), _ptr(correction), _i32(_tag(correction, "moe_route") if correction is not None else 0),
          _ptr(idx), _ptr(weight), _i32(tokens), _i32(n), _i32(top), _i32(ROUTER_SCORES[score]),
-         _i32(1 if renormalize else 0), _stream())
+         _i32(1 if renormalize else 0), _i32(groups[0]), _i32(groups[1]), _f32(weight_scale), _stream())
 
 
 def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[torch.Tensor], top: int, idx: torch.Tensor,
-               weight: torch.Tensor, score: str = "softmax", renormalize: bool = True) -> None:
+               weight: torch.Tensor, score: str = "softmax", renormalize: bool = True, groups: tuple = (0, 0),
+               weight_scale: float = 1.0) -> None:
     """``moe_route`` of the logits x w_router^T, which are formed in float32 inside the kernel.  ``score``: softmax
-    over all outputs or a sigmoid of each; ``renormalize`` False leaves the chosen scores as the weights."""
+    over all outputs or a sigmoid of each; ``renormalize`` False leaves the chosen scores as the weights.  ``groups`` =
+    (count, keep), count > 1: the outputs form ``count`` equal groups of neighbours and only those of the ``keep`` groups
+    with the largest sums of their two best choice scores can be chosen.  ``weight_scale``: a factor on the weights."""
     _need(score in ROUTER_SCORES, f"moe_router: unknown score function '{score}'")
     _gpu("moe_router", x, w_router, correction, idx, weight)
     tokens, hidden = x.shape
@@ -1505,7 +1580,8 @@ def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[tor
           f"moe_router: idx int32 and weight float32 must be [{tokens}, {top}]")
     call("pulse_moe_router", _ptr(x), _i32(_tag(x, "moe_router")), _ptr(w_router), _ptr(correction),
          _i32(_tag(w_router, "moe_router")), _ptr(idx), _ptr(weight), _i32(tokens), _i32(hidden), _i32(n), _i32(top),
-         _i32(ROUTER_SCORES[score]), _i32(1 if renormalize else 0), _stream())
+         _i32(ROUTER_SCORES[score]), _i32(1 if renormalize else 0), _i32(groups[0]), _i32(groups[1]), _f32(weight_scale),
+         _stream())
 
 
 def _in_weight(what: str, in_weight: Optional[torch.Tensor], tokens: int, top: int) -> None:
@@ -1573,12 +1649,13 @@ def moe_max_tiles(pairs: int, experts: int, tile_rows: int) -> int:
 
 
 def moe_grouped(x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, idx: torch.Tensor,
-                weight: torch.Tensor, act: torch.Tensor, y: torch.Tensor, out: torch.Tensor, scratch: torch.Tensor,
+                weight: torch.Tensor, act: torch.Tensor, y: torch.Tensor, out: Optional[torch.Tensor], scratch: torch.Tensor,
                 tile_rows: int, weight_on_input: bool = False, activation: str = "silu", limit: float = 0.0) -> None:
     """out[t] = sum_k weight[t, k] * (expert idx[t, k] of x[t], or x[t] itself for an identity expert), the experts'
     products grouped by expert on the matrix cores.  ``act`` bfloat16 [T * top, ff] and ``y`` float32 [T * top, hidden]
     are scratch; ``scratch`` int32 holds 2 * T * top + 3 * moe_max_tiles + 1 entries.  ``weight_on_input``: an expert is
-    fed weight * x and the results are added as they are; ``activation`` / ``limit`` as for ``moe_gate_up``."""
+    fed weight * x and the results are added as they are; ``activation`` / ``limit`` as for ``moe_gate_up``.  ``out`` None:
+    the sum is left to the caller, ``y`` [T * top, hidden] holds what the experts gave."""
     _need(activation in EXPERT_ACTIVATIONS, f"moe_grouped: unknown activation '{activation}'")
     _gpu("moe_grouped", x, w_gate, w_up, w_down, idx, weight, act, y, out, scratch)
     tokens, hidden = x.shape
@@ -1595,7 +1672,7 @@ def moe_grouped(x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_dow
           "moe_grouped: idx int32 and weight float32 must be [T, top]")
     _need(act.dtype == torch.bfloat16 and act.is_contiguous() and tuple(act.shape) == (pairs, ff)
           and y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (pairs, hidden)
-          and out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (tokens, hidden),
+          and (out is None or (out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (tokens, hidden))),
           "moe_grouped: act, y or out of the wrong shape or storage type")
     tiles = moe_max_tiles(pairs, experts, tile_rows)
     _need(scratch.dtype == torch.int32 and scratch.is_contiguous() and scratch.numel() >= 2 * pairs + 3 * tiles + 1,
@@ -1611,6 +1688,8 @@ def moe_grouped(x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_dow
          _i32(EXPERT_ACTIVATIONS[activation]), _f32(limit), _stream())
     call("pulse_moe_down_grouped", _ptr(act), _ptr(w_down), order, t_expert, t_row0, t_rows, count, _i32(tiles),
          _i32(tile_rows), _ptr(y), _i32(hidden), _i32(ff), _stream())
+    if out is None:
+        return
     call("pulse_moe_combine", _ptr(x), _i32(_tag(x, "moe_grouped")), _ptr(y), _ptr(idx),
          _ptr(None if weight_on_input else weight), _ptr(out),
          _i32(tokens), _i32(hidden), _i32(experts), _i32(top), _stream())

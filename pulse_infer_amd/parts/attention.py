@@ -25,6 +25,9 @@ Variations, all parameters of the part:
 * ``score_cap = c``: a scaled score s becomes c * tanh(s / c) before the softmax;
 * ``sink = True``: a learned number per query head (tensor ``sink`` [heads]) whose exponential is one more term of
   the softmax's denominator; it has no key and no value;
+* ``fixed_sink = s``: the same with the number s for every head, which is no tensor (s = 0: "one added to the sum");
+* ``chunk = n`` (in place of a window): positions fall into chunks of n, counted from 0, and a token sees the earlier tokens
+  of its own chunk only: lo = position - position mod n;
 * ``names``: the tensors' names below the part's prefix.
 """
 from __future__ import annotations
@@ -38,6 +41,15 @@ from ..ops import attention_mfma, kernels
 from ..weights.store import TensorSpec
 from .base import MIXERS, BuildContext, LazyNorm, PagedCacheView, Part, StepContext, StepCost, joined
 from .linear import Linear
+
+
+def keys_seen(start: int, count: int, window: Optional[int] = None, chunk: Optional[int] = None):
+    """(keys seen by all tokens of a portion together, keys of the context that any of them sees)"""
+    end = start + count
+    if chunk:
+        return sum(p % chunk + 1 for p in range(start, end)), end - start // chunk * chunk
+    return (sum(min(p + 1, window) if window else p + 1 for p in range(start, end)),
+            min(end, window + count - 1) if window else end)
 
 
 @MIXERS.register("attention")
@@ -79,12 +91,9 @@ class PagedAttention(Part):
         cost = super().step_cost(params, entries, weight_bytes, cache_bytes)
         nq, nkv, d, window = params["num_heads"], params["num_kv_heads"], params["head_dim"], params.get("window")
         for start, count in entries:
-            seen = 0
-            for p in range(start, start + count):
-                seen += min(p + 1, window) if window else p + 1
+            seen, kept = keys_seen(start, count, window, params.get("chunk"))
             cost.flops += 4.0 * nq * d * seen
-            context = start + count
-            cost.cache_bytes += 2.0 * nkv * d * cache_bytes * (min(context, window + count - 1) if window else context)
+            cost.cache_bytes += 2.0 * nkv * d * cache_bytes * kept
         return cost
 
     def __init__(self, params: Dict[str, Any], prefix: str, build: BuildContext):
@@ -98,6 +107,7 @@ class PagedAttention(Part):
         self.window = params.get("window")
         if self.window is not None and int(self.window) <= 0:
             raise ValueError(f"an attention window must be positive, got {self.window}")
+        self.chunk = self._read_chunk(params)
         self.qk_norm = bool(params.get("qk_norm", False))
         self.plain_norm = self.qk_norm and not params.get("qk_norm_weights", True)
         self.eps = float(params.get("qk_norm_eps", 0.0))
@@ -137,13 +147,14 @@ class PagedAttention(Part):
         weighted = self.qk_norm and not self.plain_norm
         self.q_w = load.get(names["q_norm"]) if weighted else None
         self.k_w = load.get(names["k_norm"]) if weighted else None
-        self.sink = self._load_sink(load, names["sink"]) if params.get("sink", False) else None
+        self.sink = self._load_sink(load, names["sink"]) if params.get("sink", False) else self._fixed_sink(params, build)
         self.act_dtype = build.act_dtype
         self.options = build.options
 
     gate_width = 0     # > 0: the output gate has a logit for each of that many channels of a head (a subclass's)
     score_cap = 0.0
     sink = None
+    chunk = 0
 
     def _read_score_form(self, params: Dict[str, Any]) -> None:
         self.score_cap = float(params.get("score_cap") or 0.0)
@@ -155,8 +166,22 @@ class PagedAttention(Part):
         """The sinks as float32 [heads], whatever the checkpoint's storage type."""
         return load.get(name).to(torch.float32).contiguous()
 
+    def _fixed_sink(self, params: Dict[str, Any], build: BuildContext) -> Optional[torch.Tensor]:
+        if params.get("fixed_sink") is None:
+            return None
+        return torch.full((self.nq,), float(params["fixed_sink"]), dtype=torch.float32, device=build.device)
+
+    def _read_chunk(self, params: Dict[str, Any]) -> int:
+        chunk = params.get("chunk")
+        if chunk is not None and int(chunk) <= 0:
+            raise ValueError(f"an attention chunk must be positive, got {chunk}")
+        if chunk is not None and self.window is not None:
+            raise ValueError("attention has a window or chunks, not both")
+        return int(chunk or 0)
+
     def cache_spec(self) -> PagedKVSpec:
-        return PagedKVSpec(self.nkv, self.d, int(self.window) if self.window is not None else None)
+        return PagedKVSpec(self.nkv, self.d, int(self.window) if self.window is not None else None,
+                           chunk=self.chunk or None)
 
     accepts_residual = True
     accepts_lazy_input = True   # the first product may take rows that are not normalised yet and scale its result
@@ -209,8 +234,6 @@ class PagedAttention(Part):
         token, the matrix-core kernel takes the sizes, and norm weights and rotation are of the kinds it prepares."""
         if self.options.get("decode_from_raw", True) is False or not self.uses_matrix_cores(qkv, cache):
             return False
-        if self.score_cap or self.sink is not None:
-            return False
         if "static:attention.single_tokens" not in ctx.extras:
             ctx.extras["static:attention.single_tokens"] = all(e.count == 1 for e in ctx.entries)
         if not ctx.extras["static:attention.single_tokens"]:
@@ -231,7 +254,7 @@ class PagedAttention(Part):
         if not self.uses_matrix_cores(q, cache):
             kernels.attn_generic(q, out, self.nq, self.nkv, self.d, cache.keys, cache.values, ctx.positions,
                                  ctx.token_entry, table, self.scale, window, gate=gate, gate_width=self.gate_width,
-                                 sink=self.sink, softcap=self.score_cap)
+                                 sink=self.sink, softcap=self.score_cap, chunk=self.chunk)
             return
         group = self.nq // self.nkv
         per = attention_mfma.tokens_per_item(group)
@@ -246,10 +269,11 @@ class PagedAttention(Part):
                 max((e.start + e.count for _, e in short), default=0))
         short_items, long_items, short_context = ctx.extras[key]
         if long_items is not None:
-            skey = f"static:attention.portion_splits:{portion}:{window}:{self.nkv}:{group}:{self.d}"
+            skey = f"static:attention.portion_splits:{portion}:{window or self.chunk}:{self.nkv}:{group}:{self.d}"
             if skey not in ctx.extras:
                 ctx.extras[skey] = attention_mfma.choose_prefill_splits(
-                    attention_mfma.split_entries(ctx.entries)[1], portion, self.nkv, group, self.d, window)
+                    attention_mfma.split_entries(ctx.entries)[1], portion, self.nkv, group, self.d,
+                    window or self.chunk)
             split_size, n_splits = ctx.extras[skey]
             part_o = part_ml = None
             if n_splits > 1:
@@ -258,14 +282,16 @@ class PagedAttention(Part):
                 part_ml = ctx.workspace.buffer("attention.portion_part_ml", rows, 2, torch.float32)
             attention_mfma.attn_prefill(q, out, self.nq, self.nkv, self.d, cache.keys, cache.values, ctx.positions,
                                         table, long_items, self.scale, window, split_size, n_splits, part_o, part_ml,
-                                        gate=gate, gate_width=self.gate_width, sink=self.sink, softcap=self.score_cap)
+                                        gate=gate, gate_width=self.gate_width, sink=self.sink, softcap=self.score_cap,
+                                        chunk=self.chunk)
         if short_items is not None:
             # a recorded step passes its context bucket as max_context: its splits must cover that
             max_context = ctx.max_context if long_items is None else short_context
             n_items = short_items.numel() // attention_mfma.ITEM_INTS
-            split_size, n_splits = attention_mfma.choose_splits(n_items, self.nkv, group, max_context)
+            split_size, n_splits = attention_mfma.choose_splits(
+                n_items, self.nkv, group, attention_mfma.split_span(max_context, self.chunk))
             plan = None
-            if ctx.uneven and long_items is None and not window:
+            if ctx.uneven and long_items is None and not window and not self.chunk:
                 # contexts that differ much: every request's keys cut by its own length, the workgroups in an order
                 # that starts the longest walks first (the plan is made on the device, once a step for all layers)
                 planned = min(attention_mfma.PLAN_SPLITS, 1024 // n_items)
@@ -295,10 +321,11 @@ class PagedAttention(Part):
                     self.eps, tables.cos if tables is not None else None, tables.sin if tables is not None else None,
                     tables.rotary_dim if tables is not None else 0, tables.pairing if tables is not None else 0,
                     new_key=write, live_context=ctx.live_context if plan is None else None, plan=plan, gate=gate,
-                    plain_norm=self.plain_norm, v_head0=self.v_head0, q_temperature=self.q_temperature)
+                    plain_norm=self.plain_norm, v_head0=self.v_head0, q_temperature=self.q_temperature, sink=self.sink,
+                    softcap=self.score_cap, chunk=self.chunk)
                 return
             attention_mfma.attn_mfma(q, out, self.nq, self.nkv, self.d, cache.keys, cache.values, ctx.positions,
                                      table, short_items, self.scale, window, split_size, n_splits,
                                      max_context, part_o, part_ml,
                                      live_context=ctx.live_context if plan is None else None, plan=plan, gate=gate,
-                                     gate_width=self.gate_width, sink=self.sink, softcap=self.score_cap)
+                                     gate_width=self.gate_width, sink=self.sink, softcap=self.score_cap, chunk=self.chunk)

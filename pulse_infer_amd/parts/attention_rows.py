@@ -10,7 +10,7 @@ and one for k, shared by the heads) or False; ``qk_norm_eps``; ``out_scale`` (a 
 float32 before their one rounding); ``output_gate``: "channel": the heads' outputs are multiplied element by element
 by sigmoid(Wg x), Wg [heads * value_dim, hidden] (tensor ``gate``), whose rows ride behind q, k and v in the stacked
 projection and whose sigmoid the attention kernels apply as they store; ``score_cap`` and ``sink`` as for
-``attention``; ``keep_first`` (with a window): a request's first ``keep_first`` tokens stay visible below the window,
+``attention`` (so are ``fixed_sink`` and ``chunk``); ``keep_first`` (with a window): a request's first ``keep_first`` tokens stay visible below the window,
 at their true positions; ``talk``: the heads' attention weights are mixed before they meet the values, weight_h <-
 sum_g T[h, g] weight_g with T the tensor ``talk`` [heads, heads] (a sink's share is not mixed); head h applies its
 mixed weights to the values of its own kv head.  Both run on ``pulse_attn_wide`` (bfloat16, the matrix cores) or the
@@ -20,6 +20,10 @@ float32, and ``pulse_head_mix`` forms the sums.
 Keys and values are stored with one width D = max(head_dim, value_dim) rounded up to a multiple of 16, the missing
 channels as zeros: zero key channels add nothing to a score, and zero value channels come out as zeros, which meet
 zero columns of the output weight.  The attention kernels then see ordinary heads of D channels.
+
+Where a row of the projection output already has the layout of ordinary heads (no bias, no norm, keys as wide as values, a
+width that needs no filling up), a step of decoded tokens goes through ``attention``'s kernel that prepares q and the
+tokens' own keys itself.
 
 It answers the protocol of a branch of ``side_by_side`` (``inner_width``, ``out_weight()``, ``forward_inner``).
 """
@@ -32,7 +36,7 @@ import torch
 from ..cache.manager import PagedKVSpec
 from ..ops import kernels
 from ..weights.store import TensorSpec
-from .attention import PagedAttention
+from .attention import PagedAttention, keys_seen
 from .base import MIXERS, BuildContext, PagedCacheView, Part, StepContext, StepCost, joined
 from .linear import Linear
 
@@ -85,12 +89,8 @@ class RowPreparedAttention(PagedAttention):
         first = int(params.get("keep_first", 0) or 0) if window else 0
         fan = nkv if params.get("talk", False) else 1     # every head's weights meet the values of every kv head
         for start, count in entries:
-            seen = 0
-            for p in range(start, start + count):
-                seen += min(p + 1, window + first) if window else p + 1
+            seen, kept = keys_seen(start, count, window + first if window else None, params.get("chunk"))
             cost.flops += 2.0 * nq * (d + dv * fan) * seen
-            context = start + count
-            kept = min(context, window + first + count - 1) if window else context
             cost.cache_bytes += 2.0 * nkv * stored_width(d, dv) * cache_bytes * kept
         return cost
 
@@ -107,6 +107,7 @@ class RowPreparedAttention(PagedAttention):
         self.window = params.get("window")
         if self.window is not None and int(self.window) <= 0:
             raise ValueError(f"an attention window must be positive, got {self.window}")
+        self.chunk = self._read_chunk(params)
         norm = params.get("qk_norm", False)
         if norm not in (False, None, "projection", "head"):
             raise ValueError(f"attention_rows norms q and k over the 'projection', by 'head' or not at all, got {norm!r}")
@@ -138,7 +139,7 @@ class RowPreparedAttention(PagedAttention):
                           build.mode)
         self.kv_cols = self.nq * self.qk_dim + self.nkv * (self.qk_dim + self.v_dim)   # where the gate's columns start
         self.gate_width = self.v_dim if self.channel_gate else 0
-        self.sink = self._load_sink(load, n["sink"]) if params.get("sink", False) else None
+        self.sink = self._load_sink(load, n["sink"]) if params.get("sink", False) else self._fixed_sink(params, build)
         self.talk = load.get(n["talk"]) if self.talks else None
         self.biases = tuple(load.get(n[k]) for k in ("q_bias", "k_bias", "v_bias")) if params.get("bias", False) else None
         weighted = self.row_norm or (self.head_norm and params.get("qk_norm_weights", False))
@@ -159,12 +160,18 @@ class RowPreparedAttention(PagedAttention):
         self.q_temperature = None
         self.q_w = self.k_w = None
 
-    accepts_residual = False
+        # columns of the projection output as the kernel that starts from it takes them
+        self.v_head0 = self.nq + self.nkv
+        self.raw_heads = (self.qk_dim == self.v_dim == self.d and self.biases is None and not norm and not self.channel_gate
+                          and self.out_scale == 1.0 and not (self.keep_first or self.talks))
+
+    accepts_residual = True
     accepts_lazy_input = False
     records_cleanly = True
 
     def cache_spec(self) -> PagedKVSpec:
-        return PagedKVSpec(self.nkv, self.d, int(self.window) if self.window is not None else None, self.keep_first)
+        return PagedKVSpec(self.nkv, self.d, int(self.window) if self.window is not None else None, self.keep_first,
+                           chunk=self.chunk or None)
 
     def uses_matrix_cores(self, q: torch.Tensor, cache: PagedCacheView) -> bool:
         # (kept first tokens and mixed heads are the generic kernel's)
@@ -183,6 +190,9 @@ class RowPreparedAttention(PagedAttention):
         self.qkv.forward(x, qkv, rows=rows)
         tables = ctx.position_product(self.position, self.encodings) if self.position is not None else None
         table = ctx.block_tables[cache.group]
+        if self.decodes_from_raw(ctx, cache, qkv, tables):
+            self.attend(qkv, out, ctx, cache, table, raw=(tables, write))
+            return
         q = ws.buffer("attention_rows.q", tokens, self.nq * self.d, self.act_dtype)
         kernels.qkv_rows(qkv, q, self.nq, self.nkv, self.qk_dim, self.v_dim, self.d, self.biases, self.norm_weights,
                          self.eps, tables.cos if tables is not None else None,
@@ -243,12 +253,19 @@ class RowPreparedAttention(PagedAttention):
         return self._eye
 
     def decodes_from_raw(self, ctx, cache, qkv, tables) -> bool:
+        return self.raw_heads and super().decodes_from_raw(ctx, cache, qkv, tables)
+
+    def takes_lazy_input(self, x, cache) -> bool:
         return False
 
-    def forward(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView, residual: Optional[torch.Tensor] = None,
+                next_scale: Optional[torch.Tensor] = None, next_offset: float = 0.0, leave_stats: bool = True):
         if self._o is None:
             self._o = Linear(self._o_weight, self.mode)
         ws = ctx.workspace
         inner = ws.buffer("attention_rows.inner", x.shape[0], self.inner_width, self.act_dtype)
         self.forward_inner(x, ctx, cache, inner)
-        return self._o.forward(inner, ws.buffer("attention_rows.out", x.shape[0], self.hidden, self.act_dtype))
+        result = ws.buffer("attention_rows.out", x.shape[0], self.hidden, self.act_dtype)
+        if residual is not None:
+            return self._o.add_into(inner, residual, result, ws, next_scale, next_offset, leave_stats)
+        return self._o.forward(inner, result)

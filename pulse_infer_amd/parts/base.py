@@ -277,6 +277,40 @@ class PostNormUpdate(DeferredUpdate):
         kernels.sandwich_step(h, **self.arguments())
 
 
+@dataclass
+class ExpertSum:
+    """A routed feed-forward's result that has not been formed yet: for token t the sum over k, in their order, of
+    weight[t, k] (one without weights) * y[t * top + k]; ``idx`` [T, top] names the experts (a number from ``experts`` on, or
+    a negative one, adds nothing)."""
+
+    y: torch.Tensor          # float32 [T * top, H]
+    idx: torch.Tensor        # int32 [T, top]
+    weight: Optional[torch.Tensor]
+    experts: int
+
+    def arguments(self) -> tuple:
+        return self.y, self.idx, self.weight, self.experts
+
+
+@dataclass
+class SumUpdate(DeferredUpdate):
+    """Several updates that go into the residual together: the terms (at most two, [T, H]; the first may come in parts), a
+    routed feed-forward's result, a vector for every row."""
+
+    terms: List[torch.Tensor]
+    experts: Optional[ExpertSum] = None
+    row: Optional[torch.Tensor] = None
+
+    taken_by = "takes_sum"
+
+    def experts_args(self) -> Optional[tuple]:
+        return self.experts.arguments() if self.experts is not None else None
+
+    def apply_to(self, h: torch.Tensor) -> None:
+        from ..ops import kernels
+        kernels.residual_norms(h, self.terms, experts=self.experts_args(), row=self.row)
+
+
 class ResidualStream:
     """The float32 residual ``h`` and the update that has not been added to it yet.
 
@@ -315,6 +349,29 @@ class ResidualStream:
             kernels.residual_add(self.h, pending)
             return None
         return pending
+
+    def take_sum(self) -> SumUpdate:
+        """What is pending as a ``SumUpdate`` (an empty one if nothing is); an update of another kind is done now."""
+        pending = self.pending
+        if isinstance(pending, torch.Tensor) and self.pending_scale == 1.0:
+            pending = SumUpdate([pending])
+        if not isinstance(pending, SumUpdate):
+            self.settle()
+            return SumUpdate([])
+        self.pending, self.copy = None, None
+        return pending
+
+    def normed_pair(self, norms: Tuple[Any, Any], outs: Tuple[torch.Tensor, torch.Tensor]) -> None:
+        """Two norms of the same h + what is pending: in one kernel if both say ``takes_sum``."""
+        if not all(getattr(norm, "takes_sum", False) for norm in norms):
+            self.settle()
+            for norm, out in zip(norms, outs):
+                self.normed(norm, out)
+            return
+        from ..ops import kernels
+        update = self.take_sum()
+        kernels.residual_norms(self.h, update.terms, experts=update.experts_args(), row=update.row,
+                               outs=[(out, norm.weight, norm.eps) for norm, out in zip(norms, outs)])
 
     def normed(self, norm: Any, out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         """out = norm(h + what is pending), of all rows or of the gathered ``rows``."""

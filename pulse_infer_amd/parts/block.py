@@ -11,6 +11,9 @@ updates; the feed-forward may be absent.
 sublayers read; a layer may have no feed-forward (``LayerSpec.ffn`` None), then
 h <- h + mixer(norm(h)).
 
+``parallel_pair``: h <- h + (mixer(norm_a(h)) + ffn(norm_b(h))): both sublayers read the same h, each through a norm of its
+own; the feed-forward may be absent.
+
 ``postnorm``: h <- norm_a(alpha h + ls_a * mixer(h)); h <- norm_b(alpha h + ls_b * ffn(h)): the
 sublayers read the stream itself, the norm comes after the sum, ``alpha`` weighs the
 stream in it and ``ls`` are optional factors, one a column, on a sublayer's result.
@@ -31,7 +34,7 @@ from ..models.spec import LayerSpec
 from ..weights.store import TensorSpec
 from ..ops import kernels
 from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, BuildContext, Part, PostNormUpdate, ResidualStream, StepContext,
-                   StreamUpdate, joined, says)
+                   StreamUpdate, SumUpdate, ExpertSum, joined, says)
 
 
 @BLOCKS.register("prenorm")
@@ -245,6 +248,54 @@ class ParallelBlock(PreNormBlock):
             stream.push(self.ffn.forward(x, ctx, residual=stream.h, **self._told(stream.after_block)))
         else:
             stream.push(self.ffn.forward(x, ctx))
+
+
+@BLOCKS.register("parallel_pair")
+class PairedParallelBlock(ScaledPreNormBlock):
+    """Mixer and feed-forward side by side on the same residual, each behind a norm of its own.  Block parameters:
+    ``mixer_norm`` / ``ffn_norm``: the norms' tensor prefixes below the layer's.  The feed-forward may be absent.
+
+    Both norms are one kernel, which also does the update that is still pending.  A feed-forward that says ``defers_sum``
+    leaves its result as an ``ExpertSum``; the layer's whole update then goes into the kernel of whoever reads the residual
+    next (``SumUpdate``).  A mixer that says ``accepts_residual`` may add its result itself."""
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: Any) -> None:
+        tokens, hidden = stream.h.shape
+        x = ctx.workspace.buffer("block.normed", tokens, hidden, self.act_dtype)
+        if self.ffn is None:
+            stream.normed(self.mixer_norm, x)
+        else:
+            x2 = ctx.workspace.buffer("block.normed_pair", tokens, hidden, self.act_dtype)
+            stream.normed_pair((self.mixer_norm, self.ffn_norm), (x, x2))
+        stream.stats = stream.copy = None
+        if getattr(self.mixer, "accepts_residual", False):
+            mixed = self.mixer.forward(x, ctx, cache, residual=stream.h, leave_stats=False)
+        else:
+            mixed = self.mixer.forward(x, ctx, cache)
+        terms = [mixed] if isinstance(mixed, torch.Tensor) else []
+        if self.ffn is None:
+            stream.push(SumUpdate(terms) if terms else None)
+            return
+        if not getattr(self.ffn, "defers_sum", False):
+            # (an update handed back in a workspace buffer must not wait while the next product runs)
+            stream.push(mixed)
+            stream.settle()
+            fed = self.ffn.forward(x2, ctx)
+            for update in (fed if isinstance(fed, tuple) else (fed,)):
+                if update is not None:
+                    stream.push(update)
+            return
+        experts = None
+        for update in self.ffn.forward(x2, ctx, defer=True):
+            if isinstance(update, ExpertSum):
+                experts = update
+            elif update is not None:
+                terms.append(update)
+        if len(terms) > 2:     # (the kernel takes two)
+            stream.push(SumUpdate(terms[:1]))
+            stream.settle()
+            terms = terms[1:]
+        stream.push(SumUpdate(terms, experts=experts))
 
 
 @BLOCKS.register("postnorm")

@@ -98,6 +98,7 @@ class OutputHead(Part):
         else:
             raise KeyError(f"'{params['name']}' is missing and the configuration does not tie it to the embedding")
         self.linear = Linear(weight, build.mode)
+        self.scale = float(params.get("scale", 1.0))   # logits <- scale * logits, before a cap
         cap = params.get("softcap")
         self.softcap = float(cap) if cap else 0.0   # logits <- cap * tanh(logits / cap)
         if self.softcap < 0.0:
@@ -106,6 +107,8 @@ class OutputHead(Part):
     def forward(self, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
         """out: float32 [R, vocab]."""
         self.linear.forward(x, out)
+        if self.scale != 1.0:
+            kernels.scale_values(out, self.scale)
         if self.softcap:
             kernels.softcap(out, self.softcap)
         return out

@@ -43,7 +43,7 @@ import torch
 from ..cache.manager import PagedKVSpec
 from ..ops import attention_mfma, kernels
 from ..weights.store import TensorSpec
-from .attention import PagedAttention
+from .attention import PagedAttention, keys_seen
 from .base import MIXERS, BuildContext, PagedCacheView, Part, StepContext, StepCost, joined
 from .linear import Linear
 
@@ -95,10 +95,9 @@ class LatentAttention(PagedAttention):
         stored = latent_stored_width(rank, rot)
         window = params.get("window")
         for start, count in entries:
-            seen = sum(min(p + 1, window) if window else p + 1 for p in range(start, start + count))
+            seen, kept = keys_seen(start, count, window)
             cost.flops += 2.0 * heads * (2 * rank + rot) * seen
-            context = start + count
-            cost.cache_bytes += 2.0 * stored * cache_bytes * (min(context, window + count - 1) if window else context)
+            cost.cache_bytes += 2.0 * stored * cache_bytes * kept
         return cost
 
     def __init__(self, params: Dict[str, Any], prefix: str, build: BuildContext):
@@ -173,7 +172,7 @@ class LatentAttention(PagedAttention):
         self.q_temperature = None
         self.q_w = self.k_w = None
 
-    accepts_residual = False
+    accepts_residual = True
     accepts_lazy_input = False
     records_cleanly = True
 
@@ -184,6 +183,9 @@ class LatentAttention(PagedAttention):
         return self._o_weight
 
     def decodes_from_raw(self, ctx, cache, qkv, tables) -> bool:
+        return False
+
+    def takes_lazy_input(self, x, cache) -> bool:
         return False
 
     def forward_inner(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView, out: torch.Tensor) -> None:
@@ -343,10 +345,14 @@ class LatentAttention(PagedAttention):
             for a, b in plan["spans"]:
                 kernels.latent_compact(o[a:b], w, out[a:b], self.nq, self.v_dim, self.out_scale)
 
-    def forward(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache: PagedCacheView, residual: Optional[torch.Tensor] = None,
+                next_scale: Optional[torch.Tensor] = None, next_offset: float = 0.0, leave_stats: bool = True):
         if self._o is None:
             self._o = Linear(self._o_weight, self.mode)
         ws = ctx.workspace
         inner = ws.buffer("latent.inner", x.shape[0], self.inner_width, self.act_dtype)
         self.forward_inner(x, ctx, cache, inner)
-        return self._o.forward(inner, ws.buffer("latent.out", x.shape[0], self.hidden, self.act_dtype))
+        result = ws.buffer("latent.out", x.shape[0], self.hidden, self.act_dtype)
+        if residual is not None:
+            return self._o.add_into(inner, residual, result, ws, next_scale, next_offset, leave_stats)
+        return self._o.forward(inner, result)

@@ -16,10 +16,14 @@ expert is fed weight * x, and the experts' results are added as they are); ``exp
 "clamped_swish" with ``limit``: g = min(gate x, limit), u = clamp(up x, -limit, limit), down(g * sigmoid(1.702 g) *
 (u + 1)); ``shared_gate`` (default False): the shared expert's result is multiplied by sigmoid(w_sg . x), one number a
 token, with w_sg the tensor ``shared_gate`` [1, hidden] below the shared expert's prefix (the product then goes into
-the routed float32 sum and the part hands back one update).
+the routed float32 sum and the part hands back one update); ``groups``: {"count", "keep"}: the router's outputs form
+``count`` equal groups of neighbours, a group's mark is the sum of its two largest s + correction, and only outputs of the
+``keep`` groups with the largest marks can be chosen; ``weight_scale`` (default 1): a factor on the weights, behind the
+division.
 
 The experts' weights are stacked at load time ([experts, rows, columns]).  ``forward`` returns the routed part
-(float32) and the shared expert's part as two updates that the block adds.
+(float32) and the shared expert's part as two updates that the block adds; with ``defer`` (a block that hands updates on
+to the next norm's kernel) the routed part may be an ``ExpertSum``: the experts' results, not added up yet.
 """
 from __future__ import annotations
 
@@ -29,7 +33,7 @@ import torch
 
 from ..ops import kernels
 from ..weights.store import TensorSpec
-from .base import FEED_FORWARDS, BuildContext, Part, StepContext, StepCost, joined
+from .base import FEED_FORWARDS, BuildContext, ExpertSum, Part, StepContext, StepCost, joined
 from .mlp import GatedMLP
 
 
@@ -117,6 +121,13 @@ class RoutedExperts(Part):
         if self.score not in kernels.ROUTER_SCORES:
             raise ValueError(f"a router scores by {sorted(kernels.ROUTER_SCORES)}, not '{self.score}'")
         self.renormalize = bool(params.get("renormalize", True))
+        self.weight_scale = float(params.get("weight_scale", 1.0))
+        groups = params.get("groups")
+        self.groups = (int(groups["count"]), int(groups["keep"])) if groups else (0, 0)
+        if groups:
+            count, keep = self.groups
+            if count < 1 or outputs % count or not 1 <= keep <= count or keep * (outputs // count) < self.top:
+                raise ValueError(f"{keep} of {count} groups of {outputs} router outputs cannot give {self.top} choices")
         weight_on = params.get("weight_on", "output")
         if weight_on not in ("output", "input"):
             raise ValueError(f"an expert's weight goes on its 'output' or its 'input', not '{weight_on}'")
@@ -135,16 +146,19 @@ class RoutedExperts(Part):
 
     records_cleanly = True   # choices stay on the device; the launches do not depend on them
     returns_two = True       # forward gives (routed update, shared update or None)
+    defers_sum = True        # with ``defer`` the routed update may be an ``ExpertSum``
 
-    def forward(self, x: torch.Tensor, ctx: StepContext):
+    def forward(self, x: torch.Tensor, ctx: StepContext, defer: bool = False):
         tokens = x.shape[0]
         ws = ctx.workspace
         idx = ws.buffer("moe.idx", tokens, self.top, torch.int32)
         weight = ws.buffer("moe.weight", tokens, self.top, torch.float32)
         kernels.moe_router(x, self.router, self.correction, self.top, idx, weight, score=self.score,
-                           renormalize=self.renormalize)   # logits in float32 inside
+                           renormalize=self.renormalize, groups=self.groups,
+                           weight_scale=self.weight_scale)   # logits in float32 inside
         act = ws.buffer("moe.act", tokens * self.top, self.ff, self.act_dtype)
         routed = ws.buffer("moe.out", tokens, self.hidden, torch.float32)
+        later = None
         if kernels.moe_grouped_takes(x, self.w_gate, self.w_down):
             # bfloat16: the pairs grouped by expert on the device, every expert's rows on the matrix cores; tiles of
             # 128 rows once an expert gets about that many
@@ -152,7 +166,10 @@ class RoutedExperts(Part):
             rows = kernels.MOE_TILE_ROWS[1] if pairs >= 64 * self.experts else kernels.MOE_TILE_ROWS[0]
             y = ws.buffer("moe.y", pairs, self.hidden, torch.float32)
             ints = ws.buffer("moe.ints", 2 * pairs + 3 * kernels.moe_max_tiles(pairs, self.experts, rows) + 1, 1, torch.int32)
-            kernels.moe_grouped(x, self.w_gate, self.w_up, self.w_down, idx, weight, act, y, routed, ints.view(-1), rows,
+            if defer and not self.identity and self.shared_gate is None:
+                later = ExpertSum(y, idx, None if self.weight_on_input else weight, self.experts)
+            kernels.moe_grouped(x, self.w_gate, self.w_up, self.w_down, idx, weight, act, y,
+                                routed if later is None else None, ints.view(-1), rows,
                                 weight_on_input=self.weight_on_input, activation=self.expert_activation,
                                 limit=self.limit)
         else:
@@ -163,4 +180,4 @@ class RoutedExperts(Part):
         if shared is not None and self.shared_gate is not None:
             kernels.token_gate_add(x, self.shared_gate, shared, routed)
             shared = None
-        return routed, shared
+        return (routed if later is None else later), shared

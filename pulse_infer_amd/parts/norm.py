@@ -12,7 +12,7 @@ import torch
 
 from ..ops import kernels
 from ..weights.store import TensorSpec
-from .base import NORMS, BuildContext, LazyNorm, Part, PostNormUpdate, RowStats, StreamUpdate, joined
+from .base import NORMS, BuildContext, LazyNorm, Part, PostNormUpdate, RowStats, StreamUpdate, SumUpdate, joined
 
 
 @NORMS.register("rmsnorm")
@@ -36,6 +36,10 @@ class RMSNorm(Part):
     def takes_post_norm(self) -> bool:   # ``apply`` takes a ``PostNormUpdate`` as the update and does it on the way
         return self.weight_offset == 0.0
 
+    @property
+    def takes_sum(self) -> bool:         # and a ``SumUpdate``; two such norms of one residual run as one kernel
+        return self.weight_offset == 0.0
+
     def as_step(self) -> tuple:
         """(kind, weight, bias, eps) as ``kernels.sandwich_step`` takes a norm."""
         if self.weight_offset != 0.0:
@@ -47,6 +51,10 @@ class RMSNorm(Part):
         """out = norm(h + delta_scale * delta) * w; h keeps the sum unless rows are gathered."""
         if isinstance(delta, PostNormUpdate):
             kernels.sandwich_step(h, **delta.arguments(), norm=self.as_step(), out=out, rows=rows)
+            return out
+        if isinstance(delta, SumUpdate):
+            kernels.residual_norms(h, delta.terms, experts=delta.experts_args(), row=delta.row,
+                                   outs=[(out, self.weight, self.eps)], rows=rows)
             return out
         kernels.add_rmsnorm(h, delta, self.weight, self.eps, out, rows=rows, weight_offset=self.weight_offset,
                             delta_scale=delta_scale)

@@ -59,7 +59,7 @@ def check(name, args):
             need(int(ent.tensor[:tokens].max()) < bt.tensor.shape[0] and bt.tensor.shape[1] == width, "table")
             need(int(pos.tensor[:tokens].max()) // page < width, "a position beyond the table")
     elif name == "pulse_attn_generic_ex":
-        (q, qs, out, os_, _, _, _, _, pos, ent, bt, width, tokens, nq, _, d, page, _, _, _, gate, gs, _, _, _, _, _, _,
+        (q, qs, out, os_, _, _, _, _, pos, ent, bt, width, tokens, nq, _, d, page, _, _, _, gate, gs, _, _, _, _, _, _, _,
          _) = args
         tokens, nq, d = val(tokens), val(nq), val(d)
         need(room(q) >= (tokens - 1) * val(qs) + nq * d and room(out) >= (tokens - 1) * val(os_) + nq * d, "q / out")
