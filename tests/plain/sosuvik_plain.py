@@ -119,13 +119,11 @@ def choice_scores(x, w, p: str, router: Dict[str, Any]) -> Tuple[torch.Tensor, t
     if not groups:
         return s, c, c
     t, n = c.shape
-    size = n // groups["count"]
-    allowed = torch.zeros(t, n, dtype=torch.bool)
-    for i in range(t):
-        marks = [sum(sorted(c[i, g * size:(g + 1) * size].tolist(), reverse=True)[:2]) for g in range(groups["count"])]
-        for g in sorted(range(groups["count"]), key=lambda g: (-marks[g], g))[:groups["keep"]]:
-            allowed[i, g * size:(g + 1) * size] = True
-    return s, c, c.masked_fill(~allowed, float("-inf"))
+    count, keep, size = groups["count"], groups["keep"], n // groups["count"]
+    marks = c.view(t, count, size).sort(dim=-1, descending=True).values[..., :2].sum(-1)
+    order = marks.sort(dim=-1, descending=True, stable=True).indices
+    allowed = torch.zeros(t, count, dtype=torch.bool).scatter(1, order[:, :keep], True)
+    return s, c, c.masked_fill(~allowed.repeat_interleave(size, dim=1), float("-inf"))
 
 
 def expert(h, w, p: str, limit: float) -> torch.Tensor:
@@ -137,12 +135,14 @@ def expert(h, w, p: str, limit: float) -> torch.Tensor:
 def routed_experts(x, w, p: str, m: Dict[str, Any]) -> torch.Tensor:
     router = m["router"]
     s, _, c = choice_scores(x, w, p, router)
+    chosen = c.sort(dim=-1, descending=True, stable=True).indices[:, :router["top"]]
+    weights = torch.gather(s, 1, chosen)
+    weights = weights / (weights.sum(dim=-1, keepdim=True) + 1e-20) * router.get("scale", 1.0)
     out = torch.zeros_like(x)
-    for t in range(x.shape[0]):
-        chosen = sorted(range(c.shape[1]), key=lambda e: (-c[t, e].item(), e))[:router["top"]]
-        total = sum(s[t, e] for e in chosen) + 1e-20
-        for e in chosen:
-            out[t] += s[t, e] / total * router.get("scale", 1.0) * expert(x[t:t + 1], w, f"{p}.e{e}", m["expert"]["limit"])[0]
+    for e in range(c.shape[1]):
+        token, place = (chosen == e).nonzero(as_tuple=True)
+        if token.numel():
+            out[token] += weights[token, place].view(-1, 1) * expert(x[token], w, f"{p}.e{e}", m["expert"]["limit"])
     return out
 
 
