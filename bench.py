@@ -55,14 +55,15 @@ def parse_args() -> argparse.Namespace:
     p.add_argument("--context", type=int, default=4096, help="context length the timed decode steps end at")
     p.add_argument("--model", choices=sorted(SHAPES), default="8b", help="layer sizes: Qwen3-8B (the default), 14B or 32B")
     p.add_argument("--layers", type=int, default=None, help="fewer layers than the model has, if memory or time needs it")
-    p.add_argument("--workload", choices=["decode", "serving", "long-prompt", "dirozen", "kesovik", "tipidra", "fosupel", "makezen"], default="decode",
+    p.add_argument("--workload", choices=["decode", "serving", "long-prompt", "dirozen", "kesovik", "tipidra", "fosupel", "makezen", "sosuvik"], default="decode",
                    help="decode: fixed batch at a fixed context; serving: continuous batching of requests with "
                         "seeded prompt lengths, chunked prefill mixed with decoding; long-prompt: one prompt of "
                         "--prompt-tokens tokens in portions of --chunk tokens; dirozen / kesovik: decoding and prefill of "
                         "that design beside Qwen3 layers of equal sizes, with both models' time by entry point; "
-                        "tipidra, fosupel: the same beside Kesovik and Qwen3 layers; makezen: beside Fosupel, Kesovik and Qwen3")
-    p.add_argument("--compare-layers", type=int, default=4, help="dirozen, kesovik, tipidra, fosupel, makezen: layers of the models that are compared")
-    p.add_argument("--compare-sizes", default="2k,4k,5k", help="dirozen, kesovik, tipidra, fosupel, makezen: which of the layer sizes 2k, 4k, 5k (widths) to run")
+                        "tipidra, fosupel: the same beside Kesovik and Qwen3 layers; makezen: beside Fosupel, Kesovik and Qwen3; "
+                        "sosuvik: beside Tipidra, Fosupel and Qwen3")
+    p.add_argument("--compare-layers", type=int, default=4, help="the designs' comparisons: layers of the models that are compared")
+    p.add_argument("--compare-sizes", default="2k,4k,5k", help="the designs' comparisons: which of the layer sizes 2k, 4k, 5k (widths) to run")
     p.add_argument("--prompt-tokens", type=int, default=16384, help="long-prompt: length of the prompt")
     p.add_argument("--requests", type=int, default=32, help="serving: number of requests")
     p.add_argument("--prompt-range", type=int, nargs=2, default=[128, 2048], help="serving: prompt lengths drawn from [lo, hi]")
@@ -316,6 +317,23 @@ def makezen_layers(size, layers):
     return out
 
 
+def sosuvik_layers(size, layers):
+    """Sosuvik layers at the comparison's sizes, in turn: attention in chunks of 1,024 tokens (heads as Qwen3's, a score cap,
+    a blended rotation on a whole head) and latent attention (heads as Qwen3's, a latent row of 512 values and a turned part
+    of 64), all beside routed experts: 16 in 4 groups of which 2 are kept, an eighth as wide as the dense feed-forward, 4
+    chosen a token."""
+    dim = size["dim"]
+    scaling = {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}
+    attention = {"dim": dim, "heads": size["heads"], "kv_heads": size["kv_heads"], "mask": {"size": 1024},
+                 "rot": {"base": 1e6, "dims": dim, "scaling": scaling}, "scale": dim ** -0.5, "softcap": 30.0, "vdim": dim}
+    latent = {"dim": dim, "heads": size["heads"], "kv_rank": 512, "rot": {"base": 1e6, "dims": 64}, "rot_dim": 64,
+              "scale": (dim + 64) ** -0.5, "vdim": dim}
+    routed = {"expert": {"ff": size["ff"] // 8, "limit": 7.0}, "kind": "moe",
+              "router": {"experts": 16, "groups": {"count": 4, "keep": 2}, "scale": 2.0, "top": 4}}
+    turn = [{"type": "attention", "mixer": attention, "mlp": routed}, {"type": "latent_attention", "mixer": latent, "mlp": routed}]
+    return [turn[i % len(turn)] for i in range(layers)]
+
+
 def dirozen_compare(args, design: str = "dirozen") -> int:
     """Dirozen (or, with ``design`` "kesovik", Kesovik, and so on) beside Qwen3 layers of equal sizes (random weights, ``--compare-layers`` layers, a vocabulary of
     32,000): decoding at batch 1 / 8 / 32 with contexts ending at ``--context`` and a prompt of ``--prefill-tokens``
@@ -325,7 +343,7 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
     import torch
 
     from pulse_infer_amd.config import (DirozenConfig, FosupelConfig, KesovikConfig, MakezenConfig, Qwen3Config,
-                                        TipidraConfig)
+                                        SosuvikConfig, TipidraConfig)
     from pulse_infer_amd.engine.engine import ContinuousBatchEngine
     from pulse_infer_amd.engine.runner import StepEntry
     from pulse_infer_amd.models.causal_lm import expected_tensors
@@ -355,18 +373,19 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
                  "mlp": {"ff": size["ff"], "kind": "dense"}}
         dirozen = DirozenConfig.from_dict({"architecture": "Dirozen", "vocab": vocab, "width": size["width"],
                                            "norm": {"eps": 1e-6}, "layers": [entry] * layers}, "<bench>")
-        if design in ("kesovik", "tipidra", "fosupel", "makezen"):
+        if design in ("kesovik", "tipidra", "fosupel", "makezen", "sosuvik"):
             kesovik = KesovikConfig.from_dict({
                 "architecture": "Kesovik", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                 "embedding": {"scale": 1.0}, "postln_alpha": 2.0, "logit_softcap": 30.0,
                 "layers": kesovik_layers(size, layers)}, "<bench>")
-            if design == "tipidra":
+            if design in ("tipidra", "sosuvik"):
                 tipidra = TipidraConfig.from_dict({
                     "architecture": "Tipidra", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                     "embedding": {"scale": 1.0}, "logit_softcap": 30.0, "streams": 4,
                     "layers": tipidra_layers(size, layers)}, "<bench>")
-                return {"tipidra": tipidra, "kesovik": kesovik, "qwen3": qwen}
-            if design in ("fosupel", "makezen"):
+                if design == "tipidra":
+                    return {"tipidra": tipidra, "kesovik": kesovik, "qwen3": qwen}
+            if design in ("fosupel", "makezen", "sosuvik"):
                 fosupel = FosupelConfig.from_dict({
                     "architecture": "Fosupel", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                     "residual_mult": 0.5, "logit_softcap": 30.0, "layers": fosupel_layers(size, layers)}, "<bench>")
@@ -375,6 +394,12 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
                         "architecture": "Makezen", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
                         "layers": makezen_layers(size, layers)}, "<bench>")
                     return {"makezen": makezen, "fosupel": fosupel, "kesovik": kesovik, "qwen3": qwen}
+                if design == "sosuvik":
+                    sosuvik = SosuvikConfig.from_dict({
+                        "architecture": "Sosuvik", "vocab": vocab, "width": size["width"], "norm": {"eps": 1e-6},
+                        "logit_scale": 0.5, "loop": {"start": 0, "stop": 2, "times": 1},
+                        "layers": sosuvik_layers(size, layers)}, "<bench>")
+                    return {"sosuvik": sosuvik, "tipidra": tipidra, "fosupel": fosupel, "qwen3": qwen}
                 return {"fosupel": fosupel, "kesovik": kesovik, "qwen3": qwen}
             return {"kesovik": kesovik, "qwen3": qwen}
         return {"dirozen": dirozen, "qwen3": qwen}
@@ -460,7 +485,8 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
         torch.cuda.empty_cache()
         return out
 
-    others = {"makezen": "fosupel_kesovik_and_qwen3", "tipidra": "kesovik_and_qwen3", "fosupel": "kesovik_and_qwen3"}
+    others = {"makezen": "fosupel_kesovik_and_qwen3", "tipidra": "kesovik_and_qwen3", "fosupel": "kesovik_and_qwen3",
+              "sosuvik": "tipidra_fosupel_and_qwen3"}
     record = {"metric": f"{design}_beside_{others.get(design, 'qwen3')}_layers", "unit": "tokens/s", "n_gpus": 1, "dtype": args.dtype,
               "data": "synthetic", "layers": layers, "vocab": vocab, "context": args.context, "sizes": {}}
     for name, size in DIROZEN_SIZES.items():
@@ -480,7 +506,7 @@ def dirozen_compare(args, design: str = "dirozen") -> int:
 
 def main() -> int:
     args = parse_args()
-    if args.workload in ("kesovik", "tipidra", "fosupel", "makezen"):
+    if args.workload in ("kesovik", "tipidra", "fosupel", "makezen", "sosuvik"):
         return dirozen_compare(args, args.workload)
     if args.workload == "dirozen":
         if args.gpus != 1:
