@@ -7,8 +7,8 @@ feed-forward (``mlp``, or null for none).  Every size and constant is taken from
 ``head``.
 
 The model: x = x0 = embed[token]; per layer x <- x + (mixer(norm1(x)) + ff(norm2(x))), both of the same x, with RMSNorms
-with plain weights.  Layers ``start`` .. ``stop - 1`` run ``times`` times in a row with the same weights (every pass with a
-cache of its own); right before pass t x becomes loop.in [x; x0] + loop.step[t].  logits = logit_scale * head final.norm(x).
+with plain weights.  The stretch of layers from ``start`` up to ``stop`` is gone through ``times`` times over (weights
+shared, caches not); pass t begins with x <- loop.in [x; x0] + loop.step[t].  logits = logit_scale * head final.norm(x).
 
 Mixers.  ``attention``: softmax attention with grouped key/value heads (``heads``, ``kv_heads``, ``dim``, ``vdim``), a
 rotation of the first ``rot.dims`` channels of every head in pairs (i, i + dims / 2), its frequencies blended by

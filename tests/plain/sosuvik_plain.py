@@ -17,7 +17,7 @@ DT = torch.float64
 
 
 def rms_norm(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
-    """x / sqrt(mean(x^2) + eps) * w over the last axis, eps inside the root."""
+    """x / sqrt(mean(x^2) + eps) * w over the last axis."""
     return x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + eps) * w
 
 
